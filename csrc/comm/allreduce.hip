@@ -579,7 +579,8 @@ RAGK_API void ragk_ar_destroy(void* hp) {
   if (!h) return;
   for (int p = 0; p < h->world; ++p)
     if (h->opened[p]) (void)hipIpcCloseMemHandle(h->peers.base[p]);
-  (void)hipFree(h->local);
+  // the uncached region stays allocated until the process ends: memory handed out again after an uncached
+  // allocation that kernels have read was freed has held wrong values
   if (h->host_err) (void)hipHostFree(h->host_err);
   delete h;
 }

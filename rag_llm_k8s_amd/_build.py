@@ -36,7 +36,9 @@ HIP_LIB = os.path.join(LIB_DIR, "libragk_hip.so")
 EXTRA_FLAGS = {"gemm_w4.hip": ["-mllvm", "-disable-post-ra"]}
 
 
-HIP_FLAGS = ["-O3", "--offload-arch=" + ARCH, "-fPIC", "-std=c++17", "-Wno-unused-result", "-munsafe-fp-atomics"]
+# packed fp32 ALU forms are disabled: some of them have returned wrong results on gfx950
+HIP_FLAGS = ["-O3", "--offload-arch=" + ARCH, "-fPIC", "-std=c++17", "-Wno-unused-result", "-munsafe-fp-atomics",
+             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def hip_sources():

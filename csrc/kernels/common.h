@@ -345,4 +345,29 @@ enum RagkEpilogue : int {
   EPI_GELU = 6,      // C = gelu_erf(acc)
   EPI_BIAS_GELU_TANH = 7,  // GPT-2 MLP
   EPI_ROPE_KV = 8,   // qkv projection (D = 128 heads): RoPE on q / k, k and v rows also into the paged KV cache
+  EPI_GLU_CLIP = 9,  // paired columns: clipped gated unit; the bias pointer holds fp32 {limit, alpha, shift}
 };
+
+// epilogues over packed [64 gate | 64 up] weight rows (one output column per pair)
+constexpr bool epi_pair(int e) { return e == EPI_SILU_MUL || e == EPI_GLU_CLIP; }
+
+struct GluPar { float limit, alpha, shift; };
+template <int EPI>
+__device__ __forceinline__ GluPar glu_par(const bf16_t* p) {
+  if constexpr (EPI == EPI_GLU_CLIP) {
+    const float* f = reinterpret_cast<const float*>(p);
+    return GluPar{f[0], f[1], f[2]};
+  }
+  return GluPar{0.f, 0.f, 0.f};
+}
+// gate/up pair -> output: silu(g) * u, or min(g, limit) * sigmoid(alpha g) * (clamp(u, -limit, limit) + shift)
+template <int EPI>
+__device__ __forceinline__ float glu_act(float g, float u, const GluPar& p) {
+  if constexpr (EPI == EPI_GLU_CLIP) {
+    g = fminf(g, p.limit);
+    u = fminf(fmaxf(u, -p.limit), p.limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __expf(-p.alpha * g)) * (u + p.shift);
+  } else {
+    return ragk::silu(g) * u;
+  }
+}

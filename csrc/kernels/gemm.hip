@@ -132,7 +132,8 @@ __global__ __launch_bounds__(TILE_THREADS, 2) void gemm_tile_kernel(
         sC[(wr * 64 + 16 * i + 4 * fh + r) * EPI_LD + wc * 64 + 16 * j + fr] = acc[i][j][r];
   __syncthreads();
 
-  if constexpr (EPI == EPI_SILU_MUL) {
+  if constexpr (epi_pair(EPI)) {
+    const GluPar gp = glu_par<EPI>(bias);
     // packed tile = [64 gate cols | 64 up cols] -> 64 output cols
     const int ocol0 = tn * 64;
 #pragma unroll
@@ -145,7 +146,7 @@ __global__ __launch_bounds__(TILE_THREADS, 2) void gemm_tile_kernel(
         const float* g = sC + row * EPI_LD + c8;
         const float* u = g + 64;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = silu(g[e]) * u[e];
+        for (int e = 0; e < 8; ++e) o[e] = glu_act<EPI>(g[e], u[e], gp);
         bf16_t* dst = reinterpret_cast<bf16_t*>(C) + (size_t)gr * ldc + ocol0 + c8;
         *reinterpret_cast<u32x4*>(dst) = pack8(o);
       }
@@ -210,7 +211,7 @@ __global__ __launch_bounds__(SK_WAVES * 64) void gemm_skinny_kernel(
     const bf16_t* __restrict__ X, int ldx, const bf16_t* __restrict__ W, int ldw, void* C, int ldc,
     const bf16_t* __restrict__ bias, const bf16_t* resid, int ldr, int M, int N, int K) {
   constexpr int WV = SK_WAVES;
-  constexpr bool PAIR = (EPI == EPI_SILU_MUL);
+  constexpr bool PAIR = epi_pair(EPI);
   constexpr int NACC = PAIR ? 2 : 1;
   __shared__ __attribute__((aligned(16))) f32x4 red[WV][NACC * MT][64];
 
@@ -299,7 +300,7 @@ __global__ __launch_bounds__(SK_WAVES * 64) void gemm_skinny_kernel(
       v += red[w][t][ln][r];
       if constexpr (PAIR) u += red[w][MT + t][ln][r];
     }
-    if constexpr (PAIR) v = silu(v) * u;
+    if constexpr (PAIR) v = glu_act<EPI>(v, u, glu_par<EPI>(bias));
     if constexpr (EPI == EPI_BIAS || EPI == EPI_BIAS_RESID || EPI == EPI_BIAS_GELU ||
                   EPI == EPI_BIAS_GELU_TANH)
       v += bf2f(bias[col]);
@@ -334,7 +335,7 @@ template <int MT, int NT, int EPI, bool OUT_F32>
 __global__ __launch_bounds__(SK_WAVES * 64) void gemm_gemv_kernel(
     const bf16_t* __restrict__ X, int ldx, const bf16_t* __restrict__ W, int ldw, void* C, int ldc,
     const bf16_t* __restrict__ bias, const bf16_t* resid, int ldr, int M, int N, int K) {
-  constexpr bool PAIR = (EPI == EPI_SILU_MUL);
+  constexpr bool PAIR = epi_pair(EPI);
   constexpr int NACC = PAIR ? 2 : 1;
   __shared__ __attribute__((aligned(16))) f32x4 red[SK_WAVES][NACC * NT * MT][64];
 
@@ -425,7 +426,7 @@ __global__ __launch_bounds__(SK_WAVES * 64) void gemm_gemv_kernel(
       v += red[w][j * MT + t][ln][r];
       if constexpr (PAIR) u += red[w][(NT + j) * MT + t][ln][r];
     }
-    if constexpr (PAIR) v = silu(v) * u;
+    if constexpr (PAIR) v = glu_act<EPI>(v, u, glu_par<EPI>(bias));
     if constexpr (EPI == EPI_BIAS || EPI == EPI_BIAS_RESID || EPI == EPI_BIAS_GELU || EPI == EPI_BIAS_GELU_TANH)
       v += bf2f(bias[col]);
     if constexpr (EPI == EPI_RESID || EPI == EPI_BIAS_RESID) v += bf2f(resid[(size_t)row * ldr + col]);
@@ -452,7 +453,7 @@ template <int EPI, bool F32>
 hipError_t dispatch_gemv(const void* X, int ldx, const void* W, int ldw, void* C, int ldc, const void* bias,
                          const void* resid, int ldr, int M, int N, int K, hipStream_t st) {
   const int mt = (M + 15) / 16;
-  const bool nt2 = M > 16 && N >= 32 * 512 && (EPI != EPI_SILU_MUL || N % 32 == 0);
+  const bool nt2 = M > 16 && N >= 32 * 512 && (!epi_pair(EPI) || N % 32 == 0);
 #define RAGK_GV(MTV)                                                                                         \
   case MTV:                                                                                                  \
     if (nt2 && MTV <= 2)                                                                                     \
@@ -502,7 +503,7 @@ hipError_t dispatch_skinny(const void* X, int ldx, const void* W, int ldw, void*
 
 }  // namespace
 
-// N here is the number of OUTPUT columns. For EPI_SILU_MUL the weight has 2*N rows
+// N here is the number of OUTPUT columns. For EPI_SILU_MUL / EPI_GLU_CLIP the weight has 2*N rows
 // in the packed [64 gate | 64 up] tile layout and N must be a multiple of 64.
 RAGK_API int ragk_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, const void* bias,
                        const void* resid, int ldr, int M, int N, int K, int epi, int out_f32, hipStream_t st) {
@@ -513,6 +514,11 @@ RAGK_API int ragk_gemm(const void* A, int lda, const void* B, int ldb, void* C, 
     if (N % 64 != 0 || out_f32) return (int)hipErrorInvalidValue;
     if (skinny) return (int)dispatch_skinny<EPI_SILU_MUL, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, N, K, st);
     return (int)launch_tile<EPI_SILU_MUL, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, 2 * N, K, st);
+  }
+  if (epi == EPI_GLU_CLIP) {
+    if (N % 64 != 0 || out_f32 || !bias) return (int)hipErrorInvalidValue;
+    if (skinny) return (int)dispatch_skinny<EPI_GLU_CLIP, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, N, K, st);
+    return (int)launch_tile<EPI_GLU_CLIP, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, 2 * N, K, st);
   }
   if (!skinny && N % 8 != 0) return (int)hipErrorInvalidValue;
 #define RAGK_GEMM_CASE(E)                                                                               \

@@ -150,7 +150,7 @@ __global__ __launch_bounds__(ST_THREADS, ROWS == 64 ? 2 : 1) void gemm_stream_ke
     void* C, int ldc, const bf16_t* __restrict__ bias, const bf16_t* resid, int ldr, int M, int N, int K, int S,
     float* ws, int* counters) {
   using G = StreamGeom<MT, FP8, ROWS>;
-  constexpr bool PAIR = (EPI == EPI_SILU_MUL);
+  constexpr bool PAIR = epi_pair(EPI);
   constexpr int NS = G::NS, J = G::J;
   __shared__ __attribute__((aligned(16))) char smem[NS * G::STAGE + 16];  // one object: see trap (a)
   int& s_flag = *reinterpret_cast<int*>(smem + NS * G::STAGE);
@@ -285,7 +285,7 @@ __global__ __launch_bounds__(ST_THREADS, ROWS == 64 ? 2 : 1) void gemm_stream_ke
         v *= wscale[gp];
         u *= wscale[gp + 64];
       }
-      finish(row, (gp >> 7) * 64 + (gp & 63), silu(v) * u);
+      finish(row, (gp >> 7) * 64 + (gp & 63), glu_act<EPI>(v, u, glu_par<EPI>(bias)));
     } else {
       if constexpr (FP8) v *= wscale[gp];
       finish(row, gp, v);
@@ -351,14 +351,14 @@ int g_stream_diag = 0;
 // 28672-row Llama gate/up grid (448 tiles) occupies all 256 CUs; 128 = one block per CU, 224 tiles.
 int g_stream_pair_rows = 64;
 
-inline int stream_rows(int epi) { return (epi == EPI_SILU_MUL && g_stream_pair_rows == 64) ? 64 : WROWS; }
+inline int stream_rows(int epi) { return (epi_pair(epi) && g_stream_pair_rows == 64) ? 64 : WROWS; }
 
 template <int MT, int EPI, bool F32, bool FP8>
 int launch_stream(const void* X, int ldx, const void* W, int ldw, const float* wscale, void* C, int ldc,
                   const void* bias, const void* resid, int ldr, int M, int N, int K, int S, float* ws, int* cnt,
                   hipStream_t st) {
-  const int Nrows = EPI == EPI_SILU_MUL ? 2 * N : N;
-  if constexpr (EPI == EPI_SILU_MUL) {
+  const int Nrows = epi_pair(EPI) ? 2 * N : N;
+  if constexpr (epi_pair(EPI)) {
 #define RAGK_ST_PAIR(NTV, R)                                                                                         \
   hipLaunchKernelGGL((gemm_stream_kernel<MT, EPI, F32, FP8, NTV, R>), dim3((Nrows + R - 1) / R, S), dim3(ST_THREADS), \
                      0, st, (const bf16_t*)X, ldx, W, ldw, wscale, C, ldc, (const bf16_t*)bias, (const bf16_t*)resid,  \
@@ -441,7 +441,7 @@ RAGK_API int ragk_gemm_stream_set_pair_rows(int rows) {
 }
 
 RAGK_API int ragk_gemm_stream_splits(int N, int K, int epi, int fp8) {
-  const int Nrows = epi == EPI_SILU_MUL ? 2 * N : N;
+  const int Nrows = epi_pair(epi) ? 2 * N : N;
   const int rows = stream_rows(epi);
   const int tiles = (Nrows + rows - 1) / rows;
   const int steps = K / (fp8 ? 128 : 64);
@@ -468,6 +468,11 @@ RAGK_API int ragk_gemm_stream(const void* X, int ldx, const void* W, int ldw, co
                                                             S, ws, counters, st)
                : dispatch_stream<EPI_SILU_MUL, false, false>(X, ldx, W, ldw, wscale, C, ldc, bias, resid, ldr, M, N,
                                                              K, S, ws, counters, st);
+  }
+  if (epi == EPI_GLU_CLIP) {
+    if (N % 64 || out_f32 || fp8 || !bias) return (int)hipErrorInvalidValue;
+    return dispatch_stream<EPI_GLU_CLIP, false, false>(X, ldx, W, ldw, wscale, C, ldc, bias, resid, ldr, M, N, K, S, ws,
+                                                       counters, st);
   }
 #define RAGK_ST_CASE(E)                                                                                             \
   case E:                                                                                                           \

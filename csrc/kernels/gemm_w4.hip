@@ -161,7 +161,7 @@ constexpr bool epi_bias(int e) {
 template <int EPI, bool OUT_F32>
 constexpr int w4_epi_vmem() {
   if constexpr (EPI == EPI_ROPE_KV) return 63;    // loads + stores over the counter's range: the bound clamps
-  if constexpr (EPI == EPI_SILU_MUL) return 16;  // 8 rows x 2 pairs of 16-B stores
+  if constexpr (epi_pair(EPI)) return 16;  // 8 rows x 2 pairs of 16-B stores
   if constexpr (OUT_F32) return 64 + (epi_res(EPI) ? 64 : 0) + (epi_bias(EPI) ? 8 : 0);
   return 32 + (epi_res(EPI) ? 32 : 0) + (epi_bias(EPI) ? 4 : 0);
 }
@@ -189,7 +189,8 @@ __device__ __forceinline__ void w4_epilogue_full_bf16(const f32x4 (&acc)[8][8], 
                                                       const bf16_t* __restrict__ bias, const bf16_t* resid, int ldr) {
   const int row0 = m0 + wr * 128 + fr;
   bf16_t* Cb = reinterpret_cast<bf16_t*>(C);
-  if constexpr (EPI == EPI_SILU_MUL) {
+  if constexpr (epi_pair(EPI)) {
+    const GluPar gp = glu_par<EPI>(bias);
     const int colw = (n0 >> 1) + wc * 64 + 8 * fh;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -198,8 +199,8 @@ __device__ __forceinline__ void w4_epilogue_full_bf16(const f32x4 (&acc)[8][8], 
         float o[8];
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
-          o[k] = silu(acc[i][2 * p][k]) * acc[i][2 * p + 4][k];
-          o[4 + k] = silu(acc[i][2 * p + 1][k]) * acc[i][2 * p + 5][k];
+          o[k] = glu_act<EPI>(acc[i][2 * p][k], acc[i][2 * p + 4][k], gp);
+          o[4 + k] = glu_act<EPI>(acc[i][2 * p + 1][k], acc[i][2 * p + 5][k], gp);
         }
         *reinterpret_cast<u32x4*>(Cb + (size_t)(row0 + 16 * i) * ldc + colw + 32 * p) = pack8(o);
         // one 8-column group at a time: interleaving all 16 groups' VALU raised the register peak past
@@ -345,7 +346,8 @@ __device__ __forceinline__ void w4_epilogue_reg(const f32x4 (&acc)[8][8], int wr
                                                 int n0, void* C, int ldc, const bf16_t* __restrict__ bias,
                                                 const bf16_t* resid, int ldr, int M, int Nout) {
   const int row0 = m0 + wr * 128 + fr;
-  if constexpr (EPI == EPI_SILU_MUL) {
+  if constexpr (epi_pair(EPI)) {
+    const GluPar gp = glu_par<EPI>(bias);
     const int colw = (n0 >> 1) + wc * 64;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -356,7 +358,7 @@ __device__ __forceinline__ void w4_epilogue_reg(const f32x4 (&acc)[8][8], int wr
         if (FULL || (gr < M && gc < Nout)) {
           float o[4];
 #pragma unroll
-          for (int k = 0; k < 4; ++k) o[k] = silu(acc[i][j][k]) * acc[i][j + 4][k];
+          for (int k = 0; k < 4; ++k) o[k] = glu_act<EPI>(acc[i][j][k], acc[i][j + 4][k], gp);
           *reinterpret_cast<uint2*>(reinterpret_cast<bf16_t*>(C) + (size_t)gr * ldc + gc) =
               make_uint2(pk2bf(o[0], o[1]), pk2bf(o[2], o[3]));
         }
@@ -566,7 +568,7 @@ __global__ __launch_bounds__(W4_THREADS, 1) void gemm_w4_kernel(const bf16_t* __
   const int nwg = tiles_m * tiles_n;
   const int nwt = KSPLIT ? nwg * nsplit : nwg;  // work items
   const int nk = K / WBK;
-  const int Nout = EPI == EPI_SILU_MUL ? N / 2 : N;
+  const int Nout = epi_pair(EPI) ? N / 2 : N;
   // byte offsets are 32-bit: the launcher guarantees rows * ld * 2 < 2^31 for both operands
   const i32x4 srd_a = make_srd(A, (unsigned)M * (unsigned)lda * 2u);
   const i32x4 srd_b = make_srd(B, (unsigned)N * (unsigned)ldb * 2u);
@@ -579,7 +581,7 @@ __global__ __launch_bounds__(W4_THREADS, 1) void gemm_w4_kernel(const bf16_t* __
   // residual epilogues the allocator spilled them to scratch straight after the asm read issued, i.e.
   // before the data landed (tools/isa_lds_hazard.py checks every instantiation for that). Those read
   // them after the epilogue instead.
-  constexpr bool LATE_F0 = !(EPI == EPI_NONE || EPI == EPI_SILU_MUL || (EPI == EPI_RESID && !OUT_F32));
+  constexpr bool LATE_F0 = !(EPI == EPI_NONE || epi_pair(EPI) || (EPI == EPI_RESID && !OUT_F32));
   static_assert(EPI != EPI_ROPE_KV || (!OUT_F32 && !KSPLIT), "rope epilogue: bf16 output, no split-K");
 
   int tile = blockIdx.x;
@@ -729,12 +731,16 @@ RAGK_API int ragk_gemm_w4(const void* A, int lda, const void* B, int ldb, void* 
                           const void* resid, int ldr, int M, int N, int K, int epi, int out_f32, hipStream_t st) {
   if (M <= 0 || N <= 0 || K <= 0) return 0;
   if (K % WBK != 0 || K / WBK < W4_MIN_KT) return (int)hipErrorInvalidValue;
-  const long long rows_b = (epi == EPI_SILU_MUL) ? 2LL * N : (long long)N;
+  const long long rows_b = epi_pair(epi) ? 2LL * N : (long long)N;
   if ((long long)M * lda * 2 >= (1LL << 31) || rows_b * ldb * 2 >= (1LL << 31))
     return (int)hipErrorInvalidValue;  // 32-bit buffer offsets
   if (epi == EPI_SILU_MUL) {
     if (N % 128 != 0 || out_f32) return (int)hipErrorInvalidValue;
     return launch_w4<EPI_SILU_MUL, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, 2 * N, K, st);
+  }
+  if (epi == EPI_GLU_CLIP) {
+    if (N % 128 != 0 || out_f32 || !bias) return (int)hipErrorInvalidValue;
+    return launch_w4<EPI_GLU_CLIP, false>(A, lda, B, ldb, C, ldc, bias, resid, ldr, M, 2 * N, K, st);
   }
   if (N % 8 != 0) return (int)hipErrorInvalidValue;
 #define RAGK_W4_CASE(E) \

@@ -41,17 +41,23 @@ HIP_FLAGS = ["-O3", "--offload-arch=" + ARCH, "-fPIC", "-std=c++17", "-Wno-unuse
              "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
-def hip_sources():
+def hip_sources(only=None):
+    """(sources, headers) of the kernel library; `only`: base names of the sources to keep."""
     kdir = os.path.join(ROOT, "csrc", "kernels")
     cdir = os.path.join(ROOT, "csrc", "comm")
     srcs = sorted(glob.glob(os.path.join(kdir, "*.hip")) + glob.glob(os.path.join(cdir, "*.hip")))
+    if only is not None:
+        missing = set(only) - {os.path.basename(s) for s in srcs}
+        if srcs and missing:
+            raise FileNotFoundError("no kernel source %s" % ", ".join(sorted(missing)))
+        srcs = [s for s in srcs if os.path.basename(s) in only]
     headers = sorted(glob.glob(os.path.join(kdir, "*.h")) + glob.glob(os.path.join(cdir, "*.h")))
     return srcs, headers
 
 
-def source_hash():
-    """Content hash of every kernel source and header plus the compile flags (no mtimes)."""
-    srcs, headers = hip_sources()
+def source_hash(only=None):
+    """Content hash of every kernel source (of `only`) and header plus the compile flags (no mtimes)."""
+    srcs, headers = hip_sources(only)
     h = hashlib.sha256()
     h.update(repr((HIP_FLAGS, sorted(EXTRA_FLAGS.items()))).encode())
     for f in srcs + headers:
@@ -99,22 +105,53 @@ def check_lds_waits(objs, jobs=4):
             "%s: %s at %#x" % (os.path.basename(o), k, h[0][0]) for o, b in bad for k, h in b[:2]))
 
 
-def build_hip(verbose=False, jobs=None):
-    os.makedirs(OBJ_DIR, exist_ok=True)
+def partial_lib(name):
+    """Path of a library with only the kernels of one model family (_lib.ensure_kernels)."""
+    return os.path.join(LIB_DIR, "libragk_hip_%s.so" % name)
+
+
+def build_partial(name, only, verbose=False):
+    """Compile just the kernel sources one model family needs; one builder at a time."""
+    import fcntl
+
+    os.makedirs(LIB_DIR, exist_ok=True)
+    with open(os.path.join(LIB_DIR, ".build_%s.lock" % name), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        return build_hip(verbose=verbose, only=tuple(only), target=partial_lib(name),
+                         obj_dir=os.path.join(ROOT, "build", "obj_" + name))
+
+
+def _stamp_file(target):
+    """Content hash of what `target` was built from, beside it: it travels with the library where the object
+    files do not."""
+    return target + ".stamp"
+
+
+def _is_current(target, stamp):
+    p = _stamp_file(target)
+    return os.path.exists(target) and os.path.exists(p) and open(p).read().strip() == stamp
+
+
+def build_hip(verbose=False, jobs=None, only=None, target=None, obj_dir=None, force=False):
+    """Build the kernel library; nothing is compiled when `target` matches the sources, unless `force`."""
+    target, obj_dir = target or HIP_LIB, obj_dir or OBJ_DIR
+    os.makedirs(obj_dir, exist_ok=True)
     os.makedirs(LIB_DIR, exist_ok=True)
     kdir = os.path.join(ROOT, "csrc", "kernels")
-    srcs, headers = hip_sources()
+    srcs, headers = hip_sources(only)
     flags = HIP_FLAGS + ["-I" + kdir]
-    stamp = source_hash()
-    stamp_txt = os.path.join(OBJ_DIR, "ragk_stamp.txt")
-    prev = open(stamp_txt).read().strip() if os.path.exists(stamp_txt) else None
+    stamp = source_hash(only)
+    if not force and _is_current(target, stamp):
+        return target
+    stamp_txt = os.path.join(obj_dir, "ragk_stamp.txt")
+    prev = open(stamp_txt).read().strip() if os.path.exists(stamp_txt) and not force else None
     objs, todo = [], []
     for s in srcs:
-        o = os.path.join(OBJ_DIR, os.path.basename(s) + ".o")
+        o = os.path.join(obj_dir, os.path.basename(s) + ".o")
         objs.append(o)
         if prev != stamp or _newer([s] + headers + [os.path.abspath(__file__)], o):
             todo.append((s, o))
-    stamp_src = os.path.join(OBJ_DIR, "ragk_stamp.cpp")
+    stamp_src = os.path.join(obj_dir, "ragk_stamp.cpp")
     stamp_obj = stamp_src + ".o"
     if prev != stamp or not os.path.exists(stamp_obj):
         with open(stamp_src, "w") as f:
@@ -132,11 +169,13 @@ def build_hip(verbose=False, jobs=None):
                 print(out)
     if todo:
         check_lds_waits([o for _, o in todo], jobs)
-    if todo or prev != stamp or _newer(objs, HIP_LIB):
-        _run([HIPCC, "-shared", "-fPIC", "--offload-arch=" + ARCH] + objs + ["-o", HIP_LIB])
+    if todo or prev != stamp or _newer(objs, target):
+        _run([HIPCC, "-shared", "-fPIC", "--offload-arch=" + ARCH] + objs + ["-o", target])
         with open(stamp_txt, "w") as f:
             f.write(stamp + "\n")
-    return HIP_LIB
+    with open(_stamp_file(target), "w") as f:
+        f.write(stamp + "\n")
+    return target
 
 
 def runtime_ext_path():
@@ -167,7 +206,7 @@ def runtime_source_hash():
     return h.hexdigest()[:32]
 
 
-def build_runtime(verbose=False):
+def build_runtime(verbose=False, force=False):
     import pybind11
 
     os.makedirs(LIB_DIR, exist_ok=True)
@@ -179,8 +218,10 @@ def build_runtime(verbose=False):
     os.makedirs(OBJ_DIR, exist_ok=True)
     inc = ["-I" + pybind11.get_include(), "-I" + sysconfig.get_paths()["include"], "-I" + rdir]
     stamp = runtime_source_hash()
+    if not force and _is_current(target, stamp):
+        return target
     stamp_txt = os.path.join(OBJ_DIR, "rt_stamp.txt")
-    prev = open(stamp_txt).read().strip() if os.path.exists(stamp_txt) else None
+    prev = open(stamp_txt).read().strip() if os.path.exists(stamp_txt) and not force else None
     flags = RT_FLAGS + ['-DRAGK_RT_STAMP="%s"' % stamp]
     objs, todo = [], []
     for s in srcs:
@@ -197,11 +238,13 @@ def build_runtime(verbose=False):
         _run(["g++", "-shared", "-fPIC"] + objs + ["-o", target])
         with open(stamp_txt, "w") as f:
             f.write(stamp + "\n")
+    with open(_stamp_file(target), "w") as f:
+        f.write(stamp + "\n")
     return target
 
 
-def build_all(verbose=False):
-    paths = [build_hip(verbose=verbose), build_runtime(verbose=verbose)]
+def build_all(verbose=False, force=False):
+    paths = [build_hip(verbose=verbose, force=force), build_runtime(verbose=verbose, force=force)]
     return [p for p in paths if p]
 
 

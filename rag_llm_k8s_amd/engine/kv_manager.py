@@ -55,6 +55,71 @@ class PyBlockManager:
             self._free.extend(reversed(t))
 
 
+class StateSlots:
+    """Recurrent-state slots: one per live sequence, whatever its length. Slot 0 is scratch (padded rows of a
+    captured decode graph). A slot is not cleared when it changes hands: a sequence's first tokens start
+    from zero state inside the kernels, which know them by their position."""
+
+    def __init__(self, num_slots: int):
+        if num_slots < 2:
+            raise ValueError("need at least 2 state slots")
+        self.num_slots = num_slots
+        self._free = list(range(num_slots - 1, 0, -1))
+        self.owner = {}
+
+    def available(self) -> int:
+        return len(self._free)
+
+    def ensure(self, seq_id) -> int:
+        if seq_id not in self.owner:
+            if not self._free:
+                raise MemoryError("recurrent-state slots exhausted")
+            self.owner[seq_id] = self._free.pop()
+        return self.owner[seq_id]
+
+    def slot(self, seq_id) -> int:
+        return self.owner[seq_id]
+
+    def free(self, seq_id):
+        s = self.owner.pop(seq_id, None)
+        if s is not None:
+            self._free.append(s)
+
+
+class SequenceCache:
+    """What one live sequence holds: its K/V blocks and, for recurrent models, its state slot."""
+
+    def __init__(self, blocks, slots=None):
+        self.blocks, self.slots = blocks, slots
+
+    def can_allocate(self, seq_id, n_tokens) -> bool:
+        if self.slots is not None and seq_id not in self.slots.owner and not self.slots.available():
+            return False
+        return self.blocks.can_allocate(seq_id, n_tokens)
+
+    def ensure(self, seq_id, n_tokens):
+        if self.slots is not None:
+            self.slots.ensure(seq_id)
+        return self.blocks.ensure(seq_id, n_tokens)
+
+    def state(self, seq_id) -> int:
+        return 0 if self.slots is None else self.slots.slot(seq_id)
+
+    def table(self, seq_id):
+        return self.blocks.table(seq_id)
+
+    def slot(self, seq_id, pos) -> int:
+        return self.blocks.slot(seq_id, pos)
+
+    def free_blocks(self) -> int:
+        return self.blocks.free_blocks()
+
+    def free(self, seq_id):
+        if self.slots is not None:
+            self.slots.free(seq_id)
+        self.blocks.free(seq_id)
+
+
 def make_block_manager(num_blocks: int):
     try:
         from ..runtime import native_rt

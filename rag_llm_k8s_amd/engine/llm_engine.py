@@ -31,10 +31,10 @@ from typing import List, Optional
 import numpy as np
 import torch
 
-from ..models.llama import StepInput
+from ..models.base import StepInput
 from ..ops.backend import AttnMeta
 from ..utils import faults
-from .kv_manager import BLOCK, make_block_manager
+from .kv_manager import BLOCK, SequenceCache, StateSlots, make_block_manager
 
 # decode batches up to this size split each row's top-k over ~31 chunks of ~4k logits (topk_wave_kernel,
 # threshold-filtered lane networks, merged by the sampler's lane network); larger batches use 7
@@ -108,9 +108,14 @@ class LLMEngine:
         self.mixed_prefill_tokens = int(mixed_prefill_tokens or 0)
         self.max_model_len = max_model_len
         self.eos = set(int(e) for e in eos_ids)
-        self.bm = make_block_manager(num_blocks)
+        # per-sequence memory: paged K/V blocks, plus one state slot when the model carries recurrent state
+        self.recurrent = bool(model.recurrent)
+        slots = StateSlots(max_batch + 1) if self.recurrent else None
+        self.bm = SequenceCache(make_block_manager(num_blocks), slots)
         self.max_blocks = -(-max_model_len // BLOCK)
         model.allocate_kv_cache(num_blocks)
+        if slots is not None:
+            model.allocate_state(slots.num_slots)
         self.waiting = deque()
         self.running: List[Sequence] = []
         self.lock = threading.Lock()
@@ -256,10 +261,13 @@ class LLMEngine:
             self.comm.check()
         return fin
 
-    def _step(self):
+    def _begin_staging(self):
         self._pin_idx ^= 1
         self._pin = self._pins[self._pin_idx]
         self._pin_off = 0
+
+    def _step(self):
+        self._begin_staging()
         fin = []
         if self._aborts:
             fin += self._drain()
@@ -484,9 +492,94 @@ class LLMEngine:
         return gv.permute(1, 0, 2).reshape(B, self.tp_size * K).contiguous(), \
             gi.permute(1, 0, 2).reshape(B, self.tp_size * K).contiguous()
 
+    # ------------------------------------------------------------------ given tokens
+    def open_sequence(self) -> Sequence:
+        """A sequence that is fed given tokens (feed) instead of being sampled; close_sequence ends it."""
+        s = Sequence([], SamplingParams(ignore_eos=True, do_sample=False), 0)
+        s.status = RUNNING
+        return s
+
+    def close_sequence(self, s: Sequence):
+        s.status, s.finish_reason = FINISHED, "closed"
+        self.bm.free(s.id)
+
+    def feed(self, entries):
+        """Run given next tokens of several sequences as one batch through the generation path's own steps:
+        entries = [(sequence, tokens, wanted places among them)] -> fp32 logits [total wanted, vocab] on the
+        host. One further token each is a decode step (the captured graph of its batch bucket), anything
+        else a packed prefill step, cut to the step budget like any prompt."""
+        if self.has_work():
+            raise RuntimeError("feed() and queued requests do not mix")
+        for s, toks, _ in entries:
+            if s.length + len(toks) > self.max_model_len:
+                raise ValueError("sequence of %d tokens exceeds max_model_len %d" % (s.length + len(toks),
+                                                                                     self.max_model_len))
+            if not self.bm.can_allocate(s.id, s.length + len(toks)):
+                raise MemoryError("cache exhausted")
+            self.bm.ensure(s.id, s.length + len(toks))
+            s.prompt.extend(int(t) for t in toks)
+            s.prompt_np = np.asarray(s.prompt, dtype=np.int32)
+        got = {}
+        decode = all(len(t) == 1 and s.computed > 0 for s, t, _ in entries)
+        step = self.max_batch if decode else None
+        groups = [entries[i:i + step] for i in range(0, len(entries), step)] if decode else [entries]
+        for g in groups:
+            self._begin_staging()
+            if decode:
+                lg = self._feed_decode([s for s, _, _ in g])
+                for i, (s, _, want) in enumerate(g):
+                    if len(want):
+                        got[s.id, 0] = lg[i]
+            else:
+                self._feed_prefill(g, got)
+        for s, _, _ in entries:
+            s.computed = s.length
+        V = self.model.w.vocab_valid
+        rows = [got[s.id, int(k)][:V] for s, _, want in entries for k in want]
+        return torch.stack(rows).float().cpu() if rows else torch.empty(0, V)
+
+    def _feed_decode(self, seqs):
+        n = len(seqs)
+        if not self.is_cuda:
+            return self.model.forward(self._decode_input_cpu(self._decode_inputs_host(seqs, n), n))
+        B = self._bucket(n)
+        e = self._decode_graph(B)
+        host = np.concatenate([self._decode_inputs_host(seqs, B), self._sampling_host(seqs, pad_to=B),
+                               np.full(B, -1, dtype=np.int32)])
+        e["packed"].copy_(self._h2d_i32(host), non_blocking=True)
+        if e["graph"] is not None:
+            e["graph"].replay()
+        else:
+            e["run"]()
+        return e["logits"][:n].float().cpu()
+
+    def _feed_prefill(self, entries, got):
+        queue = deque((s, s.computed, len(t), 0, set(int(k) for k in want)) for s, t, want in entries)
+        while queue:
+            chunks, wanted, budget, row = [], [], self.max_prefill_tokens, 0
+            while queue and budget > 0 and len(chunks) < self.max_batch:
+                s, start, n, off, want = queue.popleft()
+                k = min(n, budget)
+                chunks.append((s, start, k))
+                wanted += [(row + i, (s.id, off + i)) for i in range(k) if off + i in want]
+                row, budget = row + k, budget - k
+                if k < n:
+                    queue.appendleft((s, start + k, n - k, off + k, want))
+            self._begin_staging()
+            inp, _, _ = self._prefill_input(chunks, [r for r, _ in wanted])
+            if not wanted:
+                self.model.hidden_states(inp)
+                if self.is_cuda:
+                    torch.cuda.current_stream(self.device).synchronize()
+                continue
+            lg = self.model.forward(inp).float().cpu()
+            for (_, key), x in zip(wanted, lg):
+                got[key] = x
+
     # ------------------------------------------------------------------ prefill
-    def _prefill_input(self, chunks):
+    def _prefill_input(self, chunks, rows=None):
         """Packed StepInput for prefill chunks [(seq, start, n)] + the sequences whose prompt ends here.
+        `rows`: packed rows that need logits instead of the prompts' last ones.
         Built with numpy slices (a 32k-token step took ~20 ms of per-token Python before)."""
         ids, pos, slots, cu, kvl, qlens, out_rows, out_seqs = [], [], [], [0], [], [], [], []
         bts = np.zeros((len(chunks), self.max_blocks), dtype=np.int32)
@@ -507,13 +600,12 @@ class LLMEngine:
             if start + n == len(s.prompt) or (start + n == s.length and start >= len(s.prompt)):
                 out_rows.append(cu[-1] - 1)
                 out_seqs.append(s)
-        from ..ops.native import build_prefill_tiles
-
-        m = self.model
-        tiles = build_prefill_tiles(qlens, m.Hq, m.Hkv)
+        tiles, qtiles = self.model.prefill_work(qlens, self.device)
         meta = AttnMeta("prefill", self._h2d_i32(kvl), self._h2d_i32(bts), cu_q=self._h2d_i32(cu),
-                        tiles=tiles.to(self.device), host_kv_lens=kvl, host_q_lens=qlens)
+                        tiles=tiles, qtiles=qtiles, host_kv_lens=kvl, host_q_lens=qlens,
+                        states=self._h2d_i32([self.bm.state(s.id) for s, _, _ in chunks]))
         ntok = cu[-1]
+        out_rows = rows if rows is not None else out_rows
         inp = StepInput(self._h2d_i32(np.concatenate(ids)), self._h2d_i32(np.concatenate(pos)),
                         self._h2d_i32(np.concatenate(slots)), meta,
                         self._h2d_i32(out_rows) if out_rows else self._h2d_i32([ntok - 1]))
@@ -600,13 +692,20 @@ class LLMEngine:
             s._bt_np, s._bt_nb = row, nb
         return row
 
-    def _decode_inputs_host(self, seqs, B):
-        """Packed int32 metadata: ids[B] pos[B] slots[B] kv_lens[B] bt[B*maxb] (+ pad to even)."""
+    def _meta_ints(self, B):
+        n = (5 + self.max_blocks) * B
+        return n + n % 2  # even: the sampling block behind it starts with int64 seeds
+
+    def _meta_views(self, buf, B):
+        """(ids, pos, slots, kv_lens, states, block tables) views of a packed int32 decode buffer."""
         mb = self.max_blocks
+        return tuple(buf[i * B:(i + 1) * B] for i in range(5)) + (buf[5 * B:(5 + mb) * B].reshape(B, mb),)
+
+    def _decode_inputs_host(self, seqs, B):
+        """Packed int32 metadata: ids[B] pos[B] slots[B] kv_lens[B] states[B] bt[B*maxb] (+ pad to even)."""
         n = len(seqs)
-        out = np.zeros(4 * B + B * mb + (4 * B + B * mb) % 2, dtype=np.int32)
-        ids, pos, slots, kvl = (out[i * B:(i + 1) * B] for i in range(4))
-        bt = out[4 * B:4 * B + B * mb].reshape(B, mb)
+        out = np.zeros(self._meta_ints(B), dtype=np.int32)
+        ids, pos, slots, kvl, states, bt = self._meta_views(out, B)
         kvl[:] = 1  # padded rows: 1 scratch token in block 0
         if n:
             p = np.fromiter((s.length - 1 for s in seqs), dtype=np.int32, count=n)
@@ -615,37 +714,34 @@ class LLMEngine:
             pos[:n] = p
             slots[:n] = bt[np.arange(n), p // BLOCK] * BLOCK + p % BLOCK
             kvl[:n] = p + 1
+            states[:n] = [self.bm.state(s.id) for s in seqs]
         return out
 
     def _decode_graph(self, B):
         if B in self.graphs:
             return self.graphs[B]
-        from ..ops.native import decode_partitions
-
         m = self.model
         dev = self.device
-        mb = self.max_blocks
-        meta_n = 4 * B + B * mb + (4 * B + B * mb) % 2  # even: the sampling block holds int64 seeds
+        meta_n = self._meta_ints(B)
         # ONE H2D copy per step: [decode metadata | sampling params (6B) | carry map (B)]
         packed = torch.zeros(meta_n + 7 * B, dtype=torch.int32, device=dev)
-        ids, pos, slots, kvl = (packed[i * B:(i + 1) * B] for i in range(4))
+        ids, pos, slots, kvl, states, bt = self._meta_views(packed, B)
         carry = packed[meta_n + 6 * B:meta_n + 7 * B]
-        bt = packed[4 * B:4 * B + B * mb].view(B, mb)
-        pt, mp = decode_partitions(self.max_model_len, B, m.Hkv)
-        ws_o = torch.empty((B, m.Hq, mp, m.D), dtype=torch.float32, device=dev) if mp > 1 else None
-        ws_ml = torch.empty((B, m.Hq, mp, 2), dtype=torch.float32, device=dev) if mp > 1 else None
-        meta = AttnMeta("decode", kvl, bt, part_tiles=pt, max_parts=mp, ws_o=ws_o, ws_ml=ws_ml)
+        pt, mp, ws_o, ws_ml = m.decode_work(self.max_model_len, B)
+        meta = AttnMeta("decode", kvl, bt, part_tiles=pt, max_parts=mp, ws_o=ws_o, ws_ml=ws_ml, states=states)
         temps, ks, ps, seeds, steps = self._sampling_views(packed[meta_n:meta_n + 6 * B], B)
         samp = dict(temps=temps, ks=ks, ps=ps, seeds=seeds, steps=steps)
         out_tok = self._tok_out[:B]
         inp = StepInput(ids, pos, slots, meta, None, carry=carry, carry_src=self._tok_out)
 
+        entry = dict(packed=packed, samp=samp, out=out_tok, graph=None, meta=meta, inp=inp, logits=None)
+
         def run():
-            logits = m.forward(inp)
+            logits = entry["logits"] = m.forward(inp)  # kept: a replayed step's logits can be read back
             self._sample_rows(logits, samp["temps"], samp["ks"], samp["ps"], samp["seeds"], samp["steps"],
                               out=out_tok)
 
-        entry = dict(packed=packed, samp=samp, out=out_tok, run=run, graph=None, meta=meta, inp=inp)
+        entry["run"] = run
         if self.use_graphs:
             kvl.fill_(1)  # scratch-only rows while capturing
             carry.fill_(-1)
@@ -686,11 +782,9 @@ class LLMEngine:
     def _decode_inputs_async(self, seqs, B, carried):
         """As _decode_inputs_host, for a step whose rows with carried[i] feed the previous step's
         in-flight token (position = committed length; id patched on the device)."""
-        mb = self.max_blocks
         n = len(seqs)
-        out = np.zeros(4 * B + B * mb + (4 * B + B * mb) % 2, dtype=np.int32)
-        ids, pos, slots, kvl = (out[i * B:(i + 1) * B] for i in range(4))
-        bt = out[4 * B:4 * B + B * mb].reshape(B, mb)
+        out = np.zeros(self._meta_ints(B), dtype=np.int32)
+        ids, pos, slots, kvl, states, bt = self._meta_views(out, B)
         kvl[:] = 1
         if n:
             c = np.asarray(carried, dtype=np.int32)
@@ -701,6 +795,7 @@ class LLMEngine:
             pos[:n] = p
             slots[:n] = bt[np.arange(n), p // BLOCK] * BLOCK + p % BLOCK
             kvl[:n] = p + 1
+            states[:n] = [self.bm.state(s.id) for s in seqs]
         return out
 
     def _decode_async(self, ready):
@@ -758,6 +853,11 @@ class LLMEngine:
         self._count_batch(n)
         self.stats["decode_s"] += time.perf_counter() - t0
         return fin
+
+    def _decode_input_cpu(self, host, n):
+        ids, pos, slots, kvl, states, bt = self._meta_views(torch.from_numpy(host), n)
+        meta = AttnMeta("decode", kvl, bt, host_kv_lens=kvl.tolist(), states=states)
+        return StepInput(ids, pos, slots, meta, None)
 
     def _count_batch(self, n):
         """Decode steps per batch size (stats["decode_batch_hist"]): how well the schedule keeps the
@@ -884,12 +984,7 @@ class LLMEngine:
                 return finished
         else:
             host = self._decode_inputs_host(seqs, n)
-            mb = self.max_blocks
-            t = torch.from_numpy(host)
-            kvl = t[3 * n:4 * n]
-            meta = AttnMeta("decode", kvl, t[4 * n:4 * n + n * mb].view(n, mb), host_kv_lens=kvl.tolist())
-            inp = StepInput(t[:n], t[n:2 * n], t[2 * n:3 * n], meta, None)
-            logits = self.model.forward(inp)
+            logits = self.model.forward(self._decode_input_cpu(host, n))
             if full_vocab:
                 tok = self._sample_full_vocab(logits, seqs)
             else:

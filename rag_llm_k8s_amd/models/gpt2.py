@@ -15,6 +15,7 @@ from dataclasses import dataclass
 import torch
 
 from ..ops.backend import get_backend
+from .base import DecoderModel
 
 
 @dataclass
@@ -98,7 +99,7 @@ class GPT2Weights:
         return cls.from_hf(cfg, lambda n: sd[n], lambda n: n in sd, device)
 
 
-class GPT2Model:
+class GPT2Model(DecoderModel):
     def __init__(self, cfg: GPT2Config, weights: GPT2Weights, device, comm=None, max_positions=None):
         self.cfg, self.w, self.device = cfg, weights, torch.device(device)
         self.be = get_backend(self.device)

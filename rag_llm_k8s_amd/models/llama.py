@@ -22,8 +22,9 @@ from typing import List, Optional
 
 import torch
 
-from ..ops.backend import AttnMeta, get_backend
+from ..ops.backend import AttnMeta, get_backend  # noqa: F401
 from ..ops.reference import pack_gate_up, rope_tables
+from .base import DecoderModel, StepInput
 
 # decode batches up to this size run the down projection on the register-streaming GEMM (fused residual)
 DECODE_DOWN_SKINNY_MAX_M = 4
@@ -225,20 +226,7 @@ class LlamaWeights:
 
 
 # ------------------------------------------------------------------------------------- model
-@dataclass
-class StepInput:
-    ids: torch.Tensor  # int32 [T]
-    positions: torch.Tensor  # int32 [T]
-    slots: torch.Tensor  # int32 [T]
-    meta: AttnMeta
-    logits_idx: Optional[torch.Tensor] = None  # int32 [n] rows that need logits (None = all)
-    # asynchronous decode: carry[i] >= 0 -> ids[i] = carry_src[carry[i]] (previous step's sampled token,
-    # resolved on the device by the embedding kernel)
-    carry: Optional[torch.Tensor] = None
-    carry_src: Optional[torch.Tensor] = None
-
-
-class LlamaModel:
+class LlamaModel(DecoderModel):
     def __init__(self, cfg: LlamaConfig, weights: LlamaWeights, device, comm=None, max_positions=None):
         self.cfg, self.w, self.device = cfg, weights, torch.device(device)
         self.be = get_backend(self.device)

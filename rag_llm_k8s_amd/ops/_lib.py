@@ -88,6 +88,17 @@ _SIGS = {
     "ragk_gemm_stream_splits": [I, I, I, I],
     "ragk_quant_fp8_rows": [P, I, P, I, P, I, I, S],
     "ragk_gemm_fp8": [P, I, P, I, P, P, I, P, P, I, P, P, I, I, I, I, I, I, S],
+    # residual.hip / gemm_f32.hip / attn_shaped.hip / ssm.hip
+    "ragk_embed_residual": [P, P, P, I, I, I, P, P, I, S],
+    "ragk_residual_norm": [P, P, I, I, I, P, P, P, I, I, I, I, F, S],
+    "ragk_slab_rows": [P, I, P, P, I, I, I, S],
+    "ragk_glu_clip": [P, P, I, I, P, S],
+    "ragk_gemm_f32": [P, I, P, I, P, I, P, I, I, I, S],
+    "ragk_shaped_kv_store": [P, I, I, I, I, I, I, I, P, P, P, P, I, P, I, S],
+    "ragk_shaped_attn_rows": [P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, F, F, I, S],
+    "ragk_ssm_conv": [P, P, P, I, I, P, I, I, P, P, P, P, I, I, I, S],
+    "ragk_ssm_scan_seq": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, I, S],
+    "ragk_ssm_gate_norm": [P, P, I, P, P, I, I, I, I, F, I, S],
     # csrc/comm/allreduce.hip (xGMI peer-mapped all-reduce)
     "ragk_ar_create": [I, I, ctypes.c_long, I, I, I],
     "ragk_ar_add_rmsnorm": [P, P, I, I, P, I, P, P, I, I, F, I, S],
@@ -109,6 +120,7 @@ _RESTYPES = {"ragk_host_word_alloc": ctypes.c_void_p, "ragk_host_word_dev": ctyp
              "ragk_ar_create": ctypes.c_void_p, "ragk_ar_error_host_ptr": ctypes.c_void_p, "ragk_ar_max_bytes": ctypes.c_long, "ragk_ar_destroy": None}
 
 _lib = None
+_partial = None  # (path, kernel sources) of the library to load when the whole one is not built
 _lock = threading.Lock()
 
 
@@ -128,13 +140,19 @@ def lib():
     with _lock:
         if _lib is not None:
             return _lib
-        if not os.path.exists(LIB_PATH):
+        path, only = LIB_PATH, None
+        if not os.path.exists(path) and _partial is not None:
+            path, only = _partial
+        if not os.path.exists(path):
             raise NativeLibraryError(
                 "gfx950 kernel library not built (%s). Run `python -m rag_llm_k8s_amd._build` "
                 "or __graft_entry__.build()." % LIB_PATH)
-        h = ctypes.CDLL(LIB_PATH, mode=ctypes.RTLD_GLOBAL)
-        _check_stamp(h)
+        h = ctypes.CDLL(path, mode=ctypes.RTLD_GLOBAL)
+        _check_stamp(h, only)
         for name, args in _SIGS.items():
+            if only is not None and not hasattr(h, name):
+                setattr(h, name, _absent(name))
+                continue
             fn = getattr(h, name)
             fn.argtypes = args
             fn.restype = _RESTYPES.get(name, ctypes.c_int)
@@ -142,14 +160,35 @@ def lib():
         return h
 
 
-def _check_stamp(h):
+def _absent(name):
+    def f(*_):
+        raise NativeLibraryError("%s is not in the partial kernel library: build the whole one "
+                                 "(python -m rag_llm_k8s_amd._build)" % name)
+    return f
+
+
+def ensure_kernels(family):
+    """Make sure the kernels a model family needs can be loaded: the whole library if it is built, else a
+    library of just that family's sources, compiled now if it is missing or out of date."""
+    global _partial
+    if _lib is not None or os.path.exists(LIB_PATH):
+        return
+    from .. import _build
+
+    if family.kernels is None:
+        _build.build_hip()
+    else:
+        _partial = (_build.build_partial(family.name, family.kernels), tuple(family.kernels))
+
+
+def _check_stamp(h, only=None):
     """The library must have been built from the kernel sources in this tree (content hash compiled in
     by _build.build_hip). RAGK_ALLOW_STALE_LIB=1 skips the check (kernel A/B work only)."""
     if os.environ.get("RAGK_ALLOW_STALE_LIB") == "1":
         return
     from .. import _build
 
-    srcs, _ = _build.hip_sources()
+    srcs, _ = _build.hip_sources(only)
     if not srcs:  # installed without sources: nothing to compare against
         return
     if not hasattr(h, "ragk_build_stamp"):
@@ -157,7 +196,7 @@ def _check_stamp(h):
     f = h.ragk_build_stamp
     f.restype = ctypes.c_char_p
     f.argtypes = []
-    got, want = f().decode(), _build.source_hash()
+    got, want = f().decode(), _build.source_hash() if only is None else _build.source_hash(only)
     if got != want:
         raise NativeLibraryError("%s was built from other kernel sources (stamp %s, tree %s): rebuild it "
                                  "(python -m rag_llm_k8s_amd._build)" % (LIB_PATH, got, want))

@@ -18,6 +18,7 @@ from typing import List, Optional
 import torch
 
 from . import reference as R
+from . import reference_seq as RS
 from .fp8 import Fp8Weight, reference_linear
 
 KV_BLOCK = 64
@@ -37,6 +38,8 @@ class AttnMeta:
     ws_ml: Optional[torch.Tensor] = None
     host_kv_lens: List[int] = field(default_factory=list)
     host_q_lens: List[int] = field(default_factory=list)
+    states: Optional[torch.Tensor] = None  # int32 [S] recurrent-state slot of every sequence
+    qtiles: dict = field(default_factory=dict)  # prefill work lists by query-tile height (shaped attention)
 
 
 class TorchBackend:
@@ -213,6 +216,44 @@ class TorchBackend:
     def pool_l2norm(self, hidden, cu, mode="cls", normalize=True):
         return R.pool_l2norm(hidden, cu.cpu(), mode=mode, normalize=normalize)
 
+    # fp32 residual stream, shaped attention, state-space mixers ---------------
+    def embed_residual(self, ids, table, carry=None, prev=None):
+        """Embedding rows as the fp32 residual stream."""
+        return self.embed(ids, table, carry=carry, prev=prev).float()
+
+    def residual_norm(self, h, y, w_post, w_next, eps, n, out_dtype):
+        return RS.residual_norm(h, y, w_post, w_next, eps, n, out_dtype)
+
+    def proj_rows(self, x, w, bias=None):
+        """Decode projection rows for a consumer that sums them: fp32 slabs [S, M, N] + the bias still to add."""
+        return self.gemm(x, w, out_f32=True).unsqueeze(0), bias
+
+    def gemm_glu(self, x, w, par):
+        """Packed gate/up projection with the clipped GLU (par = [limit, alpha, shift])."""
+        g, u = R.unpack_gate_up(w)
+        xf = x.float()
+        return RS.glu_clip(xf @ g.float().t(), xf @ u.float().t(), par).to(x.dtype)
+
+    def shaped_kv_store(self, row, spec, slots, kc, vc, v_first=None, lam=None):
+        return RS.kv_store(row, spec, slots, kc, vc, v_first, lam)
+
+    def shaped_attn_prefill(self, row, spec, table, kc, vc, meta: AttnMeta, out):
+        return RS.attention(row, spec, table, kc, vc, meta.block_tables, meta.host_q_lens, meta.host_kv_lens, out)
+
+    def shaped_attn_decode(self, P, bias, spec, table, slots, kc, vc, meta: AttnMeta, out, v_first=None, lam=None):
+        """One new token per sequence from its projection slabs: cache append, attention, gate. Returns own values."""
+        row = RS.rows_of(P, bias)
+        own = RS.kv_store(row, spec, slots, kc, vc, v_first, lam)
+        RS.attention(row, spec, table, kc, vc, meta.block_tables, [1] * row.shape[0], meta.host_kv_lens, out)
+        return own
+
+    def ssm_prefill(self, row, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
+        return RS.ssm(row, spec, w, eps, meta.host_q_lens, meta.host_kv_lens, meta.states, conv_state, ssm_state, out)
+
+    def ssm_decode(self, P, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
+        row = RS.rows_of(P, None)
+        return RS.ssm(row, spec, w, eps, [1] * row.shape[0], meta.host_kv_lens, meta.states, conv_state, ssm_state, out)
+
     # sampling -----------------------------------------------------------------
     def topk_candidates(self, logits, K, vocab_offset=0, max_cand=512, chunks=None):
         k = min(K, logits.shape[1])
@@ -246,14 +287,18 @@ class NativeBackend(TorchBackend):
 
     def __init__(self, device="cuda"):
         super().__init__(device)
-        from . import native
+        from . import native, seq_native
 
-        self.n = native
+        self.n, self.q = native, seq_native
         native._lib.lib()  # fail loudly now if the gfx950 library is missing
 
     def gemm(self, x, w, bias=None, resid=None, epi="none", out=None, out_f32=False):
         if isinstance(w, Fp8Weight):
             return self.n.gemm_fp8(x, w, bias=bias, resid=resid, epi=epi, out=out, out_f32=out_f32)
+        if w.dtype == torch.float32:  # exact replay: plain rows with at most a bias
+            if resid is not None or out is not None or epi not in ("none", "bias"):
+                raise ValueError("fp32 gemm has no %s epilogue" % epi)
+            return self.q.gemm_f32(x, w, bias)
         return self.n.gemm(x, w, bias=bias, resid=resid, epi=epi, out=out, out_f32=out_f32)
 
     def rmsnorm(self, x, w, eps, out=None):
@@ -269,6 +314,8 @@ class NativeBackend(TorchBackend):
         return self.n.embed_ln(ids, pos_ids, word, pos, type_row, g, b, eps, do_ln=do_ln)
 
     def gather_rows(self, x, idx):
+        if x.dtype == torch.float32:  # the same bytes as rows of twice as many 16-bit columns
+            return self.n.gather_rows(x.view(torch.bfloat16), idx).view(torch.float32)
         return self.n.gather_rows(x, idx)
 
     def silu_mul(self, x):
@@ -353,6 +400,45 @@ class NativeBackend(TorchBackend):
     def attn_decode(self, q, kc, vc, meta: AttnMeta, out, Hq, Hkv, D):
         return self.n.attn_decode(q, kc, vc, meta.block_tables, meta.kv_lens, out, Hq, Hkv, D, meta.part_tiles,
                                   meta.max_parts, meta.ws_o, meta.ws_ml)
+
+    # fp32 residual stream, shaped attention, state-space mixers ---------------
+    def embed_residual(self, ids, table, carry=None, prev=None):
+        return self.q.embed_residual(ids, table, carry, prev)
+
+    def residual_norm(self, h, y, w_post, w_next, eps, n, out_dtype):
+        return self.q.residual_norm(h, y, w_post, w_next, eps, n, out_dtype)
+
+    def proj_rows(self, x, w, bias=None):
+        if w.dtype == torch.float32:
+            return self.q.gemm_f32(x, w, bias).unsqueeze(0), None
+        if self.part_ok(x.shape[0], w):
+            return self.n.gemm_part(x, w), bias
+        return self.n.gemm(x, w, out_f32=True).unsqueeze(0), bias
+
+    def gemm_glu(self, x, w, par):
+        if w.dtype == torch.float32:
+            return self.q.glu_clip_f32(self.q.gemm_f32(x, w), par)
+        return self.n.gemm_glu(x, w, par)
+
+    def shaped_kv_store(self, row, spec, slots, kc, vc, v_first=None, lam=None):
+        return self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
+
+    def shaped_attn_prefill(self, row, spec, table, kc, vc, meta: AttnMeta, out):
+        return self.q.attn_rows(row, spec, table, kc, vc, meta, out)
+
+    def shaped_attn_decode(self, P, bias, spec, table, slots, kc, vc, meta: AttnMeta, out, v_first=None, lam=None):
+        row = self.q.slab_rows(P, bias, out.dtype)
+        own = self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
+        self.q.attn_rows(row, spec, table, kc, vc, meta, out)
+        return own
+
+    def ssm_prefill(self, row, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
+        xbc = self.q.ssm_conv(row, spec, w, meta, conv_state, ssm_state)
+        y = self.q.ssm_scan_seq(xbc, row, spec, w, meta, ssm_state)
+        return self.q.ssm_gate_norm(y, row, spec, w, eps, out)
+
+    def ssm_decode(self, P, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
+        return self.ssm_prefill(self.q.slab_rows(P, None, out.dtype), spec, w, eps, meta, conv_state, ssm_state, out)
 
     def attn_encoder(self, qkv, cu, lens_host, tiles, out, H, D):
         return self.n.attn_prefill(qkv, qkv[:, H * D:], qkv[:, 2 * H * D:], cu, _lens_dev(cu), tiles, out, H, H, D,

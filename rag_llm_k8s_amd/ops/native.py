@@ -17,6 +17,9 @@ from ._lib import check, ptr, stream_ptr
 from .reference import EPI
 
 
+PAIR_EPI = ("silu_mul", "glu_clip")  # epilogues over packed [64 gate | 64 up] weight rows
+
+
 def _req(cond, msg):
     if not cond:
         raise ValueError(msg)
@@ -58,7 +61,7 @@ def dec_workspace(device):
 def use_dec(M, N, K, epi):
     """v3 (LDS-shared activations) wins over v1 only on vocab-sized N at M > 16 (lm_head: 5.1 vs
     3.1 TB/s at M=32, cache-cold); v1 stays the default elsewhere (profiles/kernels_r1_decode.json)."""
-    return 16 < M <= 64 and N >= 32768 and K % 256 == 0 and epi != "silu_mul"
+    return 16 < M <= 64 and N >= 32768 and K % 256 == 0 and epi not in PAIR_EPI
 
 
 STREAM_DEFAULT = True
@@ -74,7 +77,7 @@ def use_stream(M, N, K, epi, fp8=False):
     no split-K: the packed gate/up projection (4.5 vs 3.4 TB/s bf16 at M=32, 4.4 vs 2.2 at M=64;
     fp8 2.6 vs 1.5 at M=32) and other 16k-32k-row weights. Below that, the fixed pipeline-fill +
     split-K reduction latencies lose to the register-streaming kernels (profiles/tune_stream_r1.json)."""
-    rows = 2 * N if epi == "silu_mul" else N
+    rows = 2 * N if epi in PAIR_EPI else N
     if M > 64 or not (STREAM_MIN_ROWS <= rows < STREAM_MAX_ROWS) or K % 128:
         return False
     if rows >= 32768 and M < STREAM_VOCAB_MIN_M:
@@ -87,7 +90,7 @@ def use_pp(M, N, K, epi):
     faster on the Llama-8B prefill shapes, profiles/gemm_w4_r1.txt) or the 8-wave ping-pong gemm_pp.hip."""
     if M < PP_MIN_M or K % 64 or K < 192:  # gemm_w4's continuous ring needs three K-tiles per tile
         return False
-    return N % 128 == 0 if epi == "silu_mul" else N % 8 == 0
+    return N % 128 == 0 if epi in PAIR_EPI else N % 8 == 0
 
 
 # Large-M GEMMs through hipBLASLt (torch) instead of gemm_w4, by epilogue (A/B only). "none" (default):
@@ -162,11 +165,14 @@ def gemm(x, w, bias=None, resid=None, epi="none", out=None, out_f32=False, path=
     _bf16_2d(w, "w")
     M, K = x.shape
     e = EPI[epi]
-    N = w.shape[0] // 2 if epi == "silu_mul" else w.shape[0]
+    N = w.shape[0] // 2 if epi in PAIR_EPI else w.shape[0]
     _req(w.shape[1] == K, "K mismatch %s vs %s" % (tuple(x.shape), tuple(w.shape)))
     _req(K % 128 == 0, "K must be a multiple of 128 (got %d)" % K)
-    if epi == "silu_mul":
-        _req(N % 64 == 0, "silu_mul needs N % 64 == 0")
+    if epi in PAIR_EPI:
+        _req(N % 64 == 0, "%s needs N %% 64 == 0" % epi)
+    if epi == "glu_clip":
+        _req(bias is not None and bias.is_cuda and bias.dtype == torch.float32 and bias.numel() >= 3
+             and bias.is_contiguous(), "glu_clip takes fp32 {limit, alpha, shift} as its bias")
     if "bias" in epi:
         _req(bias is not None and bias.is_cuda and bias.dtype == torch.bfloat16 and bias.numel() == N
              and bias.is_contiguous(), "bias must be bf16[N]")
@@ -177,7 +183,7 @@ def gemm(x, w, bias=None, resid=None, epi="none", out=None, out_f32=False, path=
     if out is None:
         out = torch.empty((M, N), dtype=odt, device=x.device)
     _req(out.dtype == odt and out.shape == (M, N) and out.stride(1) == 1, "out shape/dtype")
-    if M > 64 and N % 8 != 0 and epi != "silu_mul":
+    if M > 64 and N % 8 != 0 and epi not in PAIR_EPI:
         raise ValueError("tile GEMM needs N % 8 == 0")
     if M == 0:
         return out
@@ -191,6 +197,11 @@ def gemm(x, w, bias=None, resid=None, epi="none", out=None, out_f32=False, path=
         rows = w.shape[0]
         # gemm_w4 addresses operands with 32-bit buffer offsets
         fits = x.stride(0) * M * 2 < 2 ** 31 and w.stride(0) * rows * 2 < 2 ** 31
+        if epi == "glu_clip" and not fits:  # gemm_pp has no clipped unit: halve the rows until they fit
+            h = (M // 2 + 127) // 128 * 128
+            gemm(x[:h], w, bias=bias, epi=epi, out=out[:h])
+            gemm(x[h:], w, bias=bias, epi=epi, out=out[h:])
+            return out
         path = 6 if fits else 2  # gemm_pp (8-wave ping-pong, 64-bit addressing): operands past 2 GiB
     if path is None and STREAM_DEFAULT and use_stream(M, N, K, epi):
         path = 5
@@ -221,6 +232,11 @@ def gemm(x, w, bias=None, resid=None, epi="none", out=None, out_f32=False, path=
                               out.stride(0), ptr(bias), ptr(resid), ldr, M, N, K, e, stream_ptr())
     check(rc, "ragk_gemm")
     return out
+
+
+def gemm_glu(x, w, par):
+    """Packed gate/up projection with the clipped gated unit (par: fp32 {limit, alpha, shift} on the device)."""
+    return gemm(x, w, bias=par, epi="glu_clip")
 
 
 PART_MIN_BLOCKS = 512
@@ -662,7 +678,7 @@ def _gemm_stream(x, w, wscale, out, bias, resid, ldr, M, N, K, epi, e, out_f32):
     fp8 = wscale is not None
     S = STREAM_S_OVERRIDE or L.ragk_gemm_stream_splits(N, K, e, int(fp8))
     ws, cnt = dec_workspace(x.device)
-    rows = 2 * N if epi == "silu_mul" else N
+    rows = 2 * N if epi in PAIR_EPI else N
     _req(S == 1 or S * M * (-(-rows // 128) * 128) <= ws.numel(), "stream GEMM workspace too small")
     _req(-(-rows // 64) <= cnt.numel(), "too many n-tiles for the counter buffer")
     return L.ragk_gemm_stream(x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), ptr(wscale), out.data_ptr(),

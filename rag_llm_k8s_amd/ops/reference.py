@@ -16,7 +16,7 @@ import torch
 import torch.nn.functional as F
 
 EPI = {"none": 0, "bias": 1, "resid": 2, "bias_resid": 3, "bias_gelu": 4, "silu_mul": 5, "gelu": 6,
-       "bias_gelu_tanh": 7}
+       "bias_gelu_tanh": 7, "glu_clip": 9}
 
 
 def pack_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:

@@ -1,0 +1,219 @@
+"""Shape-checked entry points of the residual-stream, shaped-attention and state-space kernels (GPU tensors).
+
+Operands are checked on the host before every launch, as in ops/native.py. `f32` paths (exact replay) take
+fp32 tensors throughout; otherwise activations and caches are bf16 and the residual stream, split-K slabs,
+norm weights and recurrent states fp32.
+"""
+from __future__ import annotations
+
+import numpy as np
+import torch
+
+from . import _lib
+from ._lib import check, ptr, stream_ptr
+from .native import _req
+
+BF16, F32, I32 = torch.bfloat16, torch.float32, torch.int32
+
+
+def _act(t, name):
+    _req(t.is_cuda and t.dtype in (BF16, F32) and t.dim() == 2 and t.stride(1) == 1, "%s must be 2-D bf16/fp32 rows" % name)
+    return int(t.dtype == F32)
+
+
+def _vec(t, n, dtype, name):
+    _req(t.is_cuda and t.dtype == dtype and t.is_contiguous() and t.numel() == n, "%s must be %s[%d]" % (name, dtype, n))
+
+
+# ------------------------------------------------------------------------------------- residual stream
+def embed_residual(ids, table, carry=None, prev=None):
+    _req(ids.dtype == I32 and ids.is_cuda and ids.is_contiguous() and table.is_contiguous(), "ids int32, table dense")
+    V, W = table.shape
+    f32 = _act(table, "table")
+    if carry is not None:
+        _req(carry.dtype == I32 and prev.dtype == I32 and carry.numel() >= ids.numel(), "carry int32")
+    h = torch.empty((ids.numel(), W), dtype=F32, device=table.device)
+    check(_lib.lib().ragk_embed_residual(ids.data_ptr(), table.data_ptr(), h.data_ptr(), ids.numel(), W, V, ptr(carry),
+                                         ptr(prev) if carry is not None else None, f32, stream_ptr()),
+          "ragk_embed_residual")
+    return h
+
+
+def residual_norm(h, y, w_post, w_next, eps, n, out_dtype):
+    """h += norm(y) * w_post (in place), returns norm(h) * w_next in out_dtype. y: rows [M, W] (bf16 / fp32),
+    fp32 slabs [S, M, W], or None."""
+    M, W = h.shape
+    _req(h.is_cuda and h.dtype == F32 and h.is_contiguous() and W % 8 == 0 and W <= 16384, "h fp32 [M, W]")
+    S, bf, ldy = 1, 0, W
+    if y is not None:
+        _req(y.is_cuda and y.dtype in (BF16, F32) and y.is_contiguous() and y.shape[-2:] == (M, W), "y rows / slabs")
+        bf = int(y.dtype == BF16)
+        S = y.shape[0] if y.dim() == 3 else 1
+        _req(S == 1 or not bf, "bf16 rows come as one slab")
+    for w, name in ((w_post, "w_post"), (w_next, "w_next")):
+        if w is not None:
+            _vec(w, W, F32, name)
+    out = torch.empty((M, W), dtype=out_dtype, device=h.device) if w_next is not None else None
+    check(_lib.lib().ragk_residual_norm(h.data_ptr(), ptr(y), ldy, S, bf, ptr(w_post), ptr(w_next), ptr(out),
+                                        int(out_dtype == F32), M, W, n, float(eps), stream_ptr()), "ragk_residual_norm")
+    return out
+
+
+def slab_rows(P, bias, dtype):
+    S, M, N = P.shape
+    _req(P.is_cuda and P.dtype == F32 and P.is_contiguous() and N % 8 == 0, "slabs fp32 [S, M, N]")
+    if bias is not None:
+        _vec(bias, N, dtype, "bias")
+    out = torch.empty((M, N), dtype=dtype, device=P.device)
+    check(_lib.lib().ragk_slab_rows(P.data_ptr(), S, ptr(bias), out.data_ptr(), M, N, int(dtype == F32), stream_ptr()),
+          "ragk_slab_rows")
+    return out
+
+
+def gemm_f32(x, w, bias=None):
+    _req(_act(x, "x") and _act(w, "w") and x.shape[1] == w.shape[1] and x.shape[1] % 32 == 0, "gemm_f32 operands")
+    _req(x.stride(0) % 4 == 0 and w.stride(0) % 4 == 0, "gemm_f32 row strides")
+    M, K = x.shape
+    N = w.shape[0]
+    if bias is not None:
+        _vec(bias, N, F32, "bias")
+    out = torch.empty((M, N), dtype=F32, device=x.device)
+    check(_lib.lib().ragk_gemm_f32(x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), out.data_ptr(), N, ptr(bias), M, N,
+                                   K, stream_ptr()), "ragk_gemm_f32")
+    return out
+
+
+def glu_clip_f32(x, par):
+    _req(_act(x, "x") and x.is_contiguous() and x.shape[1] % 128 == 0, "packed gate/up rows")
+    _vec(par, 4, F32, "par")
+    M, F = x.shape[0], x.shape[1] // 2
+    out = torch.empty((M, F), dtype=F32, device=x.device)
+    check(_lib.lib().ragk_glu_clip(x.data_ptr(), out.data_ptr(), M, F, par.data_ptr(), stream_ptr()), "ragk_glu_clip")
+    return out
+
+
+# ------------------------------------------------------------------------------------- work lists
+def query_tiles(q_lens, qt):
+    """(seq, first query) work list of qt-row query tiles, latest (heaviest) first."""
+    ql = np.asarray(q_lens, dtype=np.int64)
+    nt = (ql + qt - 1) // qt
+    seq = np.repeat(np.arange(len(ql)), nt)
+    first = np.repeat(np.cumsum(nt) - nt, nt)
+    q0 = (np.arange(int(nt.sum())) - first) * qt
+    order = np.argsort(-q0, kind="stable")
+    return torch.from_numpy(np.stack([seq[order], q0[order]], 1).astype(np.int32)).reshape(-1, 2)
+
+
+def decode_split(specs, max_kv_len, batch, device):
+    return 1, 1, None, None
+
+
+# ------------------------------------------------------------------------------------- shaped attention
+def _caches(kc, vc, spec, dtype):
+    _req(kc.dim() == 4 and kc.shape[1:] == (spec.kv_heads, 64, spec.dkp) and kc.is_contiguous() and kc.dtype == dtype,
+         "K pages [blocks, kv_heads, 64, dk]")
+    _req(vc.shape == (kc.shape[0], spec.kv_heads, 64, spec.dvp) and vc.is_contiguous() and vc.dtype == dtype,
+         "V pages [blocks, kv_heads, 64, dv]")
+
+
+def kv_store(row, spec, slots, kc, vc, v_first=None, lam=None):
+    """k and (mixed) v of each token into the pages at `slots`; returns the tokens' own values (a view)."""
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    _req(row.shape[1] >= spec.off_g and row.stride(0) % 8 == 0, "projection rows")
+    _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == T, "slots int32[T]")
+    _caches(kc, vc, spec, row.dtype)
+    ldf = 0
+    if v_first is not None:
+        _req(v_first.dtype == row.dtype and v_first.shape == (T, spec.kv_heads * spec.dvp) and v_first.stride(1) == 1
+             and v_first.data_ptr() % 16 == 0, "v_first rows")
+        _vec(lam, 1, F32, "lam")
+        ldf = v_first.stride(0)
+    check(_lib.lib().ragk_shaped_kv_store(row.data_ptr(), row.stride(0), spec.off_k, spec.off_v, T, spec.kv_heads, spec.dkp,
+                                          spec.dvp, slots.data_ptr(), kc.data_ptr(), vc.data_ptr(), ptr(v_first), ldf,
+                                          ptr(lam) if v_first is not None else None, f32, stream_ptr()),
+          "ragk_shaped_kv_store")
+    return row[:, spec.off_v:spec.off_g]
+
+
+def _table(table, spec):
+    if table is not None:
+        _vec(table.reshape(-1), spec.heads * (spec.far + 1), F32, "bias table")
+
+
+def _meta(meta, T, decode):
+    S = meta.kv_lens.numel()
+    _req(meta.kv_lens.dtype == I32 and meta.block_tables.dtype == I32 and meta.block_tables.shape[0] == S
+         and meta.block_tables.stride(1) == 1, "kv_lens / block tables int32")
+    if decode:
+        _req(S == T, "one token per sequence")
+    else:
+        _req(meta.cu_q is not None and meta.cu_q.dtype == I32 and meta.cu_q.numel() == S + 1, "cu_q int32[S + 1]")
+    return S, None if decode else meta.cu_q.data_ptr()
+
+
+def attn_rows(row, spec, table, kc, vc, meta, out):
+    """Plain attention, one wave per (token, head): any head size, bf16 or fp32."""
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    S, cu = _meta(meta, T, meta.kind == "decode")
+    _caches(kc, vc, spec, row.dtype)
+    _table(table, spec)
+    _req(out.dtype == row.dtype and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
+    check(_lib.lib().ragk_shaped_attn_rows(
+        row.data_ptr(), row.stride(0), kc.data_ptr(), vc.data_ptr(), meta.block_tables.data_ptr(),
+        meta.block_tables.stride(0), cu, meta.kv_lens.data_ptr(), ptr(table), out.data_ptr(), out.stride(0), T, S,
+        spec.heads, spec.kv_heads, spec.dkp, spec.dvp, spec.off_g if spec.gate else -1, spec.window, spec.keep_first,
+        spec.far, int(spec.sink), float(spec.scale), float(spec.softcap), f32, stream_ptr()), "ragk_shaped_attn_rows")
+    return out
+
+
+# ------------------------------------------------------------------------------------- state space
+def _states(meta, spec, conv_state, ssm_state):
+    n = ssm_state.shape[0]
+    _req(meta.states is not None and meta.states.dtype == I32 and meta.states.numel() == meta.kv_lens.numel(), "state slots")
+    _req(ssm_state.dtype == F32 and ssm_state.is_contiguous()
+         and ssm_state.shape == (n, spec.heads, spec.state, spec.vdim), "ssm_state")
+    _req(conv_state.dtype == F32 and conv_state.is_contiguous() and conv_state.shape == (n, spec.taps - 1, spec.channels),
+         "conv_state")
+
+
+def ssm_conv(row, spec, w, meta, conv_state, ssm_state):
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    S, cu = _meta(meta, T, meta.kind == "decode")
+    _states(meta, spec, conv_state, ssm_state)
+    _req(row.shape[1] >= spec.off_dt + spec.heads, "projection rows")
+    _vec(w["conv_w"].reshape(-1), spec.taps * spec.channels, F32, "conv_w")
+    _vec(w["conv_b"], spec.channels, F32, "conv_b")
+    xbc = torch.empty((T, spec.channels), dtype=row.dtype, device=row.device)
+    check(_lib.lib().ragk_ssm_conv(cu, meta.kv_lens.data_ptr(), meta.states.data_ptr(), T, S, row.data_ptr(), row.stride(0),
+                                   spec.off_x, w["conv_w"].data_ptr(), w["conv_b"].data_ptr(), conv_state.data_ptr(),
+                                   xbc.data_ptr(), spec.channels, spec.taps, f32, stream_ptr()), "ragk_ssm_conv")
+    return xbc
+
+
+def ssm_scan_seq(xbc, row, spec, w, meta, ssm_state):
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    S, cu = _meta(meta, T, meta.kind == "decode")
+    for k in ("dt_bias", "A", "D"):
+        _vec(w[k], spec.heads, F32, k)
+    y = torch.empty((T, spec.inner), dtype=F32, device=row.device)
+    check(_lib.lib().ragk_ssm_scan_seq(cu, meta.kv_lens.data_ptr(), meta.states.data_ptr(), T, S, xbc.data_ptr(),
+                                       xbc.stride(0), row.data_ptr(), row.stride(0), spec.off_dt, w["dt_bias"].data_ptr(),
+                                       w["A"].data_ptr(), w["D"].data_ptr(), ssm_state.data_ptr(), y.data_ptr(), spec.heads,
+                                       spec.vdim, spec.state, spec.groups, f32, stream_ptr()), "ragk_ssm_scan_seq")
+    return y
+
+
+def ssm_gate_norm(y, row, spec, w, eps, out):
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    _req(y.dtype == F32 and y.is_contiguous() and y.shape == (T, spec.inner), "y fp32 [T, inner]")
+    _req(out.dtype == row.dtype and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
+    _vec(w["norm"], spec.inner, F32, "norm")
+    check(_lib.lib().ragk_ssm_gate_norm(y.data_ptr(), row.data_ptr(), row.stride(0), w["norm"].data_ptr(), out.data_ptr(),
+                                        out.stride(0), T, spec.inner, spec.norm_groups, float(eps), f32, stream_ptr()),
+          "ragk_ssm_gate_norm")
+    return out

@@ -1,7 +1,7 @@
 """Assemble a RagService from a RagConfig (the reference's module-scope init, rag.py:13-33,199-204).
 
 Model directory = the reference's /models PVC layout (download_model.py file list). The
-generator architecture is read from config.json (llama or gpt2); the embedder from
+generator architecture is read from config.json (models/registry.py); the embedder from
 EMBED_MODEL (a local sentence-transformers directory: the reference fetched BAAI/bge-m3
 from the network at startup, /root/reference/llm/rag.py:33, which is dropped here).
 """
@@ -29,7 +29,7 @@ def kv_blocks_for(model, cfg, device):
     per = model.kv_bytes_per_block()
     if torch.device(device).type == "cuda":
         free, _ = torch.cuda.mem_get_info(torch.device(device))
-        budget = int(free * cfg.kv_cache_fraction)
+        budget = int(free * cfg.kv_cache_fraction) - model.state_bytes_per_slot() * (cfg.max_batch + 1)
     else:
         budget = 2 << 30
     need = cfg.max_batch * (-(-cfg.max_model_len // 64)) + 8
@@ -40,30 +40,14 @@ def build_generator(cfg, device, tp_rank=0, tp_size=1, comm=None, tp_group=None)
     from ..engine.llm_engine import LLMEngine
     from ..runtime.tokenizer import Tokenizer
 
-    mcfg = _load_json(os.path.join(cfg.model_path, "config.json"))
-    if mcfg is None:
-        raise FileNotFoundError("no config.json under MODEL_PATH=%s" % cfg.model_path)
+    from ..models.registry import build_model, model_limits, read_config
+
+    raw = read_config(cfg.model_path)
     gen = _load_json(os.path.join(cfg.model_path, "generation_config.json"), {})
     tok = Tokenizer(cfg.model_path)
-    mt = mcfg.get("model_type", "llama")
-    if mt == "gpt2":
-        from ..models.gpt2 import GPT2Config, GPT2Model, GPT2Weights
-
-        c = GPT2Config.from_dict(mcfg)
-        w = GPT2Weights.from_checkpoint(cfg.model_path, c, device)
-        model = GPT2Model(c, w, device)
-        max_len = min(cfg.max_model_len, c.n_positions)
-        eos = [c.eos_token_id]
-    else:
-        from ..models.llama import LlamaConfig, LlamaModel, LlamaWeights
-
-        c = LlamaConfig.from_dict(mcfg)
-        w = LlamaWeights.from_checkpoint(cfg.model_path, c, device, tp_rank, tp_size)
-        if cfg.dtype == "fp8":  # DTYPE=fp8: e4m3fn linear weights, per-row scales
-            w.quantize_fp8()
-        max_len = min(cfg.max_model_len, c.max_position_embeddings)
-        model = LlamaModel(c, w, device, comm=comm, max_positions=max_len)
-        eos = c.eos_token_id
+    model = build_model(cfg.model_path, device, cfg.dtype, raw, tp_rank, tp_size, comm, cfg.max_model_len)
+    limit, eos = model_limits(model)
+    max_len = min(cfg.max_model_len, limit)
     geos = gen.get("eos_token_id", eos)
     eos = geos if isinstance(geos, list) else [geos]
     cfg.max_model_len = max_len

@@ -9,6 +9,15 @@
 //
 //  * kv_store     : k, and v mixed with the first mixing layer's values of the same token, into the pages.
 //  * attn_rows    : one wave per (token, query head), plain fp32 arithmetic. Any head size; the fp32 path.
+//  * attn_prefill : MFMA flash attention over 64-key pages, 4 waves = GB query heads of one KV head x (4 / GB)
+//                   groups of 32 query rows. Only pages with a visible key are visited: the pages of the kept first
+//                   tokens, then those of the window. The bias table row of each head sits in LDS.
+//  * attn_decode  : one query per sequence. Takes the projection as fp32 split-K slabs, so the slab sum, the bias
+//                   add, the value mix and the cache append need no launch of their own; the pages of a
+//                   sequence are split over partitions (attn_merge joins them) when batch x KV heads is small.
+//
+// The MFMA kernels keep the softmax weights at 16 significant bits for P.V (bf16 high + low part, two products).
+#include "attn_tiles.h"
 #include "seq_common.h"
 using namespace ragk;
 
@@ -126,7 +135,571 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(ShapedArgs a) {
   }
 }
 
+// ---- visited pages of a query range [qmin, qmax]: the kept first pages, then the window's ----
+struct Pages {
+  int n_keep, first, n;  // iteration it -> page it < n_keep ? it : first + it - n_keep
+  __device__ __forceinline__ int page(int it) const { return it < n_keep ? it : first + it - n_keep; }
+};
+__device__ __forceinline__ Pages visited(int qmin, int qmax, int window, int keep) {
+  const int n_pages = qmax / KT + 1;
+  if (window <= 0) return Pages{n_pages, n_pages, n_pages};
+  const int nk = min(n_pages, (keep + KT - 1) / KT);
+  const int f = max(nk, max(0, qmin - window + 1) / KT);
+  return Pages{nk, f, nk + max(0, n_pages - f)};
+}
+
+// softcapped score in log2 units: cap2 * tanh(x / cap) = cap2 - 2 cap2 / (1 + 2^(x * c1)); c1 = 2 scale log2e / cap
+struct Shape {
+  float c1, cap2, c;  // cap2 > 0: soft-capped; else s = x * c
+  __device__ __forceinline__ float operator()(float x) const {
+    if (cap2 > 0.f) return __builtin_fmaf(-2.f * cap2, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * c1)), cap2);
+    return x * c;
+  }
+};
+constexpr float LOG2E = 1.4426950408889634f;
+__device__ __forceinline__ Shape make_shape(float scale, float softcap) {
+  return Shape{softcap > 0.f ? 2.f * scale * LOG2E / softcap : 0.f, softcap > 0.f ? softcap * LOG2E : 0.f, scale * LOG2E};
+}
+
+// high and low bf16 parts of 8 probabilities as MFMA operands
+__device__ __forceinline__ void split_p(const f32x4& a, const f32x4& b, bf16x8& hi, bf16x8& lo) {
+  u32x4 h, l;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    h[i] = pk2bf(a[2 * i], a[2 * i + 1]);
+    h[2 + i] = pk2bf(b[2 * i], b[2 * i + 1]);
+    l[i] = pk2bf(a[2 * i] - __uint_as_float(h[i] << 16), a[2 * i + 1] - __uint_as_float(h[i] & 0xffff0000u));
+    l[2 + i] = pk2bf(b[2 * i] - __uint_as_float(h[2 + i] << 16), b[2 * i + 1] - __uint_as_float(h[2 + i] & 0xffff0000u));
+  }
+  hi = __builtin_bit_cast(bf16x8, h);
+  lo = __builtin_bit_cast(bf16x8, l);
+}
+
+struct ShapedPrefill {
+  ShapedArgs a;
+  const int* tiles; int n_hg, gb;  // work list (seq, first query); head groups; heads per block
+  int sb_stride;                   // floats per head of the LDS bias table, 0: none
+};
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_shaped_prefill_kernel(ShapedPrefill pa) {
+  using CK = Cfg<DK>;
+  using CV = Cfg<DV>;
+  const ShapedArgs& a = pa.a;
+  extern __shared__ __attribute__((aligned(16))) char smem[];  // [buf][K | V], page list, bias tables
+  int* s_bt = reinterpret_cast<int*>(smem + 2 * (CK::TILEB + CV::TILEB));
+  float* s_bias = reinterpret_cast<float*>(s_bt + MAX_BT);
+
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int wid_u = __builtin_amdgcn_readfirstlane(wid);
+  const int tix = (int)blockIdx.x / pa.n_hg, hg = (int)blockIdx.x - tix * pa.n_hg;
+  const int seq = pa.tiles[2 * tix], q_start = pa.tiles[2 * tix + 1];
+  const int G = a.H / a.G, gb = pa.gb, per_kv = G / gb;
+  const int kvh = hg / per_kv, h0 = kvh * G + (hg % per_kv) * gb, hb = wid_u % gb, hq = h0 + hb;
+  const int pbase = q_start + (wid_u / gb) * 32;
+  const int q_off = a.cu_q[seq], q_len = a.cu_q[seq + 1] - q_off, kv_len = a.kv_lens[seq];
+  const int ctx0 = kv_len - q_len;
+  const int qt_rows = 32 * (4 / gb);
+  const Pages pg = visited(ctx0 + q_start, ctx0 + min(q_start + qt_rows, q_len) - 1, a.window, a.keep);
+  const int wave_pmin = ctx0 + pbase, wave_pmax = ctx0 + min(pbase + 31, q_len - 1);
+  const int fr = lane & 15, fh = lane >> 4;
+
+  bf16x8 qf[2][CK::KS];
+#pragma unroll
+  for (int qt = 0; qt < 2; ++qt) {
+    const int qi = min(pbase + 16 * qt + fr, q_len - 1);
+    const bf16_t* qp = (const bf16_t*)a.q + (size_t)(q_off + qi) * a.ldq + hq * DK + 8 * fh;
+#pragma unroll
+    for (int s = 0; s < CK::KS; ++s) qf[qt][s] = *reinterpret_cast<const bf16x8*>(qp + 32 * s);
+  }
+  f32x4 o[CV::DT][2];
+#pragma unroll
+  for (int dt = 0; dt < CV::DT; ++dt)
+#pragma unroll
+    for (int qt = 0; qt < 2; ++qt) o[dt][qt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  // the extra zero score: running max 0, one unit in the sum (one of a query's four lanes holds it)
+  float m_i[2], l_i[2];
+#pragma unroll
+  for (int qt = 0; qt < 2; ++qt) {
+    m_i[qt] = a.sink ? 0.f : -INFINITY;
+    l_i[qt] = a.sink && fh == 0 ? 1.f : 0.f;
+  }
+  const int* bt = a.block_tables + (size_t)seq * a.bt_stride;
+  for (int i = threadIdx.x; i < pg.n; i += 256) s_bt[i] = bt[pg.page(i)];
+  if (a.table && pa.sb_stride)
+    for (int h = 0; h < gb; ++h)
+      for (int i = threadIdx.x; i <= a.far; i += 256)
+        s_bias[h * pa.sb_stride + i] = a.table[(size_t)(h0 + h) * (a.far + 1) + i] * LOG2E;
+  __syncthreads();
+  const float* tb = a.table ? (pa.sb_stride ? s_bias + hb * pa.sb_stride : a.table + (size_t)hq * (a.far + 1)) : nullptr;
+  const float tb_scale = pa.sb_stride ? 1.f : LOG2E;
+  const float far_bias = tb ? tb[a.far] * tb_scale : 0.f;
+  const Shape shape = make_shape(a.scale, a.softcap);
+
+  auto stage = [&](int it, int buf) {
+    char* sK = smem + buf * (CK::TILEB + CV::TILEB);
+    const size_t pgi = (size_t)s_bt[it] * a.G + kvh;
+    const bf16_t* kb = (const bf16_t*)a.kc + pgi * KT * DK;
+    const bf16_t* vb = (const bf16_t*)a.vc + pgi * KT * DV;
+    stage_kv<DK, false, false, 4>(sK, wid_u, 4, lane, [&](int r) { return kb + (size_t)r * DK; });
+    stage_kv<DV, true, false, 4>(sK + CK::TILEB, wid_u, 4, lane, [&](int r) { return vb + (size_t)r * DV; });
+  };
+  stage(0, 0);  // pg.n >= 1: a query always sees its own page
+  wait_vmcnt0();
+  __syncthreads();
+
+  for (int it = 0; it < pg.n; ++it) {
+    const int cur = it & 1, k0 = pg.page(it) * KT;
+    const char* sK = smem + cur * (CK::TILEB + CV::TILEB);
+    const char* sV = sK + CK::TILEB;
+    const bool active = k0 <= wave_pmax && (a.window <= 0 || wave_pmin - (k0 + KT - 1) < a.window || k0 < a.keep);
+    f32x4 s[4][2];
+    if (active) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        s[t][0] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        s[t][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < CK::KS; ++ks) {
+          const bf16x8 kf = load_k<DK>(sK, t, ks, lane);
+          s[t][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[0][ks], s[t][0], 0, 0, 0);
+          s[t][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[1][ks], s[t][1], 0, 0, 0);
+        }
+      }
+    }
+    if (it + 1 < pg.n) stage(it + 1, cur ^ 1);  // DMA of the next page behind the QK^T products
+    if (active) {
+      const bool all_visible = k0 + KT - 1 <= wave_pmin && (a.window <= 0 || wave_pmax - k0 < a.window || k0 + KT <= a.keep);
+      const bool far_only = wave_pmin - (k0 + KT - 1) >= a.far;  // one bias for the whole page
+      float alpha[2];
+#pragma unroll
+      for (int qt = 0; qt < 2; ++qt) {
+        const int qpos = ctx0 + pbase + 16 * qt + fr;
+        const int d0 = qpos - k0 - 4 * fh;  // distance of this lane's key 0
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[t][qt][r] = shape(s[t][qt][r]);
+        if (tb) {
+          if (far_only) {
+#pragma unroll
+            for (int t = 0; t < 4; ++t) s[t][qt] += far_bias;
+          } else {
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+              for (int r = 0; r < 4; ++r)
+                s[t][qt][r] = __builtin_fmaf(tb[max(0, min(d0 - 16 * t - r, a.far))], tb_scale, s[t][qt][r]);
+          }
+        }
+        if (!all_visible) {
+#pragma unroll
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const int d = d0 - 16 * t - r;
+              const bool ok = d >= 0 && (a.window <= 0 || d < a.window || qpos - d < a.keep);
+              s[t][qt][r] = ok ? s[t][qt][r] : -INFINITY;
+            }
+        }
+        float mx = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][qt][r]);
+        mx = max_xor32(max_xor16(mx));
+        alpha[qt] = 1.f;
+        if (mx > m_i[qt] + RESCALE_LOG2) {
+          alpha[qt] = m_i[qt] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_i[qt] - mx);
+          m_i[qt] = mx;
+        }
+        const float mref = m_i[qt] == -INFINITY ? 0.f : m_i[qt];
+        float ls = 0.f;
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float p = __builtin_amdgcn_exp2f(s[t][qt][r] - mref);
+            s[t][qt][r] = p;
+            ls += p;
+          }
+        l_i[qt] = l_i[qt] * alpha[qt] + ls;
+      }
+      if (__builtin_amdgcn_ballot_w64(alpha[0] != 1.f || alpha[1] != 1.f)) {
+#pragma unroll
+        for (int dt = 0; dt < CV::DT; ++dt)
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) o[dt][qt] *= alpha[qt];
+      }
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks) {
+        bf16x8 hi[2], lo[2];
+#pragma unroll
+        for (int qt = 0; qt < 2; ++qt) split_p(s[2 * ks][qt], s[2 * ks + 1][qt], hi[qt], lo[qt]);
+#pragma unroll
+        for (int dt = 0; dt < CV::DT; ++dt) {
+          const bf16x8 vf = load_vt<DV>(sV, dt, ks, lane);
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) {
+            o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[qt], o[dt][qt], 0, 0, 0);
+            o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[qt], o[dt][qt], 0, 0, 0);
+          }
+        }
+      }
+    }
+    wait_vmcnt0();
+    __syncthreads();
+  }
+
+#pragma unroll
+  for (int qt = 0; qt < 2; ++qt) {
+    float l = l_i[qt];
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    float inv = l > 0.f ? 1.f / l : 0.f;
+    const int qi = pbase + 16 * qt + fr;
+    if (qi < q_len) {
+      if (a.off_g >= 0) {
+        const float g = bf2f(((const bf16_t*)a.q)[(size_t)(q_off + qi) * a.ldq + a.off_g + hq]);
+        inv *= __builtin_amdgcn_rcpf(1.f + __expf(-g));
+      }
+      bf16_t* op = (bf16_t*)a.out + (size_t)(q_off + qi) * a.ldo + hq * DV + 4 * fh;
+#pragma unroll
+      for (int dt = 0; dt < CV::DT; ++dt) {
+        const f32x4 v = o[dt][qt] * inv;
+        *reinterpret_cast<uint2*>(op + 16 * dt) = make_uint2(pk2bf(v[0], v[1]), pk2bf(v[2], v[3]));
+      }
+    }
+  }
+}
+
+// ---- decode ----
+struct ShapedDecode {
+  const float* P; int S; int ldp; size_t slab;  // projection slabs [S][B][ldp]
+  const bf16_t* bias;                            // [ldp] or null
+  bf16_t* kc; bf16_t* vc;
+  const int* block_tables; int bt_stride;
+  const int* kv_lens; const int* slots;
+  const float* table;
+  const float* v_first; const float* lam;        // [B][G * DV] values to mix in, or null
+  float* v_own;                                  // [B][G * DV] own values out, or null
+  bf16_t* out; int ldo;
+  float* part_o; float* part_ml;                 // [B][H][max_parts][DV], [B][H][max_parts][2]
+  int B, H, G, off_k, off_v, off_g;
+  int window, keep, far, sink, min_tiles, max_parts;
+  float scale, softcap;
+};
+
+__device__ __forceinline__ void slab_row8(const ShapedDecode& a, int b, int col, float* f) {
+  sum_slabs8(a.P + (size_t)b * a.ldp + col, a.S, a.slab, f);
+  if (a.bias) {
+    float w[8];
+    ld8(a.bias + col, w);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] += w[e];
+  }
+}
+__device__ __forceinline__ float slab_gate(const ShapedDecode& a, int b, int h) {
+  if (a.off_g < 0) return 1.f;
+  float g = a.bias ? bf2f(a.bias[a.off_g + h]) : 0.f;
+  for (int s = 0; s < a.S; ++s) g += a.P[s * a.slab + (size_t)b * a.ldp + a.off_g + h];
+  return __builtin_amdgcn_rcpf(1.f + __expf(-g));
+}
+// pages per partition: the visited pages spread over all partitions, at least min_tiles each
+__device__ __forceinline__ int part_pages(int n, const ShapedDecode& a) {
+  return max(a.min_tiles, (n + a.max_parts - 1) / a.max_parts);
+}
+
+constexpr int DEC_HEADS = 16;  // query heads per decode block (one MFMA column each)
+
+// grid: (max_parts, KV heads x groups of 16 query heads, batch), 4 waves; a wave takes every 4th page
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_shaped_decode_kernel(ShapedDecode a) {
+  using CK = Cfg<DK>;
+  using CV = Cfg<DV>;
+  __shared__ __attribute__((aligned(16))) char smem[4 * CV::TILEB + DEC_HEADS * DK * 2 + 4 * (16 + 64) * 4];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int wid_u = __builtin_amdgcn_readfirstlane(wid);
+  const int part = blockIdx.x, b = blockIdx.z;
+  const int Gq = a.H / a.G, chunks = (Gq + DEC_HEADS - 1) / DEC_HEADS;
+  const int kvh = blockIdx.y / chunks, hc = blockIdx.y % chunks;
+  const int h0 = kvh * Gq + hc * DEC_HEADS, nh = min(DEC_HEADS, Gq - hc * DEC_HEADS);
+  const int pos = a.kv_lens[b] - 1;
+  const Pages pg = visited(pos, pos, a.window, a.keep);
+  const int pt = part_pages(pg.n, a);
+  const int it0 = part * pt;
+  if (it0 >= pg.n) return;  // block-uniform, before any barrier
+  const int it1 = min(it0 + pt, pg.n), nparts = (pg.n + pt - 1) / pt;
+  const int fr = lane & 15, fh = lane >> 4;
+  const int* bt = a.block_tables + (size_t)b * a.bt_stride;
+  char* sV = smem + wid_u * CV::TILEB;
+  bf16_t* s_q = reinterpret_cast<bf16_t*>(smem + 4 * CV::TILEB);
+
+  // the wave's first page is requested before the prologue (not the page that the new token goes into)
+  const bool pre = it0 + wid_u < it1 && it0 + wid_u != pg.n - 1;
+  bf16x8 kf[4][CK::KS];
+  auto request = [&](int it) {
+    const size_t pgi = (size_t)bt[pg.page(it)] * a.G + kvh;
+    const bf16_t* kb = a.kc + pgi * KT * DK;
+    const bf16_t* vb = a.vc + pgi * KT * DV;
+    stage_kv<DV, true, false, 1>(sV, 0, 1, lane, [&](int r) { return vb + (size_t)r * DV; });
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int s = 0; s < CK::KS; ++s)
+        kf[t][s] = *reinterpret_cast<const bf16x8*>(kb + (size_t)(16 * t + fr) * DK + 32 * s + 8 * fh);
+  };
+  if (pre) request(it0 + wid_u);
+
+  constexpr int QV = DK / 8, VV = DV / 8;
+  const bool append = it1 == pg.n;
+  const int n_q = nh * QV, n_all = n_q + (append ? QV + VV : 0);
+  for (int i = threadIdx.x; i < n_all; i += 256) {
+    float f[8];
+    if (i < n_q) {
+      slab_row8(a, b, h0 * DK + i * 8, f);
+      st8(s_q + i * 8, f);
+    } else {
+      const int slot = a.slots[b];
+      const size_t row = ((size_t)(slot >> 6) * a.G + kvh) * KT + (slot & 63);
+      const int j = i - n_q;
+      if (j < QV) {
+        slab_row8(a, b, a.off_k + kvh * DK + j * 8, f);
+        st8(a.kc + row * DK + j * 8, f);
+      } else {
+        const int c = (j - QV) * 8;
+        slab_row8(a, b, a.off_v + kvh * DV + c, f);
+        const size_t vo = ((size_t)b * a.G + kvh) * DV + c;
+        if (a.v_own) st8(a.v_own + vo, f);
+        if (a.v_first) {
+          const float lm = a.lam[0];
+          float w[8];
+          ld8(a.v_first + vo, w);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) f[e] = (1.f - lm) * f[e] + lm * w[e];
+        }
+        st8(a.vc + row * DV + c, f);
+      }
+    }
+  }
+  __syncthreads();  // q in LDS; the appended row visible to the whole block
+  bf16x8 qf[CK::KS];
+#pragma unroll
+  for (int s = 0; s < CK::KS; ++s)
+    qf[s] = fr < nh ? *reinterpret_cast<const bf16x8*>(s_q + fr * DK + 32 * s + 8 * fh) : (bf16x8){0, 0, 0, 0, 0, 0, 0, 0};
+
+  const Shape shape = make_shape(a.scale, a.softcap);
+  const float* tb = a.table ? a.table + (size_t)(h0 + min(fr, nh - 1)) * (a.far + 1) : nullptr;
+  f32x4 o[CV::DT];
+#pragma unroll
+  for (int dt = 0; dt < CV::DT; ++dt) o[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m_i = -INFINITY, l_i = 0.f;
+  for (int it = it0 + wid_u; it < it1; it += 4) {
+    if (!(pre && it == it0 + wid_u)) {
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the previous page's V reads have retired
+      request(it);
+    }
+    const int k0 = pg.page(it) * KT;
+    f32x4 s4[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      s4[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < CK::KS; ++s) s4[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[t][s], qf[s], s4[t], 0, 0, 0);
+    }
+    float mx = -INFINITY;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = k0 + 16 * t + 4 * fh + r, d = pos - j;
+        const bool ok = d >= 0 && (a.window <= 0 || d < a.window || j < a.keep);
+        float x = shape(s4[t][r]);
+        if (tb) x = __builtin_fmaf(tb[max(0, min(d, a.far))], LOG2E, x);
+        x = ok ? x : -INFINITY;
+        s4[t][r] = x;
+        mx = fmaxf(mx, x);
+      }
+    mx = max_xor32(max_xor16(mx));
+    const float m_new = fmaxf(m_i, mx), m_use = m_new == -INFINITY ? 0.f : m_new;
+    const float alpha = __builtin_amdgcn_exp2f(m_i - m_use);
+    float ls = 0.f;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = __builtin_amdgcn_exp2f(s4[t][r] - m_use);
+        s4[t][r] = p;
+        ls += p;
+      }
+    l_i = l_i * alpha + ls;
+    m_i = m_new;
+#pragma unroll
+    for (int dt = 0; dt < CV::DT; ++dt) o[dt] *= alpha;
+    bf16x8 hi[2], lo[2];
+    split_p(s4[0], s4[1], hi[0], lo[0]);
+    split_p(s4[2], s4[3], hi[1], lo[1]);
+    wait_vmcnt0();  // the V page is in this wave's LDS
+#pragma unroll
+    for (int dt = 0; dt < CV::DT; ++dt)
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks) {
+        const bf16x8 vf = load_vt<DV>(sV, dt, ks, lane);
+        o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[ks], o[dt], 0, 0, 0);
+        o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[ks], o[dt], 0, 0, 0);
+      }
+  }
+
+  // combine the 4 waves: O [4][16][DV] reuses the V pages, statistics sit behind the q rows
+  __syncthreads();
+  float* so = reinterpret_cast<float*>(smem);
+  float* sm = reinterpret_cast<float*>(smem + 4 * CV::TILEB + DEC_HEADS * DK * 2);
+  float* sl = sm + 64;
+  if (fh == 0) sm[wid * 16 + fr] = m_i;
+  sl[wid * 64 + lane] = l_i;
+#pragma unroll
+  for (int dt = 0; dt < CV::DT; ++dt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) so[(wid * 16 + fr) * DV + 16 * dt + 4 * fh + r] = o[dt][r];
+  __syncthreads();
+  for (int e = threadIdx.x; e < nh * DV; e += 256) {
+    const int g = e / DV, d = e % DV, h = h0 + g;
+    float M = nparts == 1 && a.sink ? 0.f : -INFINITY;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) M = fmaxf(M, sm[w * 16 + g]);
+    const float Mu = M == -INFINITY ? 0.f : M;
+    float L = nparts == 1 && a.sink ? __builtin_amdgcn_exp2f(-Mu) : 0.f, O = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float sc = __builtin_amdgcn_exp2f(sm[w * 16 + g] - Mu);
+      L += (sl[w * 64 + g] + sl[w * 64 + g + 16] + sl[w * 64 + g + 32] + sl[w * 64 + g + 48]) * sc;
+      O += so[(w * 16 + g) * DV + d] * sc;
+    }
+    if (nparts == 1) {
+      a.out[(size_t)b * a.ldo + h * DV + d] = f2bf(L > 0.f ? O / L * slab_gate(a, b, h) : 0.f);
+    } else {
+      const size_t pi = ((size_t)b * a.H + h) * a.max_parts + part;
+      a.part_o[pi * DV + d] = O;
+      if (d == 0) {
+        a.part_ml[pi * 2] = M;
+        a.part_ml[pi * 2 + 1] = L;
+      }
+    }
+  }
+}
+
+// join the partitions of one (head, sequence), add the extra zero score, apply the gate; DV threads
+__global__ void attn_shaped_merge_kernel(ShapedDecode a, int DV) {
+  const int h = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
+  const int pos = a.kv_lens[b] - 1;
+  const int n = visited(pos, pos, a.window, a.keep).n, pt = part_pages(n, a), nparts = (n + pt - 1) / pt;
+  if (nparts == 1) return;  // written by the decode kernel
+  const size_t p0 = ((size_t)b * a.H + h) * a.max_parts;
+  float M = a.sink ? 0.f : -INFINITY;
+  for (int p = 0; p < nparts; ++p) M = fmaxf(M, a.part_ml[(p0 + p) * 2]);
+  const float Mu = M == -INFINITY ? 0.f : M;
+  float L = a.sink ? __builtin_amdgcn_exp2f(-Mu) : 0.f, O = 0.f;
+  int p = 0;
+  for (; p + 4 <= nparts; p += 4) {
+    float v[4], m[4], l[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      v[i] = a.part_o[(p0 + p + i) * DV + d];
+      m[i] = a.part_ml[(p0 + p + i) * 2];
+      l[i] = a.part_ml[(p0 + p + i) * 2 + 1];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float sc = __builtin_amdgcn_exp2f(m[i] - Mu);
+      L += l[i] * sc;
+      O += v[i] * sc;
+    }
+  }
+  for (; p < nparts; ++p) {
+    const float sc = __builtin_amdgcn_exp2f(a.part_ml[(p0 + p) * 2] - Mu);
+    L += a.part_ml[(p0 + p) * 2 + 1] * sc;
+    O += a.part_o[(p0 + p) * DV + d] * sc;
+  }
+  a.out[(size_t)b * a.ldo + h * DV + d] = f2bf(L > 0.f ? O / L * slab_gate(a, b, h) : 0.f);
+}
+
+template <int DK, int DV>
+int launch_prefill(ShapedPrefill pa, int n_tiles, hipStream_t st) {
+  constexpr int base = 2 * (Cfg<DK>::TILEB + Cfg<DV>::TILEB) + MAX_BT * 4;
+  constexpr int room = ((DK <= 128 && DV <= 128) ? 80 * 1024 : 160 * 1024) - base;
+  int extra = pa.a.table ? pa.gb * (pa.a.far + 1) * 4 : 0;
+  if (extra > room) extra = 0;  // a very long table is read through the caches
+  pa.sb_stride = extra ? pa.a.far + 1 : 0;
+  const int lds = base + (extra + 15) / 16 * 16;
+  (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
+  return (int)hipGetLastError();
+}
+
+template <int DK, int DV>
+int launch_decode(const ShapedDecode& a, hipStream_t st) {
+  const int chunks = (a.H / a.G + DEC_HEADS - 1) / DEC_HEADS;
+  hipLaunchKernelGGL((attn_shaped_decode_kernel<DK, DV>), dim3(a.max_parts, a.G * chunks, a.B), dim3(256), 0, st, a);
+  if (a.max_parts > 1)
+    hipLaunchKernelGGL(attn_shaped_merge_kernel, dim3(a.H, a.B), dim3(DV), 0, st, a, DV);
+  return (int)hipGetLastError();
+}
+
+#define RAGK_SHAPED_DISPATCH(FN, ...)                                  \
+  do {                                                                 \
+    if (DK == 32 && DV == 32) return FN<32, 32>(__VA_ARGS__);          \
+    if (DK == 32 && DV == 64) return FN<32, 64>(__VA_ARGS__);          \
+    if (DK == 32 && DV == 128) return FN<32, 128>(__VA_ARGS__);        \
+    if (DK == 32 && DV == 256) return FN<32, 256>(__VA_ARGS__);        \
+    if (DK == 64 && DV == 32) return FN<64, 32>(__VA_ARGS__);          \
+    if (DK == 64 && DV == 64) return FN<64, 64>(__VA_ARGS__);          \
+    if (DK == 64 && DV == 128) return FN<64, 128>(__VA_ARGS__);        \
+    if (DK == 64 && DV == 256) return FN<64, 256>(__VA_ARGS__);        \
+    if (DK == 128 && DV == 32) return FN<128, 32>(__VA_ARGS__);        \
+    if (DK == 128 && DV == 64) return FN<128, 64>(__VA_ARGS__);        \
+    if (DK == 128 && DV == 128) return FN<128, 128>(__VA_ARGS__);      \
+    if (DK == 128 && DV == 256) return FN<128, 256>(__VA_ARGS__);      \
+    if (DK == 256 && DV == 32) return FN<256, 32>(__VA_ARGS__);        \
+    if (DK == 256 && DV == 64) return FN<256, 64>(__VA_ARGS__);        \
+    if (DK == 256 && DV == 128) return FN<256, 128>(__VA_ARGS__);      \
+    if (DK == 256 && DV == 256) return FN<256, 256>(__VA_ARGS__);      \
+    return (int)hipErrorInvalidValue;                                  \
+  } while (0)
+
 }  // namespace
+
+// bf16. tiles: [n_tiles][2] (sequence, first query) of 128 / gb query rows each; gb in {1, 2, 4} divides H / G.
+RAGK_API int ragk_shaped_attn_prefill(const void* q, int ldq, const void* kc, const void* vc, const int* block_tables,
+                                      int bt_stride, const int* cu_q, const int* kv_lens, const int* tiles, int n_tiles,
+                                      int gb, const float* table, void* out, int ldo, int H, int G, int DK, int DV,
+                                      int off_g, int window, int keep, int far, int sink, float scale, float softcap,
+                                      hipStream_t st) {
+  if (n_tiles <= 0) return 0;
+  if (H % G || (gb != 1 && gb != 2 && gb != 4) || (H / G) % gb || bt_stride > MAX_BT || ldq % 8 || ldo % 4 || !cu_q ||
+      window < 0 || keep < 0 || far < 0)
+    return (int)hipErrorInvalidValue;
+  const ShapedArgs a{q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, 0, 0, H, G, DK, DV,
+                     off_g, window, keep, far, sink, scale, softcap};
+  const ShapedPrefill pa{a, tiles, H / gb, gb, 0};
+  RAGK_SHAPED_DISPATCH(launch_prefill, pa, n_tiles, st);
+}
+
+// bf16 caches, fp32 slabs P [S][B][ldp] (+ bias). The new token's k / v go to `slots`; out [B][ldo].
+RAGK_API int ragk_shaped_attn_decode(const float* P, int S, int ldp, const void* bias, void* kc, void* vc,
+                                     const int* block_tables, int bt_stride, const int* kv_lens, const int* slots,
+                                     const float* table, const float* v_first, const float* lam, float* v_own, void* out,
+                                     int ldo, float* part_o, float* part_ml, int B, int H, int G, int DK, int DV,
+                                     int off_k, int off_v, int off_g, int window, int keep, int far, int sink,
+                                     int min_tiles, int max_parts, float scale, float softcap, hipStream_t st) {
+  if (B <= 0) return 0;
+  if (S < 1 || H % G || ldp % 8 || off_k % 8 || off_v % 8 || min_tiles < 1 || max_parts < 1 || (v_first && !lam) ||
+      (max_parts > 1 && (!part_o || !part_ml)) || B > 65535 || window < 0 || keep < 0 || far < 0)
+    return (int)hipErrorInvalidValue;
+  const ShapedDecode a{P, S, ldp, (size_t)B * ldp, (const bf16_t*)bias, (bf16_t*)kc, (bf16_t*)vc, block_tables, bt_stride,
+                       kv_lens, slots, table, v_first, lam, v_own, (bf16_t*)out, ldo, part_o, part_ml, B, H, G, off_k,
+                       off_v, off_g, window, keep, far, sink, min_tiles, max_parts, scale, softcap};
+  RAGK_SHAPED_DISPATCH(launch_decode, a, st);
+}
 
 // row: projection rows [T][ld] (fp32 when f32). v_first: [T][ldf] own values of the first mixing layer, or null.
 RAGK_API int ragk_shaped_kv_store(const void* row, int ld, int off_k, int off_v, int T, int G, int DK, int DV,

@@ -728,7 +728,8 @@ class LLMEngine:
         ids, pos, slots, kvl, states, bt = self._meta_views(packed, B)
         carry = packed[meta_n + 6 * B:meta_n + 7 * B]
         pt, mp, ws_o, ws_ml = m.decode_work(self.max_model_len, B)
-        meta = AttnMeta("decode", kvl, bt, part_tiles=pt, max_parts=mp, ws_o=ws_o, ws_ml=ws_ml, states=states)
+        meta = AttnMeta("decode", kvl, bt, part_tiles=pt, max_parts=mp, ws_o=ws_o, ws_ml=ws_ml, states=states,
+                        max_kv=self.max_model_len)
         temps, ks, ps, seeds, steps = self._sampling_views(packed[meta_n:meta_n + 6 * B], B)
         samp = dict(temps=temps, ks=ks, ps=ps, seeds=seeds, steps=steps)
         out_tok = self._tok_out[:B]

@@ -98,7 +98,12 @@ _SIGS = {
     "ragk_shaped_attn_rows": [P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, F, F, I, S],
     "ragk_ssm_conv": [P, P, P, I, I, P, I, I, P, P, P, P, I, I, I, S],
     "ragk_ssm_scan_seq": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, I, S],
-    "ragk_ssm_gate_norm": [P, P, I, P, P, I, I, I, I, F, I, S],
+    "ragk_shaped_attn_prefill": [P, I, P, P, P, I, P, P, P, I, I, P, P, I, I, I, I, I, I, I, I, I, I, F, F, S],
+    "ragk_shaped_attn_decode": [P, I, I, P, P, P, P, I, P, P, P, P, P, P, P, I, P, P, I, I, I, I, I, I, I, I, I, I, I, I,
+                                I, I, F, F, S],
+    "ragk_ssm_scan_chunk": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, S],
+    "ragk_ssm_decode": [P, I, I, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, S],
+    "ragk_ssm_gate_norm": [P, I, P, I, P, P, I, I, I, I, F, I, S],
     # csrc/comm/allreduce.hip (xGMI peer-mapped all-reduce)
     "ragk_ar_create": [I, I, ctypes.c_long, I, I, I],
     "ragk_ar_add_rmsnorm": [P, P, I, I, P, I, P, P, I, I, F, I, S],

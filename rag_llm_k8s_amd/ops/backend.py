@@ -40,6 +40,7 @@ class AttnMeta:
     host_q_lens: List[int] = field(default_factory=list)
     states: Optional[torch.Tensor] = None  # int32 [S] recurrent-state slot of every sequence
     qtiles: dict = field(default_factory=dict)  # prefill work lists by query-tile height (shaped attention)
+    max_kv: int = 0  # longest context the decode workspace was sized for (shaped attention)
 
 
 class TorchBackend:
@@ -424,9 +425,13 @@ class NativeBackend(TorchBackend):
         return self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
 
     def shaped_attn_prefill(self, row, spec, table, kc, vc, meta: AttnMeta, out):
-        return self.q.attn_rows(row, spec, table, kc, vc, meta, out)
+        if row.dtype == torch.float32:
+            return self.q.attn_rows(row, spec, table, kc, vc, meta, out)
+        return self.q.attn_prefill(row, spec, table, kc, vc, meta, out)
 
     def shaped_attn_decode(self, P, bias, spec, table, slots, kc, vc, meta: AttnMeta, out, v_first=None, lam=None):
+        if out.dtype == torch.bfloat16:
+            return self.q.attn_decode(P, bias, spec, table, slots, kc, vc, meta, out, v_first, lam)
         row = self.q.slab_rows(P, bias, out.dtype)
         own = self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
         self.q.attn_rows(row, spec, table, kc, vc, meta, out)
@@ -434,10 +439,16 @@ class NativeBackend(TorchBackend):
 
     def ssm_prefill(self, row, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
         xbc = self.q.ssm_conv(row, spec, w, meta, conv_state, ssm_state)
-        y = self.q.ssm_scan_seq(xbc, row, spec, w, meta, ssm_state)
+        if row.dtype == torch.bfloat16 and self.q.scan_chunk_ok(spec):
+            y = self.q.ssm_scan_chunk(xbc, row, spec, w, meta, ssm_state)
+        else:
+            y = self.q.ssm_scan_seq(xbc, row, spec, w, meta, ssm_state)
         return self.q.ssm_gate_norm(y, row, spec, w, eps, out)
 
     def ssm_decode(self, P, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
+        if out.dtype == torch.bfloat16 and self.q.ssm_decode_ok(spec):
+            yz = self.q.ssm_decode(P, spec, w, meta, conv_state, ssm_state)
+            return self.q.ssm_gate_norm(yz, None, spec, w, eps, out)
         return self.ssm_prefill(self.q.slab_rows(P, None, out.dtype), spec, w, eps, meta, conv_state, ssm_state, out)
 
     def attn_encoder(self, qkv, cu, lens_host, tiles, out, H, D):

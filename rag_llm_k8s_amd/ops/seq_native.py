@@ -104,8 +104,27 @@ def query_tiles(q_lens, qt):
     return torch.from_numpy(np.stack([seq[order], q0[order]], 1).astype(np.int32)).reshape(-1, 2)
 
 
+DECODE_TARGET_BLOCKS = 512  # decode attention grid: partitions x KV heads x batch
+DECODE_MIN_PAGES = 4
+
+
+def decode_parts(spec, max_kv_len, batch):
+    """Partitions per (sequence, KV head): the pages a query can visit, spread to fill the chip."""
+    pages = -(-max_kv_len // 64)
+    if spec.window > 0:
+        pages = min(pages, -(-spec.keep_first // 64) + -(-spec.window // 64) + 1)
+    rows = batch * spec.kv_heads * -(-spec.group // 16)
+    return max(1, min(-(-DECODE_TARGET_BLOCKS // rows), -(-pages // DECODE_MIN_PAGES)))
+
+
 def decode_split(specs, max_kv_len, batch, device):
-    return 1, 1, None, None
+    """(min pages per partition, 1, partition sums, partition statistics): one workspace all layers share."""
+    need = [(batch * s.heads * p, s.dvp) for s in specs for p in [decode_parts(s, max_kv_len, batch)] if p > 1]
+    if not need:
+        return DECODE_MIN_PAGES, 1, None, None
+    f32 = dict(dtype=F32, device=device)
+    return (DECODE_MIN_PAGES, 1, torch.empty(max(r * d for r, d in need), **f32),
+            torch.empty(max(r for r, _ in need) * 2, **f32))
 
 
 # ------------------------------------------------------------------------------------- shaped attention
@@ -168,6 +187,57 @@ def attn_rows(row, spec, table, kc, vc, meta, out):
     return out
 
 
+def attn_prefill(row, spec, table, kc, vc, meta, out):
+    """MFMA prefill attention over the pages (bf16)."""
+    T = row.shape[0]
+    _req(_act(row, "row") == 0, "bf16 rows")
+    S, cu = _meta(meta, T, False)
+    _caches(kc, vc, spec, row.dtype)
+    _table(table, spec)
+    tiles = meta.qtiles[spec.q_tile]
+    _req(tiles.dtype == I32 and tiles.is_cuda and tiles.is_contiguous(), "query tiles")
+    _req(out.dtype == row.dtype and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
+    _req(meta.block_tables.stride(0) <= 2048, "block tables wider than 2048 blocks (128k tokens)")
+    check(_lib.lib().ragk_shaped_attn_prefill(
+        row.data_ptr(), row.stride(0), kc.data_ptr(), vc.data_ptr(), meta.block_tables.data_ptr(),
+        meta.block_tables.stride(0), cu, meta.kv_lens.data_ptr(), tiles.data_ptr(), tiles.shape[0], spec.heads_per_block,
+        ptr(table), out.data_ptr(), out.stride(0), spec.heads, spec.kv_heads, spec.dkp, spec.dvp,
+        spec.off_g if spec.gate else -1, spec.window, spec.keep_first, spec.far, int(spec.sink), float(spec.scale),
+        float(spec.softcap), stream_ptr()), "ragk_shaped_attn_prefill")
+    return out
+
+
+def attn_decode(P, bias, spec, table, slots, kc, vc, meta, out, v_first=None, lam=None):
+    """One new token per sequence from projection slabs (bf16 caches): value mix, cache append, attention, gate.
+    Returns the tokens' own values [B, kv_heads * dv] (fp32)."""
+    S, B, N = P.shape
+    _req(P.is_cuda and P.dtype == F32 and P.is_contiguous() and N >= spec.off_g + (spec.heads if spec.gate else 0), "slabs")
+    _meta(meta, B, True)
+    _caches(kc, vc, spec, BF16)
+    _table(table, spec)
+    _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == B, "slots int32[B]")
+    _req(out.dtype == BF16 and out.shape == (B, spec.out_row) and out.is_contiguous(), "out rows")
+    if bias is not None:
+        _vec(bias, N, BF16, "bias")
+    nv = spec.kv_heads * spec.dvp
+    if v_first is not None:
+        _req(v_first.dtype == F32 and v_first.shape == (B, nv) and v_first.is_contiguous(), "v_first fp32 [B, values]")
+        _vec(lam, 1, F32, "lam")
+    own = torch.empty((B, nv), dtype=F32, device=P.device)
+    parts = decode_parts(spec, meta.max_kv, B) if meta.ws_o is not None else 1
+    if parts > 1:
+        _req(meta.ws_o.numel() >= B * spec.heads * parts * spec.dvp and meta.ws_ml.numel() >= B * spec.heads * parts * 2,
+             "decode workspace too small")
+    check(_lib.lib().ragk_shaped_attn_decode(
+        P.data_ptr(), S, N, ptr(bias), kc.data_ptr(), vc.data_ptr(), meta.block_tables.data_ptr(),
+        meta.block_tables.stride(0), meta.kv_lens.data_ptr(), slots.data_ptr(), ptr(table), ptr(v_first),
+        ptr(lam) if v_first is not None else None, own.data_ptr(), out.data_ptr(), out.stride(0), ptr(meta.ws_o),
+        ptr(meta.ws_ml), B, spec.heads, spec.kv_heads, spec.dkp, spec.dvp, spec.off_k, spec.off_v,
+        spec.off_g if spec.gate else -1, spec.window, spec.keep_first, spec.far, int(spec.sink), DECODE_MIN_PAGES, parts,
+        float(spec.scale), float(spec.softcap), stream_ptr()), "ragk_shaped_attn_decode")
+    return own
+
+
 # ------------------------------------------------------------------------------------- state space
 def _states(meta, spec, conv_state, ssm_state):
     n = ssm_state.shape[0]
@@ -207,13 +277,62 @@ def ssm_scan_seq(xbc, row, spec, w, meta, ssm_state):
     return y
 
 
-def ssm_gate_norm(y, row, spec, w, eps, out):
-    f32 = _act(row, "row")
+def scan_chunk_ok(spec):
+    return spec.vdim % 8 == 0 and spec.state % 8 == 0 and spec.state <= 256
+
+
+def ssm_scan_chunk(xbc, row, spec, w, meta, ssm_state):
+    """MFMA chunked scan of packed prompts (bf16)."""
+    _req(_act(row, "row") == 0 and xbc.dtype == BF16 and xbc.is_contiguous() and scan_chunk_ok(spec), "chunk scan operands")
     T = row.shape[0]
-    _req(y.dtype == F32 and y.is_contiguous() and y.shape == (T, spec.inner), "y fp32 [T, inner]")
-    _req(out.dtype == row.dtype and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
+    S, cu = _meta(meta, T, meta.kind == "decode")
+    _req(xbc.shape == (T, spec.channels), "xbc rows")
+    for k in ("dt_bias", "A", "D"):
+        _vec(w[k], spec.heads, F32, k)
+    y = torch.empty((T, spec.inner), dtype=BF16, device=row.device)
+    check(_lib.lib().ragk_ssm_scan_chunk(cu, meta.kv_lens.data_ptr(), meta.states.data_ptr(), T, S, xbc.data_ptr(),
+                                         xbc.stride(0), row.data_ptr(), row.stride(0), spec.off_dt, w["dt_bias"].data_ptr(),
+                                         w["A"].data_ptr(), w["D"].data_ptr(), ssm_state.data_ptr(), y.data_ptr(),
+                                         spec.heads, spec.vdim, spec.state, spec.groups, stream_ptr()),
+          "ragk_ssm_scan_chunk")
+    return y
+
+
+def ssm_decode_ok(spec):
+    return spec.vdim % 4 == 0 and spec.vdim <= 256 and spec.state % 4 == 0
+
+
+def ssm_decode(P, spec, w, meta, conv_state, ssm_state):
+    """One token per sequence from projection slabs: convolution, state update, gate. Returns y * silu(z), fp32."""
+    S, B, N = P.shape
+    _req(P.is_cuda and P.dtype == F32 and P.is_contiguous() and N >= spec.off_dt + spec.heads and ssm_decode_ok(spec),
+         "slabs")
+    _meta(meta, B, True)
+    _states(meta, spec, conv_state, ssm_state)
+    _vec(w["conv_w"].reshape(-1), spec.taps * spec.channels, F32, "conv_w")
+    _vec(w["conv_b"], spec.channels, F32, "conv_b")
+    for k in ("dt_bias", "A", "D"):
+        _vec(w[k], spec.heads, F32, k)
+    act = torch.empty((B, N), dtype=F32, device=P.device)
+    yz = torch.empty((B, spec.inner), dtype=F32, device=P.device)
+    check(_lib.lib().ragk_ssm_decode(P.data_ptr(), S, N, meta.kv_lens.data_ptr(), meta.states.data_ptr(),
+                                     w["conv_w"].data_ptr(), w["conv_b"].data_ptr(), w["dt_bias"].data_ptr(),
+                                     w["A"].data_ptr(), w["D"].data_ptr(), conv_state.data_ptr(), ssm_state.data_ptr(),
+                                     act.data_ptr(), yz.data_ptr(), B, spec.heads, spec.vdim, spec.state, spec.groups,
+                                     spec.taps, stream_ptr()), "ragk_ssm_decode")
+    return yz
+
+
+def ssm_gate_norm(y, row, spec, w, eps, out):
+    """group_norm(y * silu(z)) * w; z = row[:, :inner], or None when y is gated already."""
+    f32 = int(out.dtype == F32)
+    T = y.shape[0]
+    _req(y.dtype in (BF16, F32) and y.is_contiguous() and y.shape == (T, spec.inner), "y [T, inner]")
+    if row is not None:
+        _req(row.dtype == out.dtype and row.shape[0] == T and row.stride(1) == 1, "projection rows")
+    _req(out.is_cuda and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
     _vec(w["norm"], spec.inner, F32, "norm")
-    check(_lib.lib().ragk_ssm_gate_norm(y.data_ptr(), row.data_ptr(), row.stride(0), w["norm"].data_ptr(), out.data_ptr(),
-                                        out.stride(0), T, spec.inner, spec.norm_groups, float(eps), f32, stream_ptr()),
-          "ragk_ssm_gate_norm")
+    check(_lib.lib().ragk_ssm_gate_norm(y.data_ptr(), int(y.dtype == BF16), ptr(row), row.stride(0) if row is not None else 0,
+                                        w["norm"].data_ptr(), out.data_ptr(), out.stride(0), T, spec.inner,
+                                        spec.norm_groups, float(eps), f32, stream_ptr()), "ragk_ssm_gate_norm")
     return out

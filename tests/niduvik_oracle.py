@@ -64,27 +64,36 @@ def sink_softmax(s, mask):
     return e / (torch.exp(-m) + e.sum(-1, keepdim=True))
 
 
+def attention_core(q, k, v, gate_logits, rel, scale, softcap, far, size, keep):
+    """q [T,H,dk], k [T,G,dk], v [T,G,dv], gate logits [T,H] -> [T,H,dv]."""
+    T, H = q.shape[:2]
+    G = k.shape[1]
+    bias = distance_bias(rel, far, T)
+    mask = visible(T, size, keep)
+    gate = 1 / (1 + torch.exp(-gate_logits))
+    out = torch.zeros(T, H, v.shape[2], dtype=q.dtype)
+    for h in range(H):
+        g = h // (H // G)
+        s = (q[:, h] @ k[:, g].T) * scale
+        s = softcap * torch.tanh(s / softcap) + bias[:, :, h]
+        out[:, h] = sink_softmax(s, mask) @ v[:, g] * gate[:, h:h + 1]
+    return out
+
+
+def mix_values(v, v_first, lam):
+    return (1 - lam) * v + lam * v_first
+
+
 def attention(h, W, p, c, v_first):
     """Returns (output [T, width], this layer's own values [T, kv_heads * vdim])."""
     T = h.shape[0]
     H, G, dk, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
     q = h @ W[p + "q"].T + W[p + "q.b"]
     k = h @ W[p + "k"].T + W[p + "k.b"]
-    v = h @ W[p + "v"].T + W[p + "v.b"]
-    own = v
-    if v_first is not None:
-        lam = W[p + "vmix"]
-        v = (1 - lam) * v + lam * v_first
-    q, k, v = q.reshape(T, H, dk), k.reshape(T, G, dk), v.reshape(T, G, dv)
-    bias = distance_bias(W[p + "rel"], c["bias_max"], T)
-    mask = visible(T, c["mask"]["size"], c["mask"]["keep_first"])
-    gate = 1 / (1 + torch.exp(-(h @ W[p + "g"].T)))
-    out = torch.zeros(T, H, dv, dtype=h.dtype)
-    for hh in range(H):
-        g = hh // (H // G)
-        s = (q[:, hh] @ k[:, g].T) * c["scale"]
-        s = c["softcap"] * torch.tanh(s / c["softcap"]) + bias[:, :, hh]
-        out[:, hh] = sink_softmax(s, mask) @ v[:, g] * gate[:, hh:hh + 1]
+    own = h @ W[p + "v"].T + W[p + "v.b"]
+    v = own if v_first is None else mix_values(own, v_first, W[p + "vmix"])
+    out = attention_core(q.reshape(T, H, dk), k.reshape(T, G, dk), v.reshape(T, G, dv), h @ W[p + "g"].T, W[p + "rel"],
+                         c["scale"], c["softcap"], c["bias_max"], c["mask"]["size"], c["mask"]["keep_first"])
     return out.reshape(T, H * dv) @ W[p + "o"].T, own
 
 

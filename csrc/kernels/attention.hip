@@ -397,18 +397,6 @@ __device__ __forceinline__ void pin_s(int& x) { asm volatile("" : "+s"(x)); }
 // The asm MFMAs are opaque to the compiler's hazard recognizer: a VALU read of an MFMA result needs
 // the XDL-write -> VALU-read wait states (18 for a 16-pass op), and a VALU write read by an MFMA a few.
 __device__ __forceinline__ void mfma_result_wait() {}
-// LDS-DMA piece as inline asm: the compiler's waitcnt pass cannot tell which LDS bytes a
-// buffer_load ... lds intrinsic writes, so it drained vmcnt(0) before the next ds_read of ANY slot
-// (an HBM round trip per fragment read). The kernel orders its slots itself (vmcnt + barrier per
-// iteration) and issues every LDS-DMA of the kernel through this, so M0 is never live for the compiler.
-__device__ __forceinline__ void blds16_asm(i32x4 srd, int voff, int soff, unsigned lds_addr) {
-  asm volatile("s_mov_b32 m0, %0\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds" ::"s"(lds_addr), "v"(voff), "s"(srd),
-               "s"(soff));
-}
-__device__ __forceinline__ unsigned lds_addr(const void* p) {
-  return (unsigned)(unsigned long long)(const __attribute__((address_space(3))) char*)p;
-}
-
 // NW = 8: two groups of 4 waves (query rows q_start + [0, 32) and + [32, 64)) share every K / V tile,
 // so each SIMD runs two of these streams and one wave's dependency stalls are the other's issue slots.
 // DIAG (stamp builds only, wrong results): 1 = no softmax chunks in the fast slots, 2 = no fragment reads

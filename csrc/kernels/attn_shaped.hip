@@ -151,11 +151,15 @@ __device__ __forceinline__ Pages visited(int qmin, int qmax, int window, int kee
 // softcapped score in log2 units: cap2 * tanh(x / cap) = cap2 - 2 cap2 / (1 + 2^(x * c1)); c1 = 2 scale log2e / cap
 struct Shape {
   float c1, cap2, c;  // cap2 > 0: soft-capped; else s = x * c
-  __device__ __forceinline__ float operator()(float x) const {
-    if (cap2 > 0.f) return __builtin_fmaf(-2.f * cap2, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * c1)), cap2);
-    return x * c;
+  __device__ __forceinline__ float sigma(float x) const {  // 1 / (1 + 2^(x * c1))
+    return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * c1));
   }
 };
+// tanh(y) / y as a polynomial in y^2, |error of tanh| < 1.4e-7 for |y| <= TANH_R (least-maximum fit): cheaper than the
+// exponential and the reciprocal, which on this ALU take four issue slots each
+constexpr float TANH_R = 0.5f;
+constexpr float TANH_C[4] = {0.999997676f, -0.333206551f, 0.131451449f, -0.0433724665f};
+
 constexpr float LOG2E = 1.4426950408889634f;
 __device__ __forceinline__ Shape make_shape(float scale, float softcap) {
   return Shape{softcap > 0.f ? 2.f * scale * LOG2E / softcap : 0.f, softcap > 0.f ? softcap * LOG2E : 0.f, scale * LOG2E};
@@ -181,7 +185,9 @@ struct ShapedPrefill {
   int sb_stride;                   // floats per head of the LDS bias table, 0: none
 };
 
-template <int DK, int DV>
+// BOUNDED: every score is known to stay within a range whose exponentials fp32 holds (soft cap + largest bias), so
+// the sums need no running maximum: the weights are 2^s, and the extra zero score adds exactly 1.
+template <int DK, int DV, bool BOUNDED>
 __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_shaped_prefill_kernel(ShapedPrefill pa) {
   using CK = Cfg<DK>;
   using CV = Cfg<DV>;
@@ -231,18 +237,40 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
       for (int i = threadIdx.x; i <= a.far; i += 256)
         s_bias[h * pa.sb_stride + i] = a.table[(size_t)(h0 + h) * (a.far + 1) + i] * LOG2E;
   __syncthreads();
-  const float* tb = a.table ? (pa.sb_stride ? s_bias + hb * pa.sb_stride : a.table + (size_t)hq * (a.far + 1)) : nullptr;
-  const float tb_scale = pa.sb_stride ? 1.f : LOG2E;
-  const float far_bias = tb ? tb[a.far] * tb_scale : 0.f;
+  const float* tb = a.table ? a.table + (size_t)hq * (a.far + 1) : nullptr;
+  const float* s_tb = s_bias + hb * pa.sb_stride;  // the same row in LDS, in log2 units
+  const float far_bias = tb ? tb[a.far] * LOG2E : 0.f;
   const Shape shape = make_shape(a.scale, a.softcap);
+  const bool capped = shape.cap2 > 0.f;
+  const int win = a.window > 0 ? a.window : 0x7fffffff;
+  // the polynomial in the raw product x: s = x (q0 + x^2 (q1 + ...)), good while |x| <= x_lim
+  const float yx = capped ? a.scale / a.softcap : 0.f, yx2 = yx * yx, x_lim = capped ? TANH_R / yx : 0.f;
+  const float q0 = shape.cap2 * yx * TANH_C[0], q1 = shape.cap2 * yx * yx2 * TANH_C[1];
+  const float q2 = shape.cap2 * yx * yx2 * yx2 * TANH_C[2], q3 = shape.cap2 * yx * yx2 * yx2 * yx2 * TANH_C[3];
 
+  // a page's rows by LDS-DMA, each wave a quarter of the 1-KiB pieces; per-lane source offsets are fixed
+  constexpr int KP = CK::PIECES / 4, VP = CV::PIECES / 4;
+  int koff[KP], voff[VP];
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int row = (wid_u + 4 * i) * CK::RPP + lane / CK::NC, ph = lane % CK::NC;
+    koff[i] = row * CK::ROWB + 16 * (ph ^ kswz<DK>(row));
+  }
+#pragma unroll
+  for (int i = 0; i < VP; ++i) {
+    const int row = (wid_u + 4 * i) * CV::RPP + lane / CV::NC, ph = lane % CV::NC;
+    voff[i] = row * CV::ROWB + 16 * (ph ^ vswz<DV>(row));
+  }
+  const unsigned lds0 = lds_addr(smem);
   auto stage = [&](int it, int buf) {
-    char* sK = smem + buf * (CK::TILEB + CV::TILEB);
-    const size_t pgi = (size_t)s_bt[it] * a.G + kvh;
-    const bf16_t* kb = (const bf16_t*)a.kc + pgi * KT * DK;
-    const bf16_t* vb = (const bf16_t*)a.vc + pgi * KT * DV;
-    stage_kv<DK, false, false, 4>(sK, wid_u, 4, lane, [&](int r) { return kb + (size_t)r * DK; });
-    stage_kv<DV, true, false, 4>(sK + CK::TILEB, wid_u, 4, lane, [&](int r) { return vb + (size_t)r * DV; });
+    const size_t pgi = (size_t)__builtin_amdgcn_readfirstlane(s_bt[it]) * a.G + kvh;
+    const i32x4 srd_k = make_srd((const bf16_t*)a.kc + pgi * KT * DK, CK::TILEB);
+    const i32x4 srd_v = make_srd((const bf16_t*)a.vc + pgi * KT * DV, CV::TILEB);
+    const unsigned l = lds0 + buf * (CK::TILEB + CV::TILEB);
+#pragma unroll
+    for (int i = 0; i < KP; ++i) blds16_asm(srd_k, koff[i], 0, l + (wid_u + 4 * i) * 1024);
+#pragma unroll
+    for (int i = 0; i < VP; ++i) blds16_asm(srd_v, voff[i], 0, l + CK::TILEB + (wid_u + 4 * i) * 1024);
   };
   stage(0, 0);  // pg.n >= 1: a query always sees its own page
   wait_vmcnt0();
@@ -252,7 +280,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     const int cur = it & 1, k0 = pg.page(it) * KT;
     const char* sK = smem + cur * (CK::TILEB + CV::TILEB);
     const char* sV = sK + CK::TILEB;
-    const bool active = k0 <= wave_pmax && (a.window <= 0 || wave_pmin - (k0 + KT - 1) < a.window || k0 < a.keep);
+    const bool active = k0 <= wave_pmax && (wave_pmin - (k0 + KT - 1) < win || k0 < a.keep);
     f32x4 s[4][2];
     if (active) {
 #pragma unroll
@@ -269,67 +297,121 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     }
     if (it + 1 < pg.n) stage(it + 1, cur ^ 1);  // DMA of the next page behind the QK^T products
     if (active) {
-      const bool all_visible = k0 + KT - 1 <= wave_pmin && (a.window <= 0 || wave_pmax - k0 < a.window || k0 + KT <= a.keep);
-      const bool far_only = wave_pmin - (k0 + KT - 1) >= a.far;  // one bias for the whole page
-      float alpha[2];
+      const bool all_visible = k0 + KT - 1 <= wave_pmin && (wave_pmax - k0 < win || k0 + KT <= a.keep);
+      const bool far_only = !tb || wave_pmin - (k0 + KT - 1) >= a.far;  // one bias for the whole page
+      // scores in log2 units, with the page-wide bias; wave-uniform branches around whole pages of elements
+      const float base = far_only ? far_bias : 0.f;
 #pragma unroll
       for (int qt = 0; qt < 2; ++qt) {
-        const int qpos = ctx0 + pbase + 16 * qt + fr;
-        const int d0 = qpos - k0 - 4 * fh;  // distance of this lane's key 0
+        if (capped) {
+          float ax = 0.f;
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
+          for (int t = 0; t < 4; ++t)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) s[t][qt][r] = shape(s[t][qt][r]);
-        if (tb) {
-          if (far_only) {
+            for (int r = 0; r < 4; ++r) ax = fmaxf(ax, fabsf(s[t][qt][r]));
+          if (!__builtin_amdgcn_ballot_w64(!(ax <= x_lim))) {
 #pragma unroll
-            for (int t = 0; t < 4; ++t) s[t][qt] += far_bias;
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+              for (int r = 0; r < 4; ++r) {
+                const float x = s[t][qt][r], z = x * x;
+                const float q = __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, q3, q2), q1), q0);
+                s[t][qt][r] = __builtin_fmaf(x, q, base);
+              }
           } else {
 #pragma unroll
             for (int t = 0; t < 4; ++t)
 #pragma unroll
               for (int r = 0; r < 4; ++r)
-                s[t][qt][r] = __builtin_fmaf(tb[max(0, min(d0 - 16 * t - r, a.far))], tb_scale, s[t][qt][r]);
+                s[t][qt][r] = __builtin_fmaf(-2.f * shape.cap2, shape.sigma(s[t][qt][r]), base + shape.cap2);
+          }
+        } else {
+#pragma unroll
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s[t][qt][r] = __builtin_fmaf(s[t][qt][r], shape.c, base);
+        }
+      }
+      if (!far_only) {
+        if (pa.sb_stride) {
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) {
+            const int d0 = ctx0 + pbase + 16 * qt + fr - k0 - 4 * fh;  // distance of this lane's key 0
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+              for (int r = 0; r < 4; ++r) s[t][qt][r] += s_tb[max(0, min(d0 - 16 * t - r, a.far))];
+          }
+        } else {
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) {
+            const int d0 = ctx0 + pbase + 16 * qt + fr - k0 - 4 * fh;
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+              for (int r = 0; r < 4; ++r)
+                s[t][qt][r] = __builtin_fmaf(tb[max(0, min(d0 - 16 * t - r, a.far))], LOG2E, s[t][qt][r]);
           }
         }
-        if (!all_visible) {
+      }
+      if (!all_visible) {
+#pragma unroll
+        for (int qt = 0; qt < 2; ++qt) {
+          const int qpos = ctx0 + pbase + 16 * qt + fr, d0 = qpos - k0 - 4 * fh;
 #pragma unroll
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int d = d0 - 16 * t - r;
-              const bool ok = d >= 0 && (a.window <= 0 || d < a.window || qpos - d < a.keep);
+              const bool ok = (d >= 0) & ((d < win) | (qpos - d < a.keep));
               s[t][qt][r] = ok ? s[t][qt][r] : -INFINITY;
             }
         }
-        float mx = -INFINITY;
-#pragma unroll
-        for (int t = 0; t < 4; ++t)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][qt][r]);
-        mx = max_xor32(max_xor16(mx));
-        alpha[qt] = 1.f;
-        if (mx > m_i[qt] + RESCALE_LOG2) {
-          alpha[qt] = m_i[qt] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_i[qt] - mx);
-          m_i[qt] = mx;
-        }
-        const float mref = m_i[qt] == -INFINITY ? 0.f : m_i[qt];
-        float ls = 0.f;
-#pragma unroll
-        for (int t = 0; t < 4; ++t)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const float p = __builtin_amdgcn_exp2f(s[t][qt][r] - mref);
-            s[t][qt][r] = p;
-            ls += p;
-          }
-        l_i[qt] = l_i[qt] * alpha[qt] + ls;
       }
-      if (__builtin_amdgcn_ballot_w64(alpha[0] != 1.f || alpha[1] != 1.f)) {
+      if constexpr (BOUNDED) {
 #pragma unroll
-        for (int dt = 0; dt < CV::DT; ++dt)
+        for (int qt = 0; qt < 2; ++qt)
 #pragma unroll
-          for (int qt = 0; qt < 2; ++qt) o[dt][qt] *= alpha[qt];
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const float p = __builtin_amdgcn_exp2f(s[t][qt][r]);
+              s[t][qt][r] = p;
+              l_i[qt] += p;
+            }
+      } else {
+        float alpha[2];
+#pragma unroll
+        for (int qt = 0; qt < 2; ++qt) {
+          float mx = -INFINITY;
+#pragma unroll
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][qt][r]);
+          mx = max_xor32(max_xor16(mx));
+          alpha[qt] = 1.f;
+          if (mx > m_i[qt] + RESCALE_LOG2) {
+            alpha[qt] = m_i[qt] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_i[qt] - mx);
+            m_i[qt] = mx;
+          }
+          const float mref = m_i[qt] == -INFINITY ? 0.f : m_i[qt];
+          float ls = 0.f;
+#pragma unroll
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const float p = __builtin_amdgcn_exp2f(s[t][qt][r] - mref);
+              s[t][qt][r] = p;
+              ls += p;
+            }
+          l_i[qt] = l_i[qt] * alpha[qt] + ls;
+        }
+        if (__builtin_amdgcn_ballot_w64(alpha[0] != 1.f || alpha[1] != 1.f)) {
+#pragma unroll
+          for (int dt = 0; dt < CV::DT; ++dt)
+#pragma unroll
+            for (int qt = 0; qt < 2; ++qt) o[dt][qt] *= alpha[qt];
+        }
       }
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
@@ -442,12 +524,13 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     const size_t pgi = (size_t)bt[pg.page(it)] * a.G + kvh;
     const bf16_t* kb = a.kc + pgi * KT * DK;
     const bf16_t* vb = a.vc + pgi * KT * DV;
-    stage_kv<DV, true, false, 1>(sV, 0, 1, lane, [&](int r) { return vb + (size_t)r * DV; });
 #pragma unroll
     for (int t = 0; t < 4; ++t)
 #pragma unroll
       for (int s = 0; s < CK::KS; ++s)
         kf[t][s] = *reinterpret_cast<const bf16x8*>(kb + (size_t)(16 * t + fr) * DK + 32 * s + 8 * fh);
+    __builtin_amdgcn_sched_barrier(0);  // K before V: the scores and the softmax run while V is landing
+    stage_kv<DV, true, false, 1>(sV, 0, 1, lane, [&](int r) { return vb + (size_t)r * DV; });
   };
   if (pre) request(it0 + wid_u);
 
@@ -490,6 +573,9 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
 
   const Shape shape = make_shape(a.scale, a.softcap);
   const float* tb = a.table ? a.table + (size_t)(h0 + min(fr, nh - 1)) * (a.far + 1) : nullptr;
+  const float far_bias = tb ? tb[a.far] * LOG2E : 0.f;
+  const bool capped = shape.cap2 > 0.f;
+  const int win = a.window > 0 ? a.window : 0x7fffffff;
   f32x4 o[CV::DT];
 #pragma unroll
   for (int dt = 0; dt < CV::DT; ++dt) o[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -507,19 +593,42 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
 #pragma unroll
       for (int s = 0; s < CK::KS; ++s) s4[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[t][s], qf[s], s4[t], 0, 0, 0);
     }
+    const int d0 = pos - k0 - 4 * fh;  // distance of this lane's key 0
+    const bool far_only = !tb || pos - (k0 + KT - 1) >= a.far;
+    const float base = (capped ? shape.cap2 : 0.f) + (far_only ? far_bias : 0.f);
+    if (capped) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s4[t][r] = __builtin_fmaf(-2.f * shape.cap2, shape.sigma(s4[t][r]), base);
+    } else {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s4[t][r] = __builtin_fmaf(s4[t][r], shape.c, base);
+    }
+    if (!far_only) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          s4[t][r] = __builtin_fmaf(tb[max(0, min(d0 - 16 * t - r, a.far))], LOG2E, s4[t][r]);
+    }
+    if (!(k0 + KT - 1 <= pos && (pos - k0 < win || k0 + KT <= a.keep))) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int d = d0 - 16 * t - r;
+          const bool ok = (d >= 0) & ((d < win) | (pos - d < a.keep));
+          s4[t][r] = ok ? s4[t][r] : -INFINITY;
+        }
+    }
     float mx = -INFINITY;
 #pragma unroll
     for (int t = 0; t < 4; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int j = k0 + 16 * t + 4 * fh + r, d = pos - j;
-        const bool ok = d >= 0 && (a.window <= 0 || d < a.window || j < a.keep);
-        float x = shape(s4[t][r]);
-        if (tb) x = __builtin_fmaf(tb[max(0, min(d, a.far))], LOG2E, x);
-        x = ok ? x : -INFINITY;
-        s4[t][r] = x;
-        mx = fmaxf(mx, x);
-      }
+      for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s4[t][r]);
     mx = max_xor32(max_xor16(mx));
     const float m_new = fmaxf(m_i, mx), m_use = m_new == -INFINITY ? 0.f : m_new;
     const float alpha = __builtin_amdgcn_exp2f(m_i - m_use);
@@ -624,15 +733,22 @@ __global__ void attn_shaped_merge_kernel(ShapedDecode a, int DV) {
 }
 
 template <int DK, int DV>
-int launch_prefill(ShapedPrefill pa, int n_tiles, hipStream_t st) {
+int launch_prefill(ShapedPrefill pa, int n_tiles, int bounded, hipStream_t st) {
   constexpr int base = 2 * (Cfg<DK>::TILEB + Cfg<DV>::TILEB) + MAX_BT * 4;
   constexpr int room = ((DK <= 128 && DV <= 128) ? 80 * 1024 : 160 * 1024) - base;
   int extra = pa.a.table ? pa.gb * (pa.a.far + 1) * 4 : 0;
   if (extra > room) extra = 0;  // a very long table is read through the caches
   pa.sb_stride = extra ? pa.a.far + 1 : 0;
   const int lds = base + (extra + 15) / 16 * 16;
-  (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
+  if (bounded) {
+    (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV, true>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV, true>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
+  } else {
+    (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV, false>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV, false>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
+  }
   return (int)hipGetLastError();
 }
 
@@ -669,19 +785,20 @@ int launch_decode(const ShapedDecode& a, hipStream_t st) {
 }  // namespace
 
 // bf16. tiles: [n_tiles][2] (sequence, first query) of 128 / gb query rows each; gb in {1, 2, 4} divides H / G.
+// bounded: the caller knows that (softcap + largest |bias|) * log2e < 80 (every 2^score and the sum over any context fit).
 RAGK_API int ragk_shaped_attn_prefill(const void* q, int ldq, const void* kc, const void* vc, const int* block_tables,
                                       int bt_stride, const int* cu_q, const int* kv_lens, const int* tiles, int n_tiles,
                                       int gb, const float* table, void* out, int ldo, int H, int G, int DK, int DV,
-                                      int off_g, int window, int keep, int far, int sink, float scale, float softcap,
-                                      hipStream_t st) {
+                                      int off_g, int window, int keep, int far, int sink, int bounded, float scale,
+                                      float softcap, hipStream_t st) {
   if (n_tiles <= 0) return 0;
   if (H % G || (gb != 1 && gb != 2 && gb != 4) || (H / G) % gb || bt_stride > MAX_BT || ldq % 8 || ldo % 4 || !cu_q ||
-      window < 0 || keep < 0 || far < 0)
+      window < 0 || keep < 0 || far < 0 || (bounded && !(softcap > 0.f)))
     return (int)hipErrorInvalidValue;
   const ShapedArgs a{q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, 0, 0, H, G, DK, DV,
                      off_g, window, keep, far, sink, scale, softcap};
   const ShapedPrefill pa{a, tiles, H / gb, gb, 0};
-  RAGK_SHAPED_DISPATCH(launch_prefill, pa, n_tiles, st);
+  RAGK_SHAPED_DISPATCH(launch_prefill, pa, n_tiles, bounded, st);
 }
 
 // bf16 caches, fp32 slabs P [S][B][ldp] (+ bias). The new token's k / v go to `slots`; out [B][ldo].

@@ -96,4 +96,16 @@ __device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
                   f2bf_s(b[0]), f2bf_s(b[1]), f2bf_s(b[2]), f2bf_s(b[3])};
 }
 
+// LDS-DMA piece as inline asm: the compiler's waitcnt pass cannot tell which LDS bytes a
+// buffer_load ... lds intrinsic writes, so it drained vmcnt(0) before the next ds_read of ANY slot
+// (an HBM round trip per fragment read). A kernel that uses this orders its slots itself (vmcnt + barrier per
+// iteration) and issues every LDS-DMA through it, so M0 is never live for the compiler.
+__device__ __forceinline__ void blds16_asm(i32x4 srd, int voff, int soff, unsigned lds_addr) {
+  asm volatile("s_mov_b32 m0, %0\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds" ::"s"(lds_addr), "v"(voff), "s"(srd),
+               "s"(soff));
+}
+__device__ __forceinline__ unsigned lds_addr(const void* p) {
+  return (unsigned)(unsigned long long)(const __attribute__((address_space(3))) char*)p;
+}
+
 }  // namespace ragk

@@ -222,6 +222,20 @@ struct ChunkArgs {
 
 constexpr int CQ = 64;  // chunk length
 
+// inclusive sum over the wave's lanes, on the VALU (row shifts, then the two row broadcasts)
+template <int CTRL, int ROWS>
+__device__ __forceinline__ float dpp_add(float v) {
+  return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, ROWS, 0xf, false));
+}
+__device__ __forceinline__ float wave_scan(float v) {
+  v = dpp_add<0x111, 0xf>(v);  // row_shr:1
+  v = dpp_add<0x112, 0xf>(v);  // row_shr:2
+  v = dpp_add<0x114, 0xf>(v);  // row_shr:4
+  v = dpp_add<0x118, 0xf>(v);  // row_shr:8
+  v = dpp_add<0x142, 0xa>(v);  // row_bcast:15 into rows 1 and 3
+  return dpp_add<0x143, 0xc>(v);  // row_bcast:31 into rows 2 and 3
+}
+
 // split 8 floats into bf16 high and low parts
 __device__ __forceinline__ void split8(const float* f, u32x4& hi, u32x4& lo) {
 #pragma unroll
@@ -240,7 +254,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunk_kernel(Chun
   constexpr int NT16 = NP / 16, SPW = (NT16 + 3) / 4;  // state row tiles, tiles per wave
   constexpr int PT = PS / 16;
   constexpr int SROW = NP * 2 + 16;  // bytes per state column in LDS (padded against bank conflicts)
-  __shared__ __attribute__((aligned(16))) char smem[CB::TILEB + 3 * CX::TILEB + 2 * PS * SROW + 3 * CQ * 4];
+  __shared__ __attribute__((aligned(16))) char smem[CB::TILEB + 3 * CX::TILEB + 2 * PS * SROW + 2 * CQ * 4];
   char* sB = smem;                  // B rows [token][n], row-read swizzle
   char* sX = sB + CB::TILEB;        // x rows [token][p], transposed-read swizzle
   char* sXh = sX + CX::TILEB;       // e^(c_end - c_s) dt_s x_s, high part
@@ -249,7 +263,6 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunk_kernel(Chun
   char* sSl = sSh + PS * SROW;      // ... low part
   float* s_cum = reinterpret_cast<float*>(sSl + PS * SROW);  // running log-decay (log2 units)
   float* s_dt = s_cum + CQ;
-  float* s_w = s_dt + CQ;
 
   const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), tid = threadIdx.x;
   const int fr = lane & 15, fh = lane >> 4;
@@ -325,17 +338,12 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunk_kernel(Chun
   for (int c0 = 0; c0 < n; c0 += CQ) {
     // every wave forms the chunk's running log-decay (lane = token) and keeps what it needs of it
     const float dt = c0 + lane < n ? softplusf(rdt + dbias) : 0.f;
-    float cum = -decay_rate * dt;
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const float v = __shfl_up(cum, o, 64);
-      cum += lane >= o ? v : 0.f;
-    }
-    const float c_end = __shfl(cum, 63, 64);
+    const float cum = wave_scan(-decay_rate * dt);
+    const float c_end = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(cum), 63));
+    const float wgt = __builtin_amdgcn_exp2f(c_end - cum) * dt;  // what this lane's token leaves in the state
     if (wid == 0) {
       s_cum[lane] = cum;
       s_dt[lane] = dt;
-      s_w[lane] = __builtin_amdgcn_exp2f(c_end - cum) * dt;
     }
 #pragma unroll
     for (int i = 0; i < BV; ++i) {
@@ -348,7 +356,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunk_kernel(Chun
 #pragma unroll
     for (int i = 0; i < XV; ++i) {
       const int v = tid + 256 * i, t = v / (PS / 8), c = v % (PS / 8);
-      const float wt = __shfl(__builtin_amdgcn_exp2f(c_end - cum) * dt, t & 63, 64);
+      const float wt = __shfl(wgt, t & 63, 64);
       if (t < CQ) {
         const int off = t * CX::ROWB + 16 * (c ^ vswz<PS>(t));
         float f[8];
@@ -367,7 +375,7 @@ __global__ __launch_bounds__(256, NP <= 128 ? 2 : 1) void scan_chunk_kernel(Chun
 
     // ---- M^T[s][t] = (B_s . C_t) e^(c_t - c_s) dt_s for s <= t; t = 16 wid + fr ----
     const int tq = 16 * wid + fr;
-    const float c_t = __shfl(cum, tq, 64);
+    const float c_t = s_cum[tq];
     f32x4 m[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -708,6 +716,14 @@ RAGK_API int ragk_ssm_scan_seq(const int* cu_q, const int* kv_lens, const int* s
   return (int)hipGetLastError();
 }
 
+static int g_scan_cols = 0;
+// value columns per scan block: 32, 64, or 0 = by the grid (tests, measurements)
+RAGK_API int ragk_ssm_scan_set_cols(int cols) {
+  if (cols != 0 && cols != 32 && cols != 64) return (int)hipErrorInvalidValue;
+  g_scan_cols = cols;
+  return 0;
+}
+
 // Chunked scan (bf16). y: bf16 [T][H*P]. P % 8 == 0, N % 8 == 0, N <= 256, ch % 8 == 0.
 RAGK_API int ragk_ssm_scan_chunk(const int* cu_q, const int* kv_lens, const int* states, int T, int S, const void* xbc,
                                  int ch, const void* row, int ld, int off_dt, const float* dt_bias, const float* A,
@@ -718,7 +734,7 @@ RAGK_API int ragk_ssm_scan_chunk(const int* cu_q, const int* kv_lens, const int*
   const ChunkArgs a{{cu_q, kv_lens, states, T, S}, (const bf16_t*)xbc, ch, (const bf16_t*)row, ld, off_dt, dt_bias, A, D,
                     ssm_state, (bf16_t*)y, H, P, N, G};
   // narrow column slices when one block per (head, sequence) would leave CUs idle
-  const bool narrow = P <= 32 || (long long)H * S * ((P + 63) / 64) < 256;
+  const bool narrow = P <= 32 || (g_scan_cols ? g_scan_cols == 32 : (long long)H * S * ((P + 63) / 64) <= 256);
 #define RAGK_SC(NPV) return narrow ? launch_scan_chunk<NPV, 32>(a, st) : launch_scan_chunk<NPV, 64>(a, st)
   if (N <= 32) RAGK_SC(32);
   if (N <= 64) RAGK_SC(64);

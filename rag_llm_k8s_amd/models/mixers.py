@@ -59,15 +59,16 @@ class AttentionMixer:
         parts = [(get("q"), get("q.b"), H, spec.dim, spec.dkp), (get("k"), get("k.b"), G, spec.dim, spec.dkp),
                  (get("v"), get("v.b"), G, spec.vdim, spec.dvp)]
         ws = [pad_head_rows(w, n, d, dp) for w, _, n, d, dp in parts]
-        bs = [pad_head_rows((torch.zeros(n * d, dtype=w.dtype) if b is None else b)[:, None], n, d, dp)[:, 0]
+        bs = [pad_head_rows((torch.zeros(n * d, dtype=w.dtype, device=w.device) if b is None else b)[:, None], n, d, dp)[:, 0]
               for w, b, n, d, dp in parts]
         if spec.gate:
             ws.append(get("g"))
-            bs.append(torch.zeros(H, dtype=ws[0].dtype))
+            bs.append(torch.zeros(H, dtype=ws[0].dtype, device=ws[0].device))
         wqkv = dev(pad2(torch.cat(ws, 0), spec.row, wp))
         bqkv = dev(pad1(torch.cat(bs, 0), spec.row))
         wo = dev(pad2(pad_head_rows(get("o").t().contiguous(), H, spec.vdim, spec.dvp).t(), wp, spec.out_row))
         table = dev(distance_table(rel, spec.far), torch.float32) if rel is not None else None
+        spec.bias_bound = float(table.abs().max()) if table is not None else 0.0
         lam = dev(get("vmix").reshape(1), torch.float32) if vmix else None
         return cls(spec, width, wqkv, bqkv, wo, table, lam, v_source)
 

@@ -98,9 +98,10 @@ _SIGS = {
     "ragk_shaped_attn_rows": [P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, F, F, I, S],
     "ragk_ssm_conv": [P, P, P, I, I, P, I, I, P, P, P, P, I, I, I, S],
     "ragk_ssm_scan_seq": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, I, S],
-    "ragk_shaped_attn_prefill": [P, I, P, P, P, I, P, P, P, I, I, P, P, I, I, I, I, I, I, I, I, I, I, F, F, S],
+    "ragk_shaped_attn_prefill": [P, I, P, P, P, I, P, P, P, I, I, P, P, I, I, I, I, I, I, I, I, I, I, I, F, F, S],
     "ragk_shaped_attn_decode": [P, I, I, P, P, P, P, I, P, P, P, P, P, P, P, I, P, P, I, I, I, I, I, I, I, I, I, I, I, I,
                                 I, I, F, F, S],
+    "ragk_ssm_scan_set_cols": [I],
     "ragk_ssm_scan_chunk": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, S],
     "ragk_ssm_decode": [P, I, I, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, S],
     "ragk_ssm_gate_norm": [P, I, P, I, P, P, I, I, I, I, F, I, S],

@@ -202,8 +202,8 @@ def attn_prefill(row, spec, table, kc, vc, meta, out):
         row.data_ptr(), row.stride(0), kc.data_ptr(), vc.data_ptr(), meta.block_tables.data_ptr(),
         meta.block_tables.stride(0), cu, meta.kv_lens.data_ptr(), tiles.data_ptr(), tiles.shape[0], spec.heads_per_block,
         ptr(table), out.data_ptr(), out.stride(0), spec.heads, spec.kv_heads, spec.dkp, spec.dvp,
-        spec.off_g if spec.gate else -1, spec.window, spec.keep_first, spec.far, int(spec.sink), float(spec.scale),
-        float(spec.softcap), stream_ptr()), "ragk_shaped_attn_prefill")
+        spec.off_g if spec.gate else -1, spec.window, spec.keep_first, spec.far, int(spec.sink), int(spec.bounded),
+        float(spec.scale), float(spec.softcap), stream_ptr()), "ragk_shaped_attn_prefill")
     return out
 
 

@@ -6,6 +6,7 @@ padding changes no result); the padded sizes are the ones in memory.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass, field
 
 import torch
@@ -42,6 +43,7 @@ class AttnSpec:
     sink: bool = False
     gate: bool = False
     far: int = 0  # last distance of the bias table (larger distances use it); bias off when no table is given
+    bias_bound: float = math.inf  # largest |bias| of the table, when known
     dkp: int = field(init=False)
     dvp: int = field(init=False)
 
@@ -73,6 +75,11 @@ class AttnSpec:
     @property
     def out_row(self):
         return ceil_to(self.heads * self.dvp, 128)
+
+    @property
+    def bounded(self):
+        """Every score's exponential, and a sum of a million of them, fits fp32: no running maximum needed."""
+        return self.softcap > 0 and (self.softcap + self.bias_bound) * 1.4427 < 80.0
 
     @property
     def heads_per_block(self):

@@ -55,6 +55,20 @@ def timed(fn, iters, warmup=2):
     return a.elapsed_time(b) / iters * 1e-3
 
 
+def timed_graph(fn, iters):
+    """Seconds per call of a decode kernel without host launch gaps: `iters` calls in one captured graph."""
+    st = torch.cuda.Stream()
+    st.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(st):
+        fn()
+    torch.cuda.current_stream().wait_stream(st)
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g, stream=st):
+        for _ in range(iters):
+            fn()
+    return timed(g.replay, 4) / iters
+
+
 def rotate(make, nbytes, cap=8):
     """Copies of an operand set that together exceed the 256 MB Infinity Cache, used in turn."""
     n = int(max(1, min(cap, 600e6 // max(1, nbytes) + 1)))
@@ -209,18 +223,18 @@ def kernel_rows(size, nid, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
         def natt():
             k, v = caches()
             be.shaped_attn_decode(P, bias, sp, att.table, slots, k, v, mN, ob)
-        add("attention " + tag, "niduvik", timed(natt, 24), kvb, 0)
+        add("attention " + tag, "niduvik", timed_graph(natt, 24), kvb, 0)
         PL = be.gemm_part(xb, LW["wqkv"])
 
         def latt():
             k, v = caches()
             be.attn_decode_rope(PL, pos, lla.cos, lla.sin, slots, k, v, mL, ob, H, G, D)
-        add("attention " + tag, "llama", timed(latt, 24), kvb, 0)
+        add("attention " + tag, "llama", timed_graph(latt, 24), kvb, 0)
         del caches
 
         def gemm_row(name, model, f, w):
             ws = rotate(lambda: w.clone(), w.numel() * 2)
-            add(name + " " + tag, model, timed(lambda: f(ws()), 24), 2.0 * w.numel(), 2.0 * B * w.numel())
+            add(name + " " + tag, model, timed_graph(lambda: f(ws()), 24), 2.0 * w.numel(), 2.0 * B * w.numel())
         gemm_row("qkv GEMM", "niduvik", lambda w: be.proj_rows(xb, w), att.wqkv)
         gemm_row("qkv GEMM", "llama", lambda w: be.gemm_part(xb, w), LW["wqkv"])
         gemm_row("in-projection GEMM", "niduvik", lambda w: be.proj_rows(xb, w), ssm.win)
@@ -235,14 +249,14 @@ def kernel_rows(size, nid, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
         sb = 2.0 * B * ss.inner * ss.state * 4
         st = rotate(lambda: torch.zeros_like(ssm.ssm_state), sb / 2)
         add("state update " + tag, "niduvik",
-            timed(lambda: be.q.ssm_decode(P2, ss, ssm.w, mN, ssm.conv_state, st()), 24), sb + P2.numel() * 4, 0)
+            timed_graph(lambda: be.q.ssm_decode(P2, ss, ssm.w, mN, ssm.conv_state, st()), 24), sb + P2.numel() * 4, 0)
         del st
         hb = torch.randn(B, W, dtype=torch.float32, device=dev)
         hl = torch.randn(B, W, **bf)
         Pd, _ = be.proj_rows(ab, mlp.wdown)
-        add("norm " + tag, "niduvik", timed(lambda: be.residual_norm(hb, Pd, w1, w1, 1e-5, W, torch.bfloat16), 24),
+        add("norm " + tag, "niduvik", timed_graph(lambda: be.residual_norm(hb, Pd, w1, w1, 1e-5, W, torch.bfloat16), 24),
             Pd.numel() * 4 + B * W * 10.0, 0)
-        add("norm " + tag, "llama", timed(lambda: be.add_partials_rmsnorm(Pd, hl, wb, 1e-5), 24),
+        add("norm " + tag, "llama", timed_graph(lambda: be.add_partials_rmsnorm(Pd, hl, wb, 1e-5), 24),
             Pd.numel() * 4 + B * W * 6.0, 0)
     return rows
 

@@ -334,8 +334,28 @@ def test_ssm_decode_from_first_token(be):
     close(state[1], S, 1e-5)  # fp32 from slabs on: only accumulation order differs
 
 
-def test_ssm_wide_grid_uses_64_column_slices(be):
-    """Enough (head, sequence) pairs that the scan takes its 64-column form."""
+def test_ssm_column_slices_agree(be):
+    """The scan's 32- and 64-column forms (chosen by grid size) give the same numbers."""
+    from rag_llm_k8s_amd.ops import _lib
+
+    for name in ("p64", "p96", "p128"):
+        spec, w, row = ssm_setup(name, 150, BF16)
+        wd = {k: v.to(DEV).contiguous() for k, v in w.items()}
+        res = []
+        for cols in (32, 64):
+            assert _lib.lib().ragk_ssm_scan_set_cols(cols) == 0
+            try:
+                conv, state = ssm_states(spec, 2, False)
+                out = torch.zeros(150, spec.out_row, dtype=BF16, device=DEV)
+                be.ssm_prefill(row.to(DEV), spec, wd, 1e-5, ssm_meta([150], [150], [1]), conv, state, out)
+                res.append((out, state))
+            finally:
+                _lib.lib().ragk_ssm_scan_set_cols(0)
+        assert torch.equal(res[0][0], res[1][0]) and torch.equal(res[0][1], res[1][1])
+
+
+def test_ssm_wide_grid(be):
+    """Enough (head, sequence) pairs that the scan takes its 64-column form by itself."""
     spec, w, _ = ssm_setup("p64", 1, BF16)
     wd = {k: v.to(DEV).contiguous() for k, v in w.items()}
     n, lens = 70, [130 - i for i in range(70)]

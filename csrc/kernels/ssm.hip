@@ -159,24 +159,26 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(SeqArgs q, const T* __re
     if (k < taps - 1) cs[(size_t)k * ch] = v[k];
 }
 
-// One block per (head, sequence): thread (r, p) owns column p of state rows r, r + R, ...
+// One block per (head, sequence, SEQ_COLS columns): thread (r, p) owns column p of state rows r, r + R, ...
+constexpr int SEQ_COLS = 64;
 template <typename T>
 __global__ __launch_bounds__(256) void scan_seq_kernel(SeqArgs q, const T* __restrict__ xbc, int ch, const T* __restrict__ row,
                                                        int ld, int off_dt, const float* __restrict__ dt_bias,
                                                        const float* __restrict__ A, const float* __restrict__ D,
                                                        float* ssm_state, float* y, int H, int P, int N, int G, int PP) {
   extern __shared__ float sm[];
-  float* S = sm;            // [N][P]
-  float* sb = S + N * P;    // [N] dt * B
+  const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x;
+  const int p0 = blockIdx.z * SEQ_COLS, W = min(SEQ_COLS, P - p0);
+  float* S = sm;            // [N][W]
+  float* sb = S + N * W;    // [N] dt * B
   float* sc = sb + N;       // [N] C
   float* part = sc + N;     // [256]
-  const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x;
   const int g = h / (H / G), R = 256 / PP, r = tid / PP, p = tid % PP;
   int t0, n;
   bool fresh;
   seq_span(q, s, t0, n, fresh);
-  float* st = ssm_state + ((size_t)q.states[s] * H + h) * N * P;
-  for (int i = tid; i < N * P; i += 256) S[i] = fresh ? 0.f : st[i];
+  float* st = ssm_state + ((size_t)q.states[s] * H + h) * N * P + p0;
+  for (int i = tid; i < N * W; i += 256) S[i] = fresh ? 0.f : st[(size_t)(i / W) * P + i % W];
   const float a = A[h], d = D[h], db = dt_bias[h];
   __syncthreads();
   for (int t = t0; t < t0 + n; ++t) {
@@ -189,24 +191,24 @@ __global__ __launch_bounds__(256) void scan_seq_kernel(SeqArgs q, const T* __res
     }
     __syncthreads();
     float acc = 0.f, x = 0.f;
-    if (p < P) {
-      x = ld1(xr + h * P + p);
+    if (p < W) {
+      x = ld1(xr + h * P + p0 + p);
       for (int i = r; i < N; i += R) {
-        const float v = decay * S[i * P + p] + sb[i] * x;
-        S[i * P + p] = v;
+        const float v = decay * S[i * W + p] + sb[i] * x;
+        S[i * W + p] = v;
         acc = fmaf(v, sc[i], acc);
       }
     }
     part[tid] = acc;
     __syncthreads();
-    if (r == 0 && p < P) {
+    if (r == 0 && p < W) {
       float o = d * x;
       for (int i = 0; i < R; ++i) o += part[i * PP + p];
-      y[(size_t)t * H * P + h * P + p] = o;
+      y[(size_t)t * H * P + h * P + p0 + p] = o;
     }
   }
   __syncthreads();
-  for (int i = tid; i < N * P; i += 256) st[i] = S[i];
+  for (int i = tid; i < N * W; i += 256) st[(size_t)(i / W) * P + i % W] = S[i];
 }
 
 // ---- chunked scan (bf16) ----
@@ -694,23 +696,25 @@ RAGK_API int ragk_ssm_conv(const int* cu_q, const int* kv_lens, const int* state
              : launch_conv<bf16_t>(q, row, ld, off, w, b, conv_state, out, ch, taps, st);
 }
 
-// Token-by-token scan. y: fp32 [T][H*P]. N * P fp32 must fit the LDS with room for two rows of N.
+// Token-by-token scan. y: fp32 [T][H*P]. 66 N floats must fit the LDS.
 RAGK_API int ragk_ssm_scan_seq(const int* cu_q, const int* kv_lens, const int* states, int T, int S, const void* xbc, int ch,
                                const void* row, int ld, int off_dt, const float* dt_bias, const float* A, const float* D,
                                float* ssm_state, float* y, int H, int P, int N, int G, int f32, hipStream_t st) {
   if (T <= 0) return 0;
-  const size_t lds = ((size_t)N * P + 2 * N + 256) * 4;
-  if (P > 256 || H % G || lds > 160 * 1024 || S < 1 || S > 65535 || (!cu_q && S != T)) return (int)hipErrorInvalidValue;
+  const int W = P < SEQ_COLS ? P : SEQ_COLS;
+  const size_t lds = ((size_t)N * W + 2 * N + 256) * 4;
+  if (H % G || lds > 160 * 1024 || S < 1 || S > 65535 || (!cu_q && S != T)) return (int)hipErrorInvalidValue;
   int PP = 1;
-  while (PP < P) PP *= 2;
+  while (PP < W) PP *= 2;
+  const dim3 grid(H, S, (P + SEQ_COLS - 1) / SEQ_COLS);
   const SeqArgs q{cu_q, kv_lens, states, T, S};
   if (f32) {
     (void)hipFuncSetAttribute((const void*)scan_seq_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL(scan_seq_kernel<float>, dim3(H, S), dim3(256), lds, st, q, (const float*)xbc, ch, (const float*)row,
+    hipLaunchKernelGGL(scan_seq_kernel<float>, grid, dim3(256), lds, st, q, (const float*)xbc, ch, (const float*)row,
                        ld, off_dt, dt_bias, A, D, ssm_state, y, H, P, N, G, PP);
   } else {
     (void)hipFuncSetAttribute((const void*)scan_seq_kernel<bf16_t>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL(scan_seq_kernel<bf16_t>, dim3(H, S), dim3(256), lds, st, q, (const bf16_t*)xbc, ch,
+    hipLaunchKernelGGL(scan_seq_kernel<bf16_t>, grid, dim3(256), lds, st, q, (const bf16_t*)xbc, ch,
                        (const bf16_t*)row, ld, off_dt, dt_bias, A, D, ssm_state, y, H, P, N, G, PP);
   }
   return (int)hipGetLastError();

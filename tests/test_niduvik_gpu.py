@@ -239,6 +239,7 @@ SSMS = {
     "p96": dict(heads=2, vdim=96, state=256, groups=2, taps=4, norm_groups=2),
     "p30": dict(heads=2, vdim=30, state=30, groups=1, taps=4, norm_groups=4),
     "p128": dict(heads=8, vdim=128, state=64, groups=2, taps=4, norm_groups=8),
+    "p200": dict(heads=2, vdim=200, state=250, groups=1, taps=8, norm_groups=4),
     "t1": dict(heads=2, vdim=16, state=32, groups=1, taps=1, norm_groups=1),
 }
 

@@ -42,7 +42,19 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* h, const TY* 
   __shared__ float red[4];
   const int row = blockIdx.x, nvec = W >> 3;
   float* hr = h + (size_t)row * W;
-  float v[MAXV][8];
+  // everything the row needs is requested before the first reduction (rows up to 8192 columns)
+  constexpr bool PRE = MAXV <= 4;
+  constexpr int PV = PRE ? MAXV : 1;
+  float v[MAXV][8], hv[PV][8], wp[PV][8], wn[PV][8];
+  if constexpr (PRE) {
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) {
+      const int vi = min((int)threadIdx.x + i * 256, nvec - 1);
+      ld8(hr + vi * 8, hv[i]);
+      if (w_post != nullptr) ld8(w_post + vi * 8, wp[i]);
+      if (w_next != nullptr) ld8(w_next + vi * 8, wn[i]);
+    }
+  }
   float ss = 0.f;
   if (y != nullptr) {
 #pragma unroll
@@ -63,12 +75,14 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* h, const TY* 
     for (int i = 0; i < MAXV; ++i) {
       const int vi = threadIdx.x + i * 256;
       if (vi < nvec) {
-        float w[8], r[8];
-        ld8(hr + vi * 8, r);
-        if (w_post != nullptr) ld8(w_post + vi * 8, w);
+        if constexpr (!PRE) {
+          ld8(hr + vi * 8, hv[0]);
+          if (w_post != nullptr) ld8(w_post + vi * 8, wp[0]);
+        }
+        const int k = PRE ? i : 0;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          v[i][e] = r[e] + (w_post != nullptr ? v[i][e] * inv * w[e] : v[i][e]);
+          v[i][e] = hv[k][e] + (w_post != nullptr ? v[i][e] * inv * wp[k][e] : v[i][e]);
           ss += v[i][e] * v[i][e];
         }
         st8(hr + vi * 8, v[i]);
@@ -79,9 +93,12 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* h, const TY* 
     for (int i = 0; i < MAXV; ++i) {
       const int vi = threadIdx.x + i * 256;
       if (vi < nvec) {
-        ld8(hr + vi * 8, v[i]);
+        if constexpr (!PRE) ld8(hr + vi * 8, hv[0]);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) ss += v[i][e] * v[i][e];
+        for (int e = 0; e < 8; ++e) {
+          v[i][e] = hv[PRE ? i : 0][e];
+          ss += v[i][e] * v[i][e];
+        }
       }
     }
   }
@@ -91,10 +108,10 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* h, const TY* 
   for (int i = 0; i < MAXV; ++i) {
     const int vi = threadIdx.x + i * 256;
     if (vi < nvec) {
-      float w[8], o[8];
-      ld8(w_next + vi * 8, w);
+      if constexpr (!PRE) ld8(w_next + vi * 8, wn[0]);
+      float o[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = v[i][e] * inv * w[e];
+      for (int e = 0; e < 8; ++e) o[e] = v[i][e] * inv * wn[PRE ? i : 0][e];
       st8(out + (size_t)row * W + vi * 8, o);
     }
   }

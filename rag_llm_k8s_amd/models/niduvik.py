@@ -202,8 +202,9 @@ class NiduvikModel(DecoderModel):
         h = be.embed_residual(inp.ids, w.embed, carry=inp.carry, prev=inp.carry_src)
         xn = be.residual_norm(h, None, None, w.layers[0]["norm1"], eps, n, dt)
         shared = {}
+        last = w.norm if inp.logits_idx is None else None  # a prompt's final norm runs on the selected rows only
         for li, L in enumerate(w.layers):
-            nxt = w.layers[li + 1]["norm1"] if li + 1 < len(w.layers) else None
+            nxt = w.layers[li + 1]["norm1"] if li + 1 < len(w.layers) else last
             y = L["mixer"].forward(be, xn, inp, shared)
             if L["mlp"] is None:
                 xn = be.residual_norm(h, y, L["norm1b"], nxt, eps, n, dt)
@@ -212,8 +213,9 @@ class NiduvikModel(DecoderModel):
                 xn = be.residual_norm(h, L["mlp"].forward(be, xn, inp), L["norm2b"], nxt, eps, n, dt)
             if trace is not None:
                 trace.append(h[:, :n].clone())
-        if inp.logits_idx is not None:
-            h = be.gather_rows(h, inp.logits_idx)
+        if last is not None:
+            return xn
+        h = be.gather_rows(h, inp.logits_idx)
         return be.residual_norm(h, None, None, w.norm, eps, n, dt)
 
     def logits(self, hs):

@@ -99,9 +99,10 @@ __device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
 // LDS-DMA piece as inline asm: the compiler's waitcnt pass cannot tell which LDS bytes a
 // buffer_load ... lds intrinsic writes, so it drained vmcnt(0) before the next ds_read of ANY slot
 // (an HBM round trip per fragment read). A kernel that uses this orders its slots itself (vmcnt + barrier per
-// iteration) and issues every LDS-DMA through it, so M0 is never live for the compiler.
+// iteration) and issues every LDS-DMA through it, so M0 is never live for the compiler. The s_nop is the wait state between
+// the write of M0 and the DMA that reads it.
 __device__ __forceinline__ void blds16_asm(i32x4 srd, int voff, int soff, unsigned lds_addr) {
-  asm volatile("s_mov_b32 m0, %0\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds" ::"s"(lds_addr), "v"(voff), "s"(srd),
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds" ::"s"(lds_addr), "v"(voff), "s"(srd),
                "s"(soff));
 }
 __device__ __forceinline__ unsigned lds_addr(const void* p) {

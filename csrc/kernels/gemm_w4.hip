@@ -8,15 +8,13 @@
 // 16 LDS-DMA pieces (buffer_load_dwordx4 ... lds, 1 KiB each) of K-tile t+2 and 32 ds_read_b128
 // fragment reads. Two 64 KiB LDS buffers (tile t & 1), lane-linear image, source-swizzled.
 //
-// K-loop schedule (w4_iter_h, the placement of hipBLASLt's gfx950 256x256x64 direct-to-LDS kernel as
-// read from its disassembly, rebuilt here with our LDS image and epilogues): three barriers per K-tile,
-// one per LDS hazard -- the weight half of buffer t&1 free (DMAs of t+2 may start), the activation half
-// free, tile t+1 landed -- with the fragment reads spread one per 2-3 MFMAs (four waves reading one
-// fragment per 16-cycle MFMA gap saturate the CU's LDS) and the next tile's first fragments read
-// 35 MFMAs before their use. Reads, DMAs and the three waits are inline asm, so hipcc's waitcnt pass
-// adds none of its own (its lgkmcnt(14)s stalled the head of every K-tile of the previous schedule).
-// Measured against the previous two-barrier schedule (same box, M = 32768, profiles/gemm_probe_r5*.log):
-// qkv 1140 -> 1103 us, o_proj+resid 810 -> 796, gate/up+SiLU 5218 -> 5173, down+resid 2709 -> 2602.
+// K-loop schedule (w4_ktile): laid out by rule from the LDS budget of a K-tile. 4 waves x 32 fragment reads
+// and 64 LDS-DMA pieces move 192 KiB through the CU's 128 B/clk, 1536 of the 2048 clocks that the MFMAs take,
+// so both kinds of traffic are spaced evenly between the MFMAs instead of issued in bursts. Two hazards of the
+// two-buffer ring need every wave: "buffer t&1 is read out" (the DMAs of t+2 may start) and "tile t+1 landed"
+// (its fragments may be read): two barriers. Fragments are read in the order in which the MFMAs use them,
+// and the counts of the waits follow from the schedule at compile time. Reads, DMAs and waits are inline asm,
+// so hipcc's waitcnt pass adds none of its own.
 //
 // Continuous K-stream: the last two iterations of tile i stage K-tiles 0 and 1 of tile i+1 (its own
 // row offsets) into the ring slots the stream would have used, the last iteration reads tile i+1's
@@ -431,20 +429,14 @@ __device__ __forceinline__ void w4_epilogue_reg(const f32x4 (&acc)[8][8], int wr
 }
 
 // ---------------------------------------------------------------------------------------------------
-// Three-barrier K-tile schedule. Per K-tile and wave, MFMA m = 8i + j per 32-deep sub-step (the
-// activation fragment a[i] held for 8 MFMAs, the weight fragment b[j] cycling):
-//   m  0..14 : 8 reads b1[j] (weights, sub-step 1 of tile t), one per 2 MFMAs
-//   m 21/22  : lgkmcnt(0), barrier X        -> every wave is done with the weight half of buffer t&1
-//   m 22..58 : 8 weight DMAs of tile t+2 into it; reads a1[i] at m 24..42 between them
-//   m 51/52  : lgkmcnt(0), barrier Y        -> the activation half of buffer t&1 is free
-//   m 61..125: 8 activation DMAs of tile t+2
-//   m 92/93  : vmcnt(13) (the 13 DMAs of this tile are the youngest), barrier: tile t+1 landed
-//   m 93..123: the 16 F0 reads of tile t+1 (8 weight, then 8 activation fragments, spread)
-// and no drain at the end of the K-tile: the next iteration waits for exactly the F0 fragments each of
-// its first MFMAs needs (lgkmcnt(7) before m 0 = b0[0..7] and a0[0] landed; 10 before m 8: a0[1]; 13
-// before m 16: a0[2]; the m 21 drain covers the rest), so the last F0 reads of a K-tile get 20+ MFMAs
-// instead of 4 to land (an lgkmcnt(0) before the last MFMA exposed their latency every K-tile).
-// M0 is set once per DMA group and post-incremented after the next MFMA (no s_nop between M0 and DMA).
+// K-tile schedule. MFMA m = 8i + j (+ 64 in the second 32-deep sub-step) uses a[i] and b[j]; after MFMA m:
+//   R1 + q * R1_STEP      read q of tile t's second sub-step, q = 0..15
+//   FREE_W / FREE         lgkmcnt(0), barrier: buffer t&1 is read out in every wave
+//   D + q * D_STEP        DMA piece q of tile t+2 into it (activation and weight pieces in turn)
+//   LAND_W / LAND         vmcnt(pieces of t+2 issued so far), barrier: tile t+1 is in LDS
+//   F0 + q * F0_STEP      read q of tile t+1's first sub-step
+// Reads go in the order of first use: a[0], b[0..7], a[1..7]. The first sub-step's are waited for row by row at
+// the head of the next K-tile (row_wait), so the last of them may be issued late.
 __device__ __forceinline__ void h_read(bf16x8& d, unsigned addr, int off_imm) {
   // off_imm is a compile-time constant at every call site (fully unrolled schedule)
   asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(d) : "v"(addr), "i"(off_imm) : "memory");
@@ -452,86 +444,94 @@ __device__ __forceinline__ void h_read(bf16x8& d, unsigned addr, int off_imm) {
 __device__ __forceinline__ void h_dma(i32x4 srd, int voff, int soff) {
   asm volatile("buffer_load_dwordx4 %0, %1, %2 offen lds" ::"v"(voff), "s"(srd), "s"(soff) : "memory");
 }
-__device__ __forceinline__ void h_m0_set(unsigned lds) { asm volatile("s_mov_b32 m0, %0" ::"s"(lds) : "memory"); }
-__device__ __forceinline__ void h_m0_inc() { asm volatile("s_add_u32 m0, m0, 0x400" ::: "memory"); }
+// the LDS address of the next piece, one MFMA ahead of it (an instruction must lie between M0 and the DMA)
+__device__ __forceinline__ void h_m0(unsigned lds, int off_imm) {
+  asm volatile("s_add_u32 m0, %0, %1" ::"s"(lds), "i"(off_imm) : "memory", "scc");
+}
 
-// MFMA index after which each DMA piece / fragment read is issued
-constexpr int H_DX[8] = {22, 25, 28, 31, 34, 52, 55, 58};              // weight pieces (operand B)
-constexpr int H_DY[8] = {61, 64, 85, 87, 89, 96, 99, 125};             // activation pieces (operand A)
-constexpr int H_RB1[8] = {0, 2, 4, 6, 8, 10, 12, 14};                  // b1[j]
-constexpr int H_RA1[8] = {24, 27, 30, 33, 36, 38, 40, 42};             // a1[i]
-constexpr int H_RB0[8] = {93, 94, 95, 97, 98, 100, 101, 102};          // b0[j] of tile t+1
-constexpr int H_RA0[8] = {104, 107, 110, 113, 116, 119, 121, 123};     // a0[i] of tile t+1
-constexpr int H_VM = 13;  // DMAs of this iteration issued before the m = 92 wait
+struct W4Sched {
+  int r1, r1_step, free_w, d, d_step, land_w, f0, f0_step;
+  constexpr int at(int first, int step, int m) const {  // q if read / piece q follows MFMA m, else -1
+    return m >= first && (m - first) % step == 0 && (m - first) / step < 16 ? (m - first) / step : -1;
+  }
+  constexpr int read1(int m) const { return at(r1, r1_step, m); }
+  constexpr int piece(int m) const { return at(d, d_step, m); }
+  constexpr int read0(int m) const { return at(f0, f0_step, m); }
+  constexpr int pieces_before(int m) const {
+    int n = 0;
+    for (int k = 0; k < m; ++k) n += piece(k) >= 0;
+    return n;
+  }
+  // LDS reads that may still be in flight before MFMA m = 8i: all but the first sub-step's first 9 + i
+  constexpr int row_wait(int m) const {
+    int n = 16 - (9 + m / 8);
+    for (int k = 0; k < m; ++k) n += read1(k) >= 0;
+    return n < 15 ? n : 15;
+  }
+  constexpr bool ok() const {
+    return r1 + 15 * r1_step < free_w && free_w < d && d + 15 * d_step < 128 && free_w < 64 && land_w < f0 &&
+           f0 >= 64 && f0 + 15 * f0_step < 128 && d > 0 && d_step > 1;
+  }
+};
+constexpr W4Sched SCH{1, 2, 37, 40, 5, 84, 87, 2};
+static_assert(SCH.ok(), "K-tile schedule");
+constexpr int H_VM = SCH.pieces_before(SCH.land_w);  // DMAs of this K-tile issued before the LAND wait
 
-constexpr int h_find(const int (&s)[8], int m) {
-  for (int q = 0; q < 8; ++q)
-    if (s[q] == m) return q;
-  return -1;
+template <int Q>
+__device__ __forceinline__ void h_fragment(unsigned ra, unsigned rb, bf16x8 (&a)[8], bf16x8 (&b)[8]) {
+  if constexpr (Q == 0) h_read(a[0], ra, 0);
+  else if constexpr (Q < 9) h_read(b[Q - 1], rb, (Q - 1) * 2048);
+  else h_read(a[Q - 8], ra, (Q - 8) * 2048);
 }
 
 // One K-tile. g = running K-tile index (ring slot g & 1); sa / sb = DMA source offsets at K-tile kst
-// (this tile's t+2 or the next tile's 0 / 1); ZERO = the F0 MFMAs start the accumulators (srcC = 0);
-// VMW = the m = 92 vmcnt bound (H_VM plus the vector-memory ops issued between the previous
-// iteration's DMAs and this one's, i.e. an epilogue). F0 = issue the 16 F0 reads of K-tile t+1 (false:
+// (this tile's t+2 or the next tile's 0 / 1); ZERO = the first sub-step's MFMAs start the accumulators
+// (srcC = 0); VMW = the LAND wait's bound (H_VM plus the vector-memory ops issued between the previous
+// K-tile's DMAs and this one's, i.e. an epilogue). F0 = issue the 16 first reads of K-tile t+1 (false:
 // the caller issues them itself, w4_read_f0). rbA / rbB: this lane's read bases (sub-step s, buffer 0)
 // of the activation / weight fragments; fragment i at + 2048 i (the swizzle of row 16 i + fr does not
 // depend on i).
 template <bool ZERO, int VMW, bool F0 = true>
-__device__ __forceinline__ void w4_iter_h(char* smem, int g, i32x4 srd_a, i32x4 srd_b, const int (&sa)[8],
-                                          const int (&sb)[8], int kst, int wid, const unsigned (&rbA)[2],
-                                          const unsigned (&rbB)[2], f32x4 (&acc)[8][8], bf16x8 (&a0)[8],
-                                          bf16x8 (&b0)[8], bf16x8 (&a1)[8], bf16x8 (&b1)[8]) {
+__device__ __forceinline__ void w4_ktile(char* smem, int g, i32x4 srd_a, i32x4 srd_b, const int (&sa)[8],
+                                         const int (&sb)[8], int kst, int wid, const unsigned (&rbA)[2],
+                                         const unsigned (&rbB)[2], f32x4 (&acc)[8][8], bf16x8 (&a0)[8],
+                                         bf16x8 (&b0)[8], bf16x8 (&a1)[8], bf16x8 (&b1)[8]) {
   static_assert(VMW >= H_VM && VMW <= 63, "vmcnt bound");
   const unsigned cur = (unsigned)(g & 1) * W_BUF, nxt = (unsigned)((g + 1) & 1) * W_BUF;
   const unsigned lds_cur = (unsigned)(unsigned long long)(const __attribute__((address_space(3))) char*)smem + cur;
-  const unsigned mX = __builtin_amdgcn_readfirstlane(lds_cur + W_TILE_A + wid * 8192);  // weight pieces
-  const unsigned mY = __builtin_amdgcn_readfirstlane(lds_cur + wid * 8192);             // activation pieces
+  const unsigned dst = __builtin_amdgcn_readfirstlane(lds_cur + wid * 8192);  // weight pieces W_TILE_A further
   const int kb = kst * WBK * 2;
   const unsigned rb1 = rbB[1] + cur, ra1 = rbA[1] + cur, rb0 = rbB[0] + nxt, ra0 = rbA[0] + nxt;
   static_for<128>([&](auto mc) __attribute__((always_inline)) {
     constexpr int m = decltype(mc)::value;
-    if constexpr (m == 0) asm volatile("s_waitcnt lgkmcnt(7)" ::: "memory");
-    if constexpr (m == 8) asm volatile("s_waitcnt lgkmcnt(10)" ::: "memory");
-    if constexpr (m == 16) asm volatile("s_waitcnt lgkmcnt(13)" ::: "memory");
-    if constexpr (m == 21 || m == 51) asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    if constexpr (m == 22 || m == 52) w4_barrier();
-    if constexpr (m == 92) asm volatile("s_waitcnt vmcnt(%0)" ::"i"(VMW) : "memory");
-    if constexpr (m == 93) w4_barrier();
+    if constexpr (m % 8 == 0 && m < SCH.free_w)
+      asm volatile("s_waitcnt lgkmcnt(%0)" ::"i"(SCH.row_wait(m)) : "memory");
+    if constexpr (m == SCH.free_w) asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    if constexpr (m == SCH.land_w) asm volatile("s_waitcnt vmcnt(%0)" ::"i"(VMW) : "memory");
+    if constexpr (m == SCH.free_w + 1 || m == SCH.land_w + 1) w4_barrier();
     if constexpr (m < 64) {
       if constexpr (ZERO) w4_mfma0(acc, a0, b0, m);
       else w4_mfma(acc, a0, b0, m);
     } else {
       w4_mfma(acc, a1, b1, m - 64);
     }
-    // post-increment M0 one MFMA after each piece; a group's M0 is set before its first piece
-    if constexpr (h_find(H_DX, m - 1) >= 0 || h_find(H_DY, m - 1) >= 0) h_m0_inc();
-    if constexpr (m == 21) h_m0_set(mX);
-    if constexpr (m == 59) h_m0_set(mY);
-    constexpr int qx = h_find(H_DX, m), qy = h_find(H_DY, m);
-    if constexpr (qx >= 0) h_dma(srd_b, sb[qx], kb);
-    if constexpr (qy >= 0) h_dma(srd_a, sa[qy], kb);
-    constexpr int r1b = h_find(H_RB1, m), r1a = h_find(H_RA1, m), r0b = h_find(H_RB0, m), r0a = h_find(H_RA0, m);
-    if constexpr (r1b >= 0) h_read(b1[r1b], rb1, r1b * 2048);
-    if constexpr (r1a >= 0) h_read(a1[r1a], ra1, r1a * 2048);
-    if constexpr (F0 && r0b >= 0) h_read(b0[r0b], rb0, r0b * 2048);
-    if constexpr (F0 && r0a >= 0) h_read(a0[r0a], ra0, r0a * 2048);
+    constexpr int q = SCH.piece(m), qn = SCH.piece(m + 1);
+    if constexpr (q >= 0) h_dma(q & 1 ? srd_b : srd_a, q & 1 ? sb[q >> 1] : sa[q >> 1], kb);
+    if constexpr (qn >= 0) h_m0(dst, (qn & 1) * W_TILE_A + (qn >> 1) * 1024);
+    constexpr int r1 = SCH.read1(m), r0 = SCH.read0(m);
+    if constexpr (r1 >= 0) h_fragment<r1>(ra1, rb1, a1, b1);
+    if constexpr (F0 && r0 >= 0) h_fragment<r0>(ra0, rb0, a0, b0);
   });
 }
 
-// The F0 reads of the K-tile in ring slot g & 1, in w4_iter_h's order (the 8 weight fragments, then the
-// 8 activation fragments), left in flight for the next w4_iter_h's counted waits.
+// The first reads of the K-tile in ring slot g & 1, in w4_ktile's order, left in flight for the next
+// w4_ktile's counted waits.
 __device__ __forceinline__ void w4_read_f0(int g, const unsigned (&rbA)[2], const unsigned (&rbB)[2],
                                            bf16x8 (&a0)[8], bf16x8 (&b0)[8]) {
   const unsigned buf = (unsigned)(g & 1) * W_BUF;
   const unsigned rb0 = rbB[0] + buf, ra0 = rbA[0] + buf;
-  static_for<8>([&](auto jc) __attribute__((always_inline)) {
-    constexpr int j = decltype(jc)::value;
-    h_read(b0[j], rb0, j * 2048);
-  });
-  static_for<8>([&](auto ic) __attribute__((always_inline)) {
-    constexpr int i = decltype(ic)::value;
-    h_read(a0[i], ra0, i * 2048);
+  static_for<16>([&](auto qc) __attribute__((always_inline)) {
+    h_fragment<decltype(qc)::value>(ra0, rb0, a0, b0);
   });
 }
 
@@ -626,10 +626,10 @@ __global__ __launch_bounds__(W4_THREADS, 1) void gemm_w4_kernel(const bf16_t* __
   for (;;) {
     const int next = tile + (int)gridDim.x;
     const bool has_next = next < nwt;
-    w4_iter_h<true, VMH0>(smem, g, srd_a, srd_b, off_a, off_b, 2, wid, rbA, rbB, acc, a0, b0, a1, b1);
+    w4_ktile<true, VMH0>(smem, g, srd_a, srd_b, off_a, off_b, 2, wid, rbA, rbB, acc, a0, b0, a1, b1);
     ++g;
     for (int t = 1; t + 2 < nk; ++t, ++g)
-      w4_iter_h<false, H_VM>(smem, g, srd_a, srd_b, off_a, off_b, t + 2, wid, rbA, rbB, acc, a0, b0, a1, b1);
+      w4_ktile<false, H_VM>(smem, g, srd_a, srd_b, off_a, off_b, t + 2, wid, rbA, rbB, acc, a0, b0, a1, b1);
     // The last two iterations stage (and read the first fragments of) the next tile; on the block's
     // last tile they re-stage this tile's K-tiles 0 / 1 instead (valid addresses, never read), so both
     // cases run the same straight-line code: a branch around the MFMA iterations made the register
@@ -652,9 +652,9 @@ __global__ __launch_bounds__(W4_THREADS, 1) void gemm_w4_kernel(const bf16_t* __
         }
       }
     }
-    w4_iter_h<false, H_VM>(smem, g, srd_a, srd_b, off_a, off_b, 0, wid, rbA, rbB, acc, a0, b0, a1, b1);
+    w4_ktile<false, H_VM>(smem, g, srd_a, srd_b, off_a, off_b, 0, wid, rbA, rbB, acc, a0, b0, a1, b1);
     ++g;
-    w4_iter_h<false, H_VM, !LATE_F0>(smem, g, srd_a, srd_b, off_a, off_b, 1, wid, rbA, rbB, acc, a0, b0, a1, b1);
+    w4_ktile<false, H_VM, !LATE_F0>(smem, g, srd_a, srd_b, off_a, off_b, 1, wid, rbA, rbB, acc, a0, b0, a1, b1);
     ++g;
     // the epilogue is compiler-scheduled code: it may move any register, so no asm read is in flight
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");

@@ -1,8 +1,10 @@
-// Attention with shaped scores over the paged cache (K pages [blocks][G][64][DK], V pages [blocks][G][64][DV]):
+// Attention with shaped scores over the paged cache (K pages [blocks][G][64][DK], V pages [blocks][G][64][DV]),
+// or over packed key / value rows of the step (row_attn_*: keys of a sequence in consecutive rows):
 //
 //   s_ij = softcap * tanh(q_i . k_j * scale / softcap) + table[h][min(i - j, far)]
 //   j visible to i:  j <= i  and  (window == 0 or i - j < window or j < keep)
 //   out_i = gate_ih * sum_j exp(s_ij) v_j / (sink + sum_j exp(s_ij)),  sink in {0, 1}
+//   gate_ih: none, one sigmoid per head, or one per head and value element
 //
 // Positions are the tokens' own in the sequence, so the kept first tokens enter with their true distances.
 // Scores, softmax and the bias are fp32.
@@ -33,8 +35,17 @@ struct ShapedArgs {
   void* out; int ldo;
   int T, S, H, G, DK, DV;
   int off_g;                   // column of the gates, -1: no gate
+  int gate_vec;                // 1: a gate per head and value element, 0: one per head
   int window, keep, far, sink;
   float scale, softcap;
+  // keys: entry e of a sequence's page list starts at kc + e * k_unit + kv head * k_head, rows k_row apart. Paged:
+  // e = block table entry; packed rows: e = key_off[seq] + first position of the page.
+  const int* key_off;          // [S] row of position 0 of each sequence (may be negative), null: paged
+  long long k_unit, v_unit;
+  int k_head, k_row, v_head, v_row;
+  __device__ __forceinline__ int entry(const int* bt, int seq, int page) const {
+    return key_off ? key_off[seq] + page * 64 : bt[page];
+  }
 };
 
 template <typename T>
@@ -68,9 +79,10 @@ __global__ __launch_bounds__(256) void kv_store_kernel(const T* __restrict__ row
   }
 }
 
-template <typename T>
+// NC: value columns per lane, sizes up to 64 NC
+template <typename T, int NC>
 __global__ __launch_bounds__(64) void attn_rows_kernel(ShapedArgs a) {
-  __shared__ float sq[256], sp[64];
+  __shared__ float sq[64 * NC], sp[64];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int s = a.cu_q ? seq_of(a.cu_q, a.S, t) : t;
   const int q0 = a.cu_q ? a.cu_q[s] : t, q1 = a.cu_q ? a.cu_q[s + 1] : t + 1;
@@ -85,11 +97,13 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(ShapedArgs a) {
   const int first_win = a.window > 0 ? max(keep_pages, max(0, i - a.window + 1) / 64) : n_pages;
   const int n_it = keep_pages + max(0, n_pages - first_win);
   float m = a.sink ? 0.f : -INFINITY, l = a.sink ? 1.f : 0.f;
-  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  float acc[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) acc[c] = 0.f;
   for (int it = 0; it < n_it; ++it) {
     const int pg = it < keep_pages ? it : first_win + it - keep_pages;
-    const int blk = bt[pg], j = pg * 64 + lane;
-    const T* kr = (const T*)a.kc + (((size_t)blk * a.G + g) * 64 + lane) * a.DK;
+    const int e0 = a.entry(bt, s, pg), j = pg * 64 + lane;
+    const T* kr = (const T*)a.kc + e0 * a.k_unit + (size_t)g * a.k_head + (size_t)lane * a.k_row;
     const bool ok = j <= i && (a.window <= 0 || i - j < a.window || j < a.keep);
     float x = 0.f;
     if (ok) {
@@ -114,23 +128,24 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(ShapedArgs a) {
     __syncthreads();
     sp[lane] = p;
     __syncthreads();
-    const T* vb = (const T*)a.vc + ((size_t)blk * a.G + g) * 64 * a.DV;
+    const T* vb = (const T*)a.vc + e0 * a.v_unit + (size_t)g * a.v_head;
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
+    for (int c = 0; c < NC; ++c) {
       const int d = lane + 64 * c;
       if (d < a.DV) {
         acc[c] *= alpha;
         const int nj = min(64, i + 1 - pg * 64);
-        for (int k = 0; k < nj; ++k) acc[c] = fmaf(sp[k], ld1(vb + (size_t)k * a.DV + d), acc[c]);
+        for (int k = 0; k < nj; ++k) acc[c] = fmaf(sp[k], ld1(vb + (size_t)k * a.v_row + d), acc[c]);
       }
     }
   }
   const float inv = l > 0.f ? 1.f / l : 0.f;
   float gate = 1.f;
-  if (a.off_g >= 0) gate = 1.f / (1.f + expf(-ld1(qr + a.off_g + h)));
+  if (a.off_g >= 0 && !a.gate_vec) gate = 1.f / (1.f + expf(-ld1(qr + a.off_g + h)));
 #pragma unroll
-  for (int c = 0; c < 4; ++c) {
+  for (int c = 0; c < NC; ++c) {
     const int d = lane + 64 * c;
+    if (d < a.DV && a.off_g >= 0 && a.gate_vec) gate = 1.f / (1.f + expf(-ld1(qr + a.off_g + h * a.DV + d)));
     if (d < a.DV) st1((T*)a.out + (size_t)t * a.ldo + h * a.DV + d, acc[c] * inv * gate);
   }
 }
@@ -231,7 +246,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     l_i[qt] = a.sink && fh == 0 ? 1.f : 0.f;
   }
   const int* bt = a.block_tables + (size_t)seq * a.bt_stride;
-  for (int i = threadIdx.x; i < pg.n; i += 256) s_bt[i] = bt[pg.page(i)];
+  for (int i = threadIdx.x; i < pg.n; i += 256) s_bt[i] = a.entry(bt, seq, pg.page(i));
   if (a.table && pa.sb_stride)
     for (int h = 0; h < gb; ++h)
       for (int i = threadIdx.x; i <= a.far; i += 256)
@@ -254,18 +269,18 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
 #pragma unroll
   for (int i = 0; i < KP; ++i) {
     const int row = (wid_u + 4 * i) * CK::RPP + lane / CK::NC, ph = lane % CK::NC;
-    koff[i] = row * CK::ROWB + 16 * (ph ^ kswz<DK>(row));
+    koff[i] = row * a.k_row * 2 + 16 * (ph ^ kswz<DK>(row));
   }
 #pragma unroll
   for (int i = 0; i < VP; ++i) {
     const int row = (wid_u + 4 * i) * CV::RPP + lane / CV::NC, ph = lane % CV::NC;
-    voff[i] = row * CV::ROWB + 16 * (ph ^ vswz<DV>(row));
+    voff[i] = row * a.v_row * 2 + 16 * (ph ^ vswz<DV>(row));
   }
   const unsigned lds0 = lds_addr(smem);
   auto stage = [&](int it, int buf) {
-    const size_t pgi = (size_t)__builtin_amdgcn_readfirstlane(s_bt[it]) * a.G + kvh;
-    const i32x4 srd_k = make_srd((const bf16_t*)a.kc + pgi * KT * DK, CK::TILEB);
-    const i32x4 srd_v = make_srd((const bf16_t*)a.vc + pgi * KT * DV, CV::TILEB);
+    const int e0 = __builtin_amdgcn_readfirstlane(s_bt[it]);
+    const i32x4 srd_k = make_srd((const bf16_t*)a.kc + e0 * a.k_unit + kvh * a.k_head, (63 * a.k_row + DK) * 2);
+    const i32x4 srd_v = make_srd((const bf16_t*)a.vc + e0 * a.v_unit + kvh * a.v_head, (63 * a.v_row + DV) * 2);
     const unsigned l = lds0 + buf * (CK::TILEB + CV::TILEB);
 #pragma unroll
     for (int i = 0; i < KP; ++i) blds16_asm(srd_k, koff[i], 0, l + (wid_u + 4 * i) * 1024);
@@ -441,14 +456,22 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     float inv = l > 0.f ? 1.f / l : 0.f;
     const int qi = pbase + 16 * qt + fr;
     if (qi < q_len) {
-      if (a.off_g >= 0) {
+      const bf16_t* gp = nullptr;
+      if (a.off_g >= 0 && a.gate_vec) {
+        gp = (const bf16_t*)a.q + (size_t)(q_off + qi) * a.ldq + a.off_g + hq * DV + 4 * fh;
+      } else if (a.off_g >= 0) {
         const float g = bf2f(((const bf16_t*)a.q)[(size_t)(q_off + qi) * a.ldq + a.off_g + hq]);
         inv *= __builtin_amdgcn_rcpf(1.f + __expf(-g));
       }
       bf16_t* op = (bf16_t*)a.out + (size_t)(q_off + qi) * a.ldo + hq * DV + 4 * fh;
 #pragma unroll
       for (int dt = 0; dt < CV::DT; ++dt) {
-        const f32x4 v = o[dt][qt] * inv;
+        f32x4 v = o[dt][qt] * inv;
+        if (gp) {
+          const bf16x4 g = *reinterpret_cast<const bf16x4*>(gp + 16 * dt);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) v[r] *= __builtin_amdgcn_rcpf(1.f + __expf(-bf2f_s(g[r])));
+        }
         *reinterpret_cast<uint2*>(op + 16 * dt) = make_uint2(pk2bf(v[0], v[1]), pk2bf(v[2], v[3]));
       }
     }
@@ -784,6 +807,31 @@ int launch_decode(const ShapedDecode& a, hipStream_t st) {
 
 }  // namespace
 
+namespace {
+ShapedArgs paged_args(const void* q, int ldq, const void* kc, const void* vc, const int* bt, int bt_stride, const int* cu_q,
+                      const int* kv_lens, const float* table, void* out, int ldo, int T, int S, int H, int G, int DK,
+                      int DV, int off_g, int window, int keep, int far, int sink, float scale, float softcap) {
+  return ShapedArgs{q, ldq, kc, vc, bt, bt_stride, cu_q, kv_lens, table, out, ldo, T, S, H, G, DK, DV, off_g, 0, window,
+                    keep, far, sink, scale, softcap, nullptr, (long long)G * 64 * DK, (long long)G * 64 * DV, 64 * DK, DK,
+                    64 * DV, DV};
+}
+// packed rows [keys][ldk]: keys at column h * DK, values at off_v + h * DV; one gate per value element
+ShapedArgs rows_args(const void* q, int ldq, const void* kv, int ldk, int off_v, size_t elem, const int* key_off,
+                     const int* cu_q, const int* kv_lens, void* out, int ldo, int T, int S, int H, int DK, int DV, int off_g,
+                     int window, float scale) {
+  return ShapedArgs{q, ldq, kv, (const char*)kv + off_v * elem, nullptr, 0, cu_q, kv_lens, nullptr, out, ldo, T, S, H, H, DK,
+                    DV, off_g, 1, window, 0, 0, 0, scale, 0.f, key_off, ldk, ldk, DK, ldk, DV, ldk};
+}
+template <typename T>
+void launch_rows(const ShapedArgs& a, hipStream_t st) {
+  if (a.DK <= 256 && a.DV <= 256) hipLaunchKernelGGL((attn_rows_kernel<T, 4>), dim3(a.T, a.H), dim3(64), 0, st, a);
+  else hipLaunchKernelGGL((attn_rows_kernel<T, 16>), dim3(a.T, a.H), dim3(64), 0, st, a);
+}
+int dispatch_prefill(int DK, int DV, const ShapedPrefill& pa, int n_tiles, int bounded, hipStream_t st) {
+  RAGK_SHAPED_DISPATCH(launch_prefill, pa, n_tiles, bounded, st);
+}
+}  // namespace
+
 // bf16. tiles: [n_tiles][2] (sequence, first query) of 128 / gb query rows each; gb in {1, 2, 4} divides H / G.
 // bounded: the caller knows that (softcap + largest |bias|) * log2e < 80 (every 2^score and the sum over any context fit).
 RAGK_API int ragk_shaped_attn_prefill(const void* q, int ldq, const void* kc, const void* vc, const int* block_tables,
@@ -795,10 +843,40 @@ RAGK_API int ragk_shaped_attn_prefill(const void* q, int ldq, const void* kc, co
   if (H % G || (gb != 1 && gb != 2 && gb != 4) || (H / G) % gb || bt_stride > MAX_BT || ldq % 8 || ldo % 4 || !cu_q ||
       window < 0 || keep < 0 || far < 0 || (bounded && !(softcap > 0.f)))
     return (int)hipErrorInvalidValue;
-  const ShapedArgs a{q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, 0, 0, H, G, DK, DV,
-                     off_g, window, keep, far, sink, scale, softcap};
+  const ShapedArgs a = paged_args(q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, 0, 0, H, G, DK,
+                                  DV, off_g, window, keep, far, sink, scale, softcap);
   const ShapedPrefill pa{a, tiles, H / gb, gb, 0};
-  RAGK_SHAPED_DISPATCH(launch_prefill, pa, n_tiles, bounded, st);
+  return dispatch_prefill(DK, DV, pa, n_tiles, bounded, st);
+}
+
+// The same kernel over packed key / value rows kv [rows][ldk] (bf16): H heads of their own, position p of sequence s in
+// row key_off[s] + p. Whole 64-row groups are read: every group that starts at a key must lie inside the rows.
+RAGK_API int ragk_row_attn_prefill(const void* q, int ldq, const void* kv, int ldk, int off_v, const int* key_off,
+                                   const int* cu_q, const int* kv_lens, const int* tiles, int n_tiles, void* out, int ldo,
+                                   int H, int DK, int DV, int off_g, int window, int max_pages, float scale,
+                                   hipStream_t st) {
+  if (n_tiles <= 0) return 0;
+  if (max_pages > MAX_BT || ldq % 8 || ldk % 8 || off_v % 8 || ldo % 4 || off_g % 4 || !cu_q || !key_off || window < 0 ||
+      H < 1 || off_v < H * DK || off_v + H * DV > ldk)
+    return (int)hipErrorInvalidValue;
+  const ShapedPrefill pa{rows_args(q, ldq, kv, ldk, off_v, 2, key_off, cu_q, kv_lens, out, ldo, 0, 0, H, DK, DV, off_g,
+                                   window, scale),
+                         tiles, H, 1, 0};
+  return dispatch_prefill(DK, DV, pa, n_tiles, 0, st);
+}
+
+// plain fp32 arithmetic over the same packed rows (fp32 when f32, else bf16); any head size up to 256
+RAGK_API int ragk_row_attn_rows(const void* q, int ldq, const void* kv, int ldk, int off_v, const int* key_off,
+                                const int* cu_q, const int* kv_lens, void* out, int ldo, int T, int S, int H, int DK,
+                                int DV, int off_g, int window, float scale, int f32, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (DK % 8 || DK > 256 || DV > 256 || H > 65535 || ldk % 8 || off_v % 8 || !cu_q || !key_off)
+    return (int)hipErrorInvalidValue;
+  const ShapedArgs a = rows_args(q, ldq, kv, ldk, off_v, f32 ? 4 : 2, key_off, cu_q, kv_lens, out, ldo, T, S, H, DK, DV,
+                                 off_g, window, scale);
+  if (f32) launch_rows<float>(a, st);
+  else launch_rows<bf16_t>(a, st);
+  return (int)hipGetLastError();
 }
 
 // bf16 caches, fp32 slabs P [S][B][ldp] (+ bias). The new token's k / v go to `slots`; out [B][ldo].
@@ -839,10 +917,10 @@ RAGK_API int ragk_shaped_attn_rows(const void* q, int ldq, const void* kc, const
                                    int ldo, int T, int S, int H, int G, int DK, int DV, int off_g, int window, int keep,
                                    int far, int sink, float scale, float softcap, int f32, hipStream_t st) {
   if (T <= 0) return 0;
-  if (DK % 8 || DK > 256 || DV > 256 || H % G || H > 65535) return (int)hipErrorInvalidValue;
-  const ShapedArgs a{q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, T, S, H, G, DK, DV,
-                     off_g, window, keep, far, sink, scale, softcap};
-  if (f32) hipLaunchKernelGGL(attn_rows_kernel<float>, dim3(T, H), dim3(64), 0, st, a);
-  else hipLaunchKernelGGL(attn_rows_kernel<bf16_t>, dim3(T, H), dim3(64), 0, st, a);
+  if (DK % 8 || DK > 1024 || DV > 1024 || H % G || H > 65535) return (int)hipErrorInvalidValue;
+  const ShapedArgs a = paged_args(q, ldq, kc, vc, block_tables, bt_stride, cu_q, kv_lens, table, out, ldo, T, S, H, G, DK,
+                                  DV, off_g, window, keep, far, sink, scale, softcap);
+  if (f32) launch_rows<float>(a, st);
+  else launch_rows<bf16_t>(a, st);
   return (int)hipGetLastError();
 }

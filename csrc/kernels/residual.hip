@@ -1,10 +1,15 @@
 // Residual-stream kernels: the stream h is fp32 rows, padded to the GEMM tile (padding columns are zero).
 //
-//  * embed_residual : h[t] = table[ids[t]] in fp32 (ids may be carried over from the previous step's samples).
+//  * embed_residual : h[t] = table[ids[t]] * scale in fp32 (ids may be carried over from the previous step's samples),
+//    plus the sinusoid of the token's position: angles are reduced in fp64, so they are exact to fp32 rounding at any
+//    position.
 //  * residual_norm  : h += norm(y) * w_post; out = norm(h) * w_next, one pass over the row. y is a sublayer's
 //    output: fp32 split-K slabs (summed here, so a decode GEMM needs no reduction launch), fp32 rows or bf16
 //    rows. Without w_post the sublayer is added as it is; without y only the norm runs; without w_next only
 //    the add. norm(x) = x / sqrt(mean(x^2) + eps) over the n real columns.
+//  * gated_residual : h += norm(y * sigmoid(z + b)) * w, the sublayer gated element by element before its norm; then
+//    the rows themselves and / or the token-shifted rows, for a next sublayer that reads the stream without a norm.
+//  * token_shift    : x[t] + (x[t-1] - x[t]) * mix; the row before a sequence's first new token is its state.
 //  * glu_clip       : the clipped gated unit over packed [64 gate | 64 up] tiles (fp32 path; the bf16 GEMMs
 //    have it as an epilogue).
 #include "seq_common.h"
@@ -15,7 +20,9 @@ namespace {
 template <typename T>
 __global__ __launch_bounds__(256) void embed_residual_kernel(int* __restrict__ ids, const T* __restrict__ table, float* h,
                                                              int W, int vocab, const int* __restrict__ carry,
-                                                             const int* __restrict__ prev) {
+                                                             const int* __restrict__ prev, float scale, int n,
+                                                             const int* __restrict__ pos,
+                                                             const double* __restrict__ turns) {
   const int t = blockIdx.x;
   int id = ids[t];
   if (carry != nullptr) {
@@ -30,7 +37,145 @@ __global__ __launch_bounds__(256) void embed_residual_kernel(int* __restrict__ i
   for (int v = threadIdx.x; v < (W >> 3); v += 256) {
     float f[8];
     ld8(table + (size_t)id * W + v * 8, f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] *= scale;
+    if (pos != nullptr) {  // columns 2i / 2i + 1: sin / cos of pos * turns[i] whole turns
+      const double p = pos[t];
+#pragma unroll
+      for (int e = 0; e < 8; e += 2) {
+        const int c = v * 8 + e;
+        if (c < n) {
+          const double a = p * turns[c >> 1];
+          float sn, cs;
+          sincospif((float)(2.0 * (a - rint(a))), &sn, &cs);
+          f[e] += sn;
+          if (c + 1 < n) f[e + 1] += cs;
+        }
+      }
+    }
     st8(h + (size_t)t * W + v * 8, f);
+  }
+}
+
+// new row of one vector of the stream -> the shifted row (prev: the row before it)
+template <typename TO>
+__device__ __forceinline__ void put_shifted(TO* dst, const float* x, const float* prev, const float* mix) {
+  float o[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) o[e] = x[e] + (prev[e] - x[e]) * mix[e];
+  st8(dst, o);
+}
+
+struct GatedArgs {
+  float* h; int W; float n, eps;
+  const void* y; int S; const void* z; int SZ; size_t slab;  // rows, or fp32 split-K slabs
+  const float* zb; const float* w;                            // [W]; zb null: y is not gated
+  void* out;                                                   // the new rows, or null
+  const float* mix; void* shifted; float* state;              // decode: one row per sequence; null: no shift
+  const int* slots; const int* kv_lens;
+};
+
+template <int MAXV, typename TY, typename TO>
+__global__ __launch_bounds__(256) void gated_residual_kernel(GatedArgs a) {
+  __shared__ float red[4];
+  const int row = blockIdx.x, nvec = a.W >> 3;
+  const size_t base = (size_t)row * a.W;
+  constexpr bool PRE = MAXV <= 2;  // the stream's row and the weights are requested before the reduction
+  constexpr int PV = PRE ? MAXV : 1;
+  float v[MAXV][8], hv[PV][8], wv[PV][8];
+  auto fetch = [&](int i, int k) {
+    const int vi = min((int)threadIdx.x + i * 256, nvec - 1);
+    ld8(a.h + base + vi * 8, hv[k]);
+    ld8(a.w + vi * 8, wv[k]);
+  };
+  if constexpr (PRE) {
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) fetch(i, i);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int vi = threadIdx.x + i * 256;
+    if (vi < nvec) {
+      const TY* yp = (const TY*)a.y + base + vi * 8;
+      if constexpr (sizeof(TY) == 4) sum_slabs8(yp, a.S, a.slab, v[i]);
+      else ld8(yp, v[i]);
+      if (a.zb != nullptr) {
+        float z[8], b[8];
+        const TY* zp = (const TY*)a.z + base + vi * 8;
+        if constexpr (sizeof(TY) == 4) sum_slabs8(zp, a.SZ, a.slab, z);
+        else ld8(zp, z);
+        ld8(a.zb + vi * 8, b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[i][e] /= 1.f + expf(-(z[e] + b[e]));
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += v[i][e] * v[i][e];
+    }
+  }
+  const float inv = rsqrtf(block_sum(ss, red) / a.n + a.eps);
+  float* st = nullptr;
+  bool fresh = false;
+  if (a.mix != nullptr) {
+    st = a.state + (size_t)a.slots[row] * a.W;
+    fresh = a.kv_lens[row] == 1;
+  }
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int vi = threadIdx.x + i * 256;
+    if (vi < nvec) {
+      const int k = PRE ? i : 0;
+      if constexpr (!PRE) fetch(i, 0);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] = hv[k][e] + v[i][e] * inv * wv[k][e];
+      st8(a.h + base + vi * 8, v[i]);
+      if (a.out != nullptr) st8((TO*)a.out + base + vi * 8, v[i]);
+      if (st != nullptr) {
+        float p[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, m[8];
+        if (!fresh) ld8(st + vi * 8, p);
+        ld8(a.mix + vi * 8, m);
+        put_shifted((TO*)a.shifted + base + vi * 8, v[i], p, m);
+        st8(st + vi * 8, v[i]);
+      }
+    }
+  }
+}
+
+template <typename TY, typename TO>
+int launch_gated(const GatedArgs& a, int M, hipStream_t st) {
+  const int per = (a.W / 8 + 255) / 256;
+  if (per <= 1) hipLaunchKernelGGL((gated_residual_kernel<1, TY, TO>), dim3(M), dim3(256), 0, st, a);
+  else if (per <= 2) hipLaunchKernelGGL((gated_residual_kernel<2, TY, TO>), dim3(M), dim3(256), 0, st, a);
+  else if (per <= 4) hipLaunchKernelGGL((gated_residual_kernel<4, TY, TO>), dim3(M), dim3(256), 0, st, a);
+  else if (per <= 8) hipLaunchKernelGGL((gated_residual_kernel<8, TY, TO>), dim3(M), dim3(256), 0, st, a);
+  else return (int)hipErrorInvalidValue;
+  return (int)hipGetLastError();
+}
+
+// cu null: one token per sequence. The block of a sequence's first new token reads the state and then replaces it by
+// the last new row, element by element in the same thread.
+template <typename TO>
+__global__ __launch_bounds__(256) void token_shift_kernel(const float* __restrict__ h, int W, const float* __restrict__ mix,
+                                                          float* state, const int* __restrict__ slots,
+                                                          const int* __restrict__ cu, const int* __restrict__ kv_lens,
+                                                          int S, TO* out, TO* shifted) {
+  const int t = blockIdx.x;
+  const int s = cu ? seq_of(cu, S, t) : t, q0 = cu ? cu[s] : t, q1 = cu ? cu[s + 1] : t + 1;
+  const bool first = t == q0, fresh = kv_lens[s] == q1 - q0;
+  float* st = state + (size_t)slots[s] * W;
+  for (int v = threadIdx.x; v < (W >> 3); v += 256) {
+    float x[8], p[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, m[8];
+    ld8(h + (size_t)t * W + v * 8, x);
+    ld8(mix + v * 8, m);
+    if (!first) ld8(h + (size_t)(t - 1) * W + v * 8, p);
+    else if (!fresh) ld8(st + v * 8, p);
+    if (out != nullptr) st8(out + (size_t)t * W + v * 8, x);
+    put_shifted(shifted + (size_t)t * W + v * 8, x, p, m);
+    if (first) {
+      float l[8];
+      ld8(h + (size_t)(q1 - 1) * W + v * 8, l);
+      st8(st + v * 8, l);
+    }
   }
 }
 
@@ -164,17 +309,49 @@ __global__ __launch_bounds__(256) void glu_clip_kernel(const float* __restrict__
 
 }  // namespace
 
-// table: [vocab][W] bf16 (f32 = 0) or fp32; h: fp32 [T][W], W % 8 == 0. carry / prev may be null.
+// table: [vocab][W] bf16 (f32 = 0) or fp32; h: fp32 [T][W], W % 8 == 0. carry / prev may be null. pos [T] and turns
+// [(n + 1) / 2] (fp64, turns per position of each column pair), or null: no sinusoid.
 RAGK_API int ragk_embed_residual(int* ids, const void* table, float* h, int T, int W, int vocab, const int* carry,
-                                 const int* prev, int f32, hipStream_t st) {
+                                 const int* prev, float scale, int n, const int* pos, const double* turns, int f32,
+                                 hipStream_t st) {
   if (T <= 0) return 0;
-  if (W % 8) return (int)hipErrorInvalidValue;
+  if (W % 8 || n > W || (pos && !turns)) return (int)hipErrorInvalidValue;
   if (f32)
     hipLaunchKernelGGL(embed_residual_kernel<float>, dim3(T), dim3(256), 0, st, ids, (const float*)table, h, W, vocab,
-                       carry, prev);
+                       carry, prev, scale, n, pos, turns);
   else
     hipLaunchKernelGGL(embed_residual_kernel<bf16_t>, dim3(T), dim3(256), 0, st, ids, (const bf16_t*)table, h, W, vocab,
-                       carry, prev);
+                       carry, prev, scale, n, pos, turns);
+  return (int)hipGetLastError();
+}
+
+// h: fp32 [M][W] += norm(y * sigmoid(z + zb)) * w. y, z: bf16 rows [M][W] (y_bf16, S = SZ = 1) or fp32 slabs [S][M][W].
+// out / shifted: [M][W], fp32 when out_f32; either may be null. shifted takes mix [W], state [slots][W], slots, kv_lens [M]
+// (one token per sequence).
+RAGK_API int ragk_gated_residual(float* h, const void* y, int S, const void* z, int SZ, int y_bf16, const float* zb,
+                                 const float* w, void* out, const float* mix, void* shifted, float* state,
+                                 const int* slots, const int* kv_lens, int out_f32, int M, int W, int n, float eps,
+                                 hipStream_t st) {
+  if (M <= 0) return 0;
+  if (W % 8 || W > 16384 || !y || !w || S < 1 || SZ < 1 || (y_bf16 && (S != 1 || SZ != 1)) || (zb && !z) ||
+      (mix && (!shifted || !state || !slots || !kv_lens)))
+    return (int)hipErrorInvalidValue;
+  const GatedArgs a{h, W, (float)n, eps, y, S, z, SZ, (size_t)M * W, zb, w, out, mix, shifted, state, slots, kv_lens};
+  if (y_bf16) return out_f32 ? launch_gated<bf16_t, float>(a, M, st) : launch_gated<bf16_t, bf16_t>(a, M, st);
+  return out_f32 ? launch_gated<float, float>(a, M, st) : launch_gated<float, bf16_t>(a, M, st);
+}
+
+// h: fp32 [T][W]; cu [S + 1] or null (one token per sequence); out (may be null) / shifted: [T][W], fp32 when f32
+RAGK_API int ragk_token_shift(const float* h, int T, int W, const float* mix, float* state, const int* slots, const int* cu,
+                              const int* kv_lens, int S, void* out, void* shifted, int f32, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (W % 8 || !mix || !state || !slots || !kv_lens || !shifted || (!cu && S != T)) return (int)hipErrorInvalidValue;
+  if (f32)
+    hipLaunchKernelGGL(token_shift_kernel<float>, dim3(T), dim3(256), 0, st, h, W, mix, state, slots, cu, kv_lens, S,
+                       (float*)out, (float*)shifted);
+  else
+    hipLaunchKernelGGL(token_shift_kernel<bf16_t>, dim3(T), dim3(256), 0, st, h, W, mix, state, slots, cu, kv_lens, S,
+                       (bf16_t*)out, (bf16_t*)shifted);
   return (int)hipGetLastError();
 }
 

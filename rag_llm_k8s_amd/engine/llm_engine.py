@@ -602,7 +602,8 @@ class LLMEngine:
                 out_seqs.append(s)
         tiles, qtiles = self.model.prefill_work(qlens, self.device)
         meta = AttnMeta("prefill", self._h2d_i32(kvl), self._h2d_i32(bts), cu_q=self._h2d_i32(cu),
-                        tiles=tiles, qtiles=qtiles, host_kv_lens=kvl, host_q_lens=qlens,
+                        tiles=tiles, qtiles=qtiles, host_kv_lens=kvl, host_q_lens=qlens, max_kv=self.max_model_len,
+                        key_rows=self.model.key_rows(qlens, kvl, self.device),
                         states=self._h2d_i32([self.bm.state(s.id) for s, _, _ in chunks]))
         ntok = cu[-1]
         out_rows = rows if rows is not None else out_rows

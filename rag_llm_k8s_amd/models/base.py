@@ -44,6 +44,10 @@ class DecoderModel:
         return (pt, mp, torch.empty((batch, self.Hq, mp, self.D), **f32),
                 torch.empty((batch, self.Hq, mp, 2), **f32))
 
+    def key_rows(self, q_lens, kv_lens, device):
+        """Packed key rows of a prefill step by window (models that expand cached latents)."""
+        return {}
+
     def state_bytes_per_slot(self):
         return 0
 

@@ -1,4 +1,4 @@
-"""Sublayers of residual-stream decoders: shaped attention, Mamba-2 state space, clipped GLU.
+"""Sublayers of residual-stream decoders: shaped attention, latent attention, Mamba-2 state space, gated MLPs.
 
 Each mixer owns its device weights and its cache (paged K/V, or per-slot state) and maps normed rows to
 either the sublayer's output rows (prefill) or fp32 split-K slabs of them (decode), which the following
@@ -9,10 +9,12 @@ norms, scores, decays and states are fp32 in both.
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..ops.reference import pack_gate_up
-from ..ops.specs import AttnSpec, SsmSpec, ceil_to, distance_table
+from ..ops.specs import AttnSpec, LatentSpec, SsmSpec, ceil_to, distance_table
 
 
 def pad2(t, rows, cols):
@@ -106,6 +108,56 @@ class AttentionMixer:
         return y
 
 
+class LatentAttentionMixer:
+    """Latent attention (ops/specs.LatentSpec). A mixer with a source reads that mixer's cached latents through its own
+    key and value maps."""
+
+    recurrent = False
+
+    def __init__(self, spec: LatentSpec, width, eps, index, win, lw, wo, source=None):
+        self.spec, self.width, self.eps, self.index = spec, width, eps, index
+        self.win, self.lw, self.wo, self.source = win, lw, wo, source
+        self.pages = None
+
+    @classmethod
+    def load(cls, spec: LatentSpec, width, eps, index, get, dev, source=None):
+        """get(name): raw tensor of 'q', 'g', 'uk', 'uv', 'o' and, in a layer of its own latents, 'dkv', 'dkv.norm'."""
+        H, wp, rp = spec.heads, ceil_to(width, 128), spec.rp
+        ws = [pad_head_rows(get("q"), H, spec.dim, spec.dkp), pad_head_rows(get("g"), H, spec.vdim, spec.dvp)]
+        if spec.own:
+            ws.append(get("dkv"))
+        win = dev(pad2(torch.cat(ws, 0), spec.row, wp))
+        maps = [pad2(pad_head_rows(get(n), H, d, dp), H * dp, rp)
+                for n, d, dp in (("uk", spec.dim, spec.dkp), ("uv", spec.vdim, spec.dvp))]
+        ukv = dev(torch.cat(maps, 0))  # expands a latent row to [k of every head | v of every head]
+        lw = dict(ukv=ukv, uv=ukv[spec.off_v:].view(H, spec.dvp, rp),
+                  uk=dev(maps[0].reshape(H, spec.dkp, rp).transpose(1, 2)), norm=None,
+                  source=index if source is None else source.index)
+        if spec.own:
+            lw["norm"] = dev(pad1(get("dkv.norm").float(), rp), torch.float32)
+        wo = dev(pad2(pad_head_rows(get("o").t().contiguous(), H, spec.vdim, spec.dvp).t(), wp, spec.out_row))
+        return cls(spec, width, eps, index, win, lw, wo, source)
+
+    def cache_bytes(self, itemsize):
+        return 64 * self.spec.rp * itemsize if self.spec.own else 0
+
+    def allocate_cache(self, num_blocks, dtype, device):
+        if self.spec.own:
+            self.pages = torch.zeros(num_blocks, 64, self.spec.rp, dtype=dtype, device=device)
+
+    def forward(self, be, x, inp, shared):
+        """`shared`: latent rows that layers of one forward hand on, by source layer."""
+        s = self.spec
+        pages = self.pages if self.source is None else self.source.pages
+        exact = s.out_row == s.heads * s.dvp
+        out = (torch.empty if exact else torch.zeros)((x.shape[0], s.out_row), dtype=x.dtype, device=x.device)
+        if inp.meta.kind == "decode":
+            be.latent_decode(be.proj_rows(x, self.win)[0], s, self.lw, self.eps, inp, pages, out)
+            return be.proj_rows(out, self.wo)[0]
+        be.latent_prefill(be.gemm(x, self.win), s, self.lw, self.eps, inp, pages, shared, out)
+        return be.gemm(out, self.wo)
+
+
 class Mamba2Mixer:
     """Mamba-2 layer: in-projection, short causal convolution, selective scan, gated grouped RMS norm."""
 
@@ -148,19 +200,28 @@ class Mamba2Mixer:
         return be.gemm(out, self.wo)
 
 
-class ClippedGluMlp:
-    """W_down (min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + shift)), g | u = packed gate/up rows."""
+class GluMlp:
+    """W_down (silu(g) * u), g | u = packed gate/up rows."""
 
-    def __init__(self, wgu, wdown, par):
+    def __init__(self, wgu, wdown, par=None):
         self.wgu, self.wdown, self.par = wgu, wdown, par
 
     @classmethod
-    def load(cls, width, ff, limit, alpha, shift, get, dev):
+    def load(cls, width, ff, get, dev, par=None):
         wp, fp = ceil_to(width, 128), ceil_to(ff, 128)
         wgu = dev(pack_gate_up(pad2(get("gate"), fp, wp), pad2(get("up"), fp, wp)))
-        return cls(wgu, dev(pad2(get("down"), wp, fp)),
-                   dev(torch.tensor([limit, alpha, shift, 0.0]), torch.float32))
+        if par is None and wgu.dtype == torch.float32:  # the fp32 unit has the clipped form only: nothing is clipped
+            par = dev(torch.tensor([math.inf, 1.0, 0.0, 0.0]), torch.float32)
+        return cls(wgu, dev(pad2(get("down"), wp, fp)), par)
 
     def forward(self, be, xn, inp):
         a = be.gemm_glu(xn, self.wgu, self.par)
         return be.proj_rows(a, self.wdown)[0] if inp.meta.kind == "decode" else be.gemm(a, self.wdown)
+
+
+class ClippedGluMlp(GluMlp):
+    """W_down (min(g, limit) sigmoid(alpha g) (clamp(u, +-limit) + shift))."""
+
+    @classmethod
+    def load(cls, width, ff, limit, alpha, shift, get, dev):
+        return super().load(width, ff, get, dev, dev(torch.tensor([limit, alpha, shift, 0.0]), torch.float32))

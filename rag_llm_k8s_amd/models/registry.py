@@ -49,6 +49,13 @@ def _niduvik(path, raw, device, dtype, tp_rank, tp_size, comm, max_len):
     return NiduvikModel(c, NiduvikWeights.from_checkpoint(path, c, device, DTYPES[dtype]), device, comm=comm)
 
 
+def _rolesun(path, raw, device, dtype, tp_rank, tp_size, comm, max_len):
+    from .rolesun import RolesunConfig, RolesunModel, RolesunWeights
+
+    c = RolesunConfig.from_dict(raw)
+    return RolesunModel(c, RolesunWeights.from_checkpoint(path, c, device, DTYPES[dtype]), device, comm=comm)
+
+
 def _names(raw):
     return {str(x).lower() for x in [raw.get("model_type"), raw.get("architecture")] + list(raw.get("architectures") or [])
             if x}
@@ -58,6 +65,9 @@ FAMILIES = (
     Family("niduvik", lambda raw: "niduvik" in _names(raw), _niduvik, ("bf16", "float32"),
            ("gemm.hip", "gemm_w4.hip", "gemm_pp.hip", "gemm_stream.hip", "gemm_dec.hip", "gemm_part.hip", "gemm_f32.hip",
             "norm.hip", "residual.hip", "attn_shaped.hip", "ssm.hip", "sampling.hip")),
+    Family("rolesun", lambda raw: "rolesun" in _names(raw), _rolesun, ("bf16", "float32"),
+           ("gemm.hip", "gemm_w4.hip", "gemm_pp.hip", "gemm_stream.hip", "gemm_dec.hip", "gemm_part.hip", "gemm_f32.hip",
+            "norm.hip", "residual.hip", "attn_shaped.hip", "latent.hip", "sampling.hip")),
     Family("gpt2", lambda raw: "gpt2" in _names(raw), _gpt2, ("bf16",)),
     Family("llama", lambda raw: True, _llama, ("bf16", "fp8")),
 )

@@ -89,7 +89,9 @@ _SIGS = {
     "ragk_quant_fp8_rows": [P, I, P, I, P, I, I, S],
     "ragk_gemm_fp8": [P, I, P, I, P, P, I, P, P, I, P, P, I, I, I, I, I, I, S],
     # residual.hip / gemm_f32.hip / attn_shaped.hip / ssm.hip
-    "ragk_embed_residual": [P, P, P, I, I, I, P, P, I, S],
+    "ragk_embed_residual": [P, P, P, I, I, I, P, P, F, I, P, P, I, S],
+    "ragk_gated_residual": [P, P, I, P, I, I, P, P, P, P, P, P, P, P, I, I, I, I, F, S],
+    "ragk_token_shift": [P, I, I, P, P, P, P, P, I, P, P, I, S],
     "ragk_residual_norm": [P, P, I, I, I, P, P, P, I, I, I, I, F, S],
     "ragk_slab_rows": [P, I, P, P, I, I, I, S],
     "ragk_glu_clip": [P, P, I, I, P, S],
@@ -101,6 +103,15 @@ _SIGS = {
     "ragk_shaped_attn_prefill": [P, I, P, P, P, I, P, P, P, I, I, P, P, I, I, I, I, I, I, I, I, I, I, I, F, F, S],
     "ragk_shaped_attn_decode": [P, I, I, P, P, P, P, I, P, P, P, P, P, P, P, I, P, P, I, I, I, I, I, I, I, I, I, I, I, I,
                                 I, I, F, F, S],
+    "ragk_row_attn_prefill": [P, I, P, I, I, P, P, P, P, I, P, I, I, I, I, I, I, I, F, S],
+    "ragk_row_attn_rows": [P, I, P, I, I, P, P, P, P, I, I, I, I, I, I, I, I, F, I, S],
+    # latent.hip
+    "ragk_latent_store": [P, I, I, I, I, P, F, P, P, P, I, I, I, S],
+    "ragk_latent_gather": [P, I, P, I, P, P, I, I, I, P, I, S],
+    "ragk_head_proj_f32": [P, I, I, P, I, P, I, P, I, I, I, S],
+    "ragk_latent_absorb": [P, I, I, I, I, I, I, I, I, I, P, P, P, P, P, F, S],
+    "ragk_latent_decode": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, S],
+    "ragk_latent_out": [P, I, I, I, I, P, P, P, P, P, I, I, I, I, I, I, I, I, S],
     "ragk_ssm_scan_set_cols": [I],
     "ragk_ssm_scan_chunk": [P, P, P, I, I, P, I, P, I, I, P, P, P, P, P, I, I, I, I, S],
     "ragk_ssm_decode": [P, I, I, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, S],

@@ -41,6 +41,7 @@ class AttnMeta:
     states: Optional[torch.Tensor] = None  # int32 [S] recurrent-state slot of every sequence
     qtiles: dict = field(default_factory=dict)  # prefill work lists by query-tile height (shaped attention)
     max_kv: int = 0  # longest context the decode workspace was sized for (shaped attention)
+    key_rows: dict = field(default_factory=dict)  # prefill: packed key rows by window (latent attention)
 
 
 class TorchBackend:
@@ -218,19 +219,35 @@ class TorchBackend:
         return R.pool_l2norm(hidden, cu.cpu(), mode=mode, normalize=normalize)
 
     # fp32 residual stream, shaped attention, state-space mixers ---------------
-    def embed_residual(self, ids, table, carry=None, prev=None):
-        """Embedding rows as the fp32 residual stream."""
-        return self.embed(ids, table, carry=carry, prev=prev).float()
+    def embed_residual(self, ids, table, carry=None, prev=None, scale=1.0, pos=None, turns=None, n=0):
+        """Embedding rows * scale as the fp32 residual stream, plus the sinusoid of `pos` over the first n columns."""
+        h = self.embed(ids, table, carry=carry, prev=prev).float() * scale
+        return h if pos is None else h + RS.sinusoid(pos, turns, n, h.shape[1])
 
     def residual_norm(self, h, y, w_post, w_next, eps, n, out_dtype):
         return RS.residual_norm(h, y, w_post, w_next, eps, n, out_dtype)
+
+    def gated_residual(self, h, y, z, zb, w, eps, n, out_dtype, keep=False, shift=None, meta=None):
+        """h += norm(y * sigmoid(z + zb)) * w. Returns (h in out_dtype if `keep`, the token-shifted rows if `shift` =
+        (mix, state) -- decode steps)."""
+        RS.gated_residual(h, y, z, zb, w, eps, n)
+        xs = None if shift is None else self.token_shift(h, shift[0], shift[1], meta, out_dtype)[1]
+        return h.to(out_dtype, copy=True) if keep else None, xs
+
+    def token_shift(self, h, mix, state, meta: AttnMeta, out_dtype, keep=True):
+        """(h in out_dtype if `keep`, the token-shifted rows); state [slots, width] holds each sequence's last row."""
+        ql = [1] * h.shape[0] if meta.kind == "decode" else meta.host_q_lens
+        xs = RS.token_shift(h, mix, state, ql, meta.host_kv_lens, meta.states)
+        return h.to(out_dtype, copy=True) if keep else None, xs.to(out_dtype)
 
     def proj_rows(self, x, w, bias=None):
         """Decode projection rows for a consumer that sums them: fp32 slabs [S, M, N] + the bias still to add."""
         return self.gemm(x, w, out_f32=True).unsqueeze(0), bias
 
     def gemm_glu(self, x, w, par):
-        """Packed gate/up projection with the clipped GLU (par = [limit, alpha, shift])."""
+        """Packed gate/up projection with the clipped GLU (par = [limit, alpha, shift]; None, in bf16: silu(g) * u)."""
+        if par is None:
+            par = (math.inf, 1.0, 0.0)
         g, u = R.unpack_gate_up(w)
         xf = x.float()
         return RS.glu_clip(xf @ g.float().t(), xf @ u.float().t(), par).to(x.dtype)
@@ -247,6 +264,23 @@ class TorchBackend:
         own = RS.kv_store(row, spec, slots, kc, vc, v_first, lam)
         RS.attention(row, spec, table, kc, vc, meta.block_tables, [1] * row.shape[0], meta.host_kv_lens, out)
         return own
+
+    def latent_prefill(self, row, spec, lw, eps, inp, pages, rows, out):
+        """Latent attention of a prompt step's projection rows: latents of `own` layers into the pages, then attention
+        over each sequence's visible latents. lw: weights (mixers.LatentAttentionMixer); rows: latent rows that the layers
+        of one forward share, by source layer."""
+        m = inp.meta
+        if spec.own:
+            RS.latent_store(row, spec, lw["norm"], eps, inp.slots, pages)
+        return RS.latent_attention(row, spec, lw["uk"], lw["uv"], pages, m.block_tables, m.host_q_lens, m.host_kv_lens, out)
+
+    def latent_decode(self, P, spec, lw, eps, inp, pages, out):
+        """One new token per sequence from its projection slabs: cache append, attention, output gate."""
+        row, m = RS.rows_of(P, None), inp.meta
+        if spec.own:
+            RS.latent_store(row, spec, lw["norm"], eps, inp.slots, pages)
+        return RS.latent_attention(row, spec, lw["uk"], lw["uv"], pages, m.block_tables, [1] * row.shape[0], m.host_kv_lens,
+                                   out)
 
     def ssm_prefill(self, row, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
         return RS.ssm(row, spec, w, eps, meta.host_q_lens, meta.host_kv_lens, meta.states, conv_state, ssm_state, out)
@@ -403,8 +437,18 @@ class NativeBackend(TorchBackend):
                                   meta.max_parts, meta.ws_o, meta.ws_ml)
 
     # fp32 residual stream, shaped attention, state-space mixers ---------------
-    def embed_residual(self, ids, table, carry=None, prev=None):
-        return self.q.embed_residual(ids, table, carry, prev)
+    def embed_residual(self, ids, table, carry=None, prev=None, scale=1.0, pos=None, turns=None, n=0):
+        return self.q.embed_residual(ids, table, carry, prev, scale, pos, turns, n)
+
+    def gated_residual(self, h, y, z, zb, w, eps, n, out_dtype, keep=False, shift=None, meta=None):
+        if out_dtype == torch.float32 and keep:  # the stream itself is the fp32 activation
+            return h, self.q.gated_residual(h, y, z, zb, w, eps, n, out_dtype, False, shift, meta)[1]
+        return self.q.gated_residual(h, y, z, zb, w, eps, n, out_dtype, keep, shift, meta)
+
+    def token_shift(self, h, mix, state, meta, out_dtype, keep=True):
+        if out_dtype == torch.float32 and keep:
+            return h, self.q.token_shift(h, mix, state, meta, out_dtype, False)[1]
+        return self.q.token_shift(h, mix, state, meta, out_dtype, keep)
 
     def residual_norm(self, h, y, w_post, w_next, eps, n, out_dtype):
         return self.q.residual_norm(h, y, w_post, w_next, eps, n, out_dtype)
@@ -419,7 +463,7 @@ class NativeBackend(TorchBackend):
     def gemm_glu(self, x, w, par):
         if w.dtype == torch.float32:
             return self.q.glu_clip_f32(self.q.gemm_f32(x, w), par)
-        return self.n.gemm_glu(x, w, par)
+        return self.n.gemm(x, w, epi="silu_mul") if par is None else self.n.gemm_glu(x, w, par)
 
     def shaped_kv_store(self, row, spec, slots, kc, vc, v_first=None, lam=None):
         return self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
@@ -436,6 +480,39 @@ class NativeBackend(TorchBackend):
         own = self.q.kv_store(row, spec, slots, kc, vc, v_first, lam)
         self.q.attn_rows(row, spec, table, kc, vc, meta, out)
         return own
+
+    def latent_prefill(self, row, spec, lw, eps, inp, pages, rows, out):
+        meta = inp.meta
+        kr = meta.key_rows[spec.window]
+        if spec.own:
+            rows[lw["source"]] = self.q.latent_store(row, spec, lw["norm"], eps, inp.slots, pages)
+        if kr.seqs:
+            key = (lw["source"], spec.window) if kr.gather else lw["source"]
+            if key not in rows:
+                rows[key] = self.q.latent_gather(pages, spec, meta, kr)
+            kv = self.gemm(rows[key][:kr.rows + self.q.KEY_PAD], lw["ukv"])
+            self.q.row_attention(row, spec, kv, kr, meta, out)
+        if kr.tail:
+            self._latent_tail(row, spec, lw, meta, kr, pages, out)
+        return out
+
+    def _latent_tail(self, row, spec, lw, meta, kr, pages, out):
+        """The one-token sequences behind a step's prompts (their latents are in the pages): as decode rows."""
+        t0 = row.shape[0] - kr.tail
+        m = AttnMeta("decode", meta.kv_lens[kr.seqs:], meta.block_tables[kr.seqs:], max_kv=meta.max_kv)
+        if row.dtype == torch.float32:
+            return self.q.latent_decode_rows(row[t0:], spec, lw["uk"], lw["uv"], pages, m, out[t0:])
+        return self.q.latent_decode(row[t0:], spec, lw["uk"], lw["uv"], pages, m, out[t0:],
+                                    ws=self.q.latent_workspace([spec], m.max_kv, kr.tail, row.device))
+
+    def latent_decode(self, P, spec, lw, eps, inp, pages, out):
+        if out.dtype == torch.bfloat16:
+            return self.q.latent_decode(P, spec, lw["uk"], lw["uv"], pages, inp.meta, out,
+                                        slots=inp.slots if spec.own else None, norm=lw["norm"], eps=eps)
+        row = self.q.slab_rows(P, None, out.dtype)
+        if spec.own:
+            self.q.latent_store(row, spec, lw["norm"], eps, inp.slots, pages, keep=False)
+        return self.q.latent_decode_rows(row, spec, lw["uk"], lw["uv"], pages, inp.meta, out)
 
     def ssm_prefill(self, row, spec, w, eps, meta: AttnMeta, conv_state, ssm_state, out):
         xbc = self.q.ssm_conv(row, spec, w, meta, conv_state, ssm_state)

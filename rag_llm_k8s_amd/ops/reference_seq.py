@@ -1,4 +1,4 @@
-"""CPU forms of the residual-stream, shaped-attention and state-space kernels (torch, fp32 arithmetic).
+"""CPU forms of the residual-stream, shaped-attention, latent-attention and state-space kernels (torch, fp32 arithmetic).
 
 Same operands and memory layouts as the GPU kernels in csrc/kernels/residual.hip, attn_shaped.hip and ssm.hip:
 paged caches [blocks, kv_heads, 64, size], per-sequence state slots, fused projection rows (ops/specs.py).
@@ -27,6 +27,64 @@ def residual_norm(h, y, w_post, w_next, eps, n, out_dtype):
         y = y.float().sum(0) if y.dim() == 3 else y.float()
         h += rms(y, w_post, eps, n) if w_post is not None else y
     return None if w_next is None else rms(h, w_next, eps, n).to(out_dtype)
+
+
+def sinusoid(pos, turns, n, width):
+    """[T, width]: sin / cos of pos * turns[i] whole turns at columns 2i / 2i + 1 below n, zero from there."""
+    a = pos.double()[:, None] * turns.double()[None, :]
+    a = 2 * math.pi * (a - torch.round(a))
+    out = torch.zeros(pos.numel(), width)
+    out[:, 0:n:2] = torch.sin(a).float()
+    out[:, 1:n:2] = torch.cos(a).float()[:, :n // 2]
+    return out
+
+
+def gated_residual(h, y, z, zb, w, eps, n):
+    """h (fp32, in place) += norm(y * sigmoid(z + zb)) * w."""
+    y = rows_of(y, None)
+    if z is not None:
+        y = y * torch.sigmoid(rows_of(z, zb))
+    h += rms(y, w, eps, n)
+
+
+def token_shift(h, mix, state, q_lens, kv_lens, states):
+    """h[t] + (h[t - 1] - h[t]) * mix per sequence; state[slot] holds the row before the first and takes the last."""
+    out, t0 = torch.empty_like(h), 0
+    for s, (ql, L) in enumerate(zip(q_lens, kv_lens)):
+        slot, x = int(states[s]), h[t0:t0 + ql]
+        before = torch.zeros_like(x[:1]) if L == ql else state[slot][None].clone()
+        out[t0:t0 + ql] = x + (torch.cat([before, x[:-1]]) - x) * mix
+        state[slot] = x[-1]
+        t0 += ql
+    return out
+
+
+def latent_store(row, spec, norm, eps, slots, pages):
+    c = rms(row[:, spec.off_c:spec.off_c + spec.rp], norm, eps, spec.rank).to(pages.dtype)
+    s = slots.long()
+    ok = s >= 0
+    pages[s[ok] // BLOCK, s[ok] % BLOCK] = c[ok]
+
+
+def latent_attention(row, spec, wuk, wuv, pages, block_tables, q_lens, kv_lens, out):
+    """Queries are the last q_lens[s] positions of each context; wuk [H, rp, dkp], wuv [H, dvp, rp]."""
+    H, t0 = spec.heads, 0
+    out.zero_()
+    uk, uv = wuk.float(), wuv.float().transpose(1, 2).contiguous()
+    for s, (ql, L) in enumerate(zip(q_lens, kv_lens)):
+        q = row[t0:t0 + ql, :spec.off_g].float().reshape(ql, H, spec.dkp).transpose(0, 1).contiguous()
+        c = paged_kv_view(pages[:, None], block_tables[s], L, BLOCK).float()[:, 0]
+        k, v = torch.matmul(c, uk), torch.matmul(c, uv)  # [H, L, dkp], [H, L, dvp]
+        sc = (q @ k.transpose(1, 2).contiguous()) * spec.scale
+        i, j = torch.arange(L - ql, L)[:, None], torch.arange(L)[None, :]
+        ok = j <= i
+        if spec.window > 0:
+            ok = ok & (i - j < spec.window)
+        o = (torch.softmax(sc.masked_fill(~ok, -math.inf), -1) @ v).transpose(0, 1).reshape(ql, -1)
+        o = o * torch.sigmoid(row[t0:t0 + ql, spec.off_g:spec.off_c].float())
+        out[t0:t0 + ql, :H * spec.dvp] = o.to(out.dtype)
+        t0 += ql
+    return out
 
 
 def glu_clip(g, u, par):

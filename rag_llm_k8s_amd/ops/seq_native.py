@@ -1,4 +1,5 @@
-"""Shape-checked entry points of the residual-stream, shaped-attention and state-space kernels (GPU tensors).
+"""Shape-checked entry points of the residual-stream, shaped-attention, latent-attention and state-space kernels
+(GPU tensors).
 
 Operands are checked on the host before every launch, as in ops/native.py. `f32` paths (exact replay) take
 fp32 tensors throughout; otherwise activations and caches are bf16 and the residual stream, split-K slabs,
@@ -6,12 +7,15 @@ norm weights and recurrent states fp32.
 """
 from __future__ import annotations
 
+from dataclasses import dataclass
+
 import numpy as np
 import torch
 
 from . import _lib
 from ._lib import check, ptr, stream_ptr
 from .native import _req
+from .specs import LatentSpec
 
 BF16, F32, I32 = torch.bfloat16, torch.float32, torch.int32
 
@@ -26,17 +30,81 @@ def _vec(t, n, dtype, name):
 
 
 # ------------------------------------------------------------------------------------- residual stream
-def embed_residual(ids, table, carry=None, prev=None):
+def embed_residual(ids, table, carry=None, prev=None, scale=1.0, pos=None, turns=None, n=0):
+    """fp32 rows table[ids] * scale, plus the sinusoid of `pos` over the first n columns (turns: fp64 turns per
+    position of every column pair)."""
     _req(ids.dtype == I32 and ids.is_cuda and ids.is_contiguous() and table.is_contiguous(), "ids int32, table dense")
     V, W = table.shape
     f32 = _act(table, "table")
     if carry is not None:
         _req(carry.dtype == I32 and prev.dtype == I32 and carry.numel() >= ids.numel(), "carry int32")
+    if pos is not None:
+        _vec(pos, ids.numel(), I32, "pos")
+        _vec(turns, (n + 1) // 2, torch.float64, "turns")
     h = torch.empty((ids.numel(), W), dtype=F32, device=table.device)
     check(_lib.lib().ragk_embed_residual(ids.data_ptr(), table.data_ptr(), h.data_ptr(), ids.numel(), W, V, ptr(carry),
-                                         ptr(prev) if carry is not None else None, f32, stream_ptr()),
+                                         ptr(prev) if carry is not None else None, float(scale), n, ptr(pos),
+                                         ptr(turns) if pos is not None else None, f32, stream_ptr()),
           "ragk_embed_residual")
     return h
+
+
+def _slabs(y, M, W, name):
+    """(rows are bf16, number of slabs) of rows [M, W] or fp32 slabs [S, M, W]."""
+    _req(y.is_cuda and y.dtype in (BF16, F32) and y.is_contiguous() and y.shape[-2:] == (M, W) and y.dim() in (2, 3), name)
+    bf, S = int(y.dtype == BF16), y.shape[0] if y.dim() == 3 else 1
+    _req(S == 1 or not bf, "bf16 rows come as one slab")
+    return bf, S
+
+
+def _shift_state(mix, state, meta, M, W):
+    _vec(mix, W, F32, "mix")
+    _req(state.dtype == F32 and state.is_contiguous() and state.dim() == 2 and state.shape[1] == W, "shift state")
+    S = meta.kv_lens.numel()
+    _req(meta.states is not None and meta.states.dtype == I32 and meta.states.numel() == S, "state slots")
+    _req(meta.kind != "decode" or S == M, "one token per sequence")
+    return S
+
+
+def gated_residual(h, y, z, zb, w, eps, n, out_dtype, keep=False, shift=None, meta=None):
+    """h += norm(y * sigmoid(z + zb)) * w in place. y / z: rows, or fp32 slabs. Returns (h in out_dtype if `keep`,
+    the token-shifted rows if `shift` = (mix, state), decode steps only)."""
+    M, W = h.shape
+    _req(h.is_cuda and h.dtype == F32 and h.is_contiguous() and W % 8 == 0 and W <= 16384, "h fp32 [M, W]")
+    bf, S = _slabs(y, M, W, "y rows / slabs")
+    SZ = 1
+    if z is not None:
+        bz, SZ = _slabs(z, M, W, "z rows / slabs")
+        _req(bz == bf, "y and z of one type")
+        _vec(zb, W, F32, "zb")
+    _vec(w, W, F32, "w")
+    out = torch.empty((M, W), dtype=out_dtype, device=h.device) if keep else None
+    mix = state = xs = None
+    if shift is not None:
+        mix, state = shift
+        _req(meta.kind == "decode", "shifted rows of a decode step")
+        _shift_state(mix, state, meta, M, W)
+        xs = torch.empty((M, W), dtype=out_dtype, device=h.device)
+    check(_lib.lib().ragk_gated_residual(
+        h.data_ptr(), y.data_ptr(), S, ptr(z), SZ, bf, ptr(zb) if z is not None else None, w.data_ptr(), ptr(out), ptr(mix),
+        ptr(xs), ptr(state), meta.states.data_ptr() if shift is not None else None,
+        meta.kv_lens.data_ptr() if shift is not None else None, int(out_dtype == F32), M, W, n, float(eps), stream_ptr()),
+        "ragk_gated_residual")
+    return out, xs
+
+
+def token_shift(h, mix, state, meta, out_dtype, keep=True):
+    """(h in out_dtype if `keep`, h[t] + (h[t - 1] - h[t]) * mix); the state holds each sequence's last row."""
+    M, W = h.shape
+    _req(h.is_cuda and h.dtype == F32 and h.is_contiguous() and W % 8 == 0, "h fp32 [M, W]")
+    S = _shift_state(mix, state, meta, M, W)
+    _, cu = _meta(meta, M, meta.kind == "decode")
+    out = torch.empty((M, W), dtype=out_dtype, device=h.device) if keep else None
+    xs = torch.empty((M, W), dtype=out_dtype, device=h.device)
+    check(_lib.lib().ragk_token_shift(h.data_ptr(), M, W, mix.data_ptr(), state.data_ptr(), meta.states.data_ptr(), cu,
+                                      meta.kv_lens.data_ptr(), S, ptr(out), xs.data_ptr(), int(out_dtype == F32),
+                                      stream_ptr()), "ragk_token_shift")
+    return out, xs
 
 
 def residual_norm(h, y, w_post, w_next, eps, n, out_dtype):
@@ -236,6 +304,182 @@ def attn_decode(P, bias, spec, table, slots, kc, vc, meta, out, v_first=None, la
         spec.off_g if spec.gate else -1, spec.window, spec.keep_first, spec.far, int(spec.sink), DECODE_MIN_PAGES, parts,
         float(spec.scale), float(spec.softcap), stream_ptr()), "ragk_shaped_attn_decode")
     return own
+
+
+# ------------------------------------------------------------------------------------- latent attention
+KEY_PAD = 64  # zero rows behind packed key rows: attention reads whole 64-row groups
+LATENT_TARGET_BLOCKS = 256  # one block of the widest latents per CU
+LATENT_MIN_PAGES = 2
+LATENT_MAX_PARTS = 64
+
+
+@dataclass
+class KeyRows:
+    """Packed key rows of a prefill step for one window: sequence s of the first `seqs` holds positions
+    first .. kv_len - 1 in rows key_off[s] + position. `gather`: rows come from the pages (a sequence continues);
+    otherwise they are the step's own rows in order. The `tail` sequences behind them bring one token each and
+    attend like decode rows."""
+    key_off: torch.Tensor  # int32 [S]
+    cu_k: torch.Tensor  # int32 [seqs + 1]
+    tiles: torch.Tensor  # query tiles of the first `seqs` sequences
+    rows: int
+    seqs: int
+    tail: int
+    gather: bool
+
+
+def key_rows(q_lens, kv_lens, window, device):
+    ql, kl = np.asarray(q_lens, dtype=np.int64), np.asarray(kv_lens, dtype=np.int64)
+    one = (ql == 1) & (kl > 1)
+    tail = len(ql) if one.all() else int(np.argmin(one[::-1]))
+    n = len(ql) - tail
+    ctx = (kl - ql)[:n]
+    first = np.maximum(0, ctx - window + 1) // 64 * 64 if window > 0 else np.zeros_like(ctx)
+    cu = np.concatenate([[0], np.cumsum(kl[:n] - first)])
+    off = np.zeros(len(ql), dtype=np.int64)
+    off[:n] = cu[:n] - first
+    i32 = lambda x: torch.from_numpy(x.astype(np.int32)).to(device)  # noqa: E731
+    return KeyRows(i32(off), i32(cu), query_tiles(ql[:n], LatentSpec.q_tile).to(device), int(cu[-1]), n, tail,
+                   bool((ctx > 0).any()))
+
+
+def latent_heads(spec):
+    """Query heads that one decode block scores."""
+    return 32 if spec.rp <= 512 and spec.heads > 16 else 16
+
+
+def latent_parts(spec, max_kv_len, batch):
+    pages = -(-max_kv_len // 64)
+    if spec.window > 0:
+        pages = min(pages, -(-spec.window // 64) + 1)
+    rows = batch * -(-spec.heads // latent_heads(spec))
+    return max(1, min(-(-LATENT_TARGET_BLOCKS // rows), -(-pages // LATENT_MIN_PAGES), LATENT_MAX_PARTS))
+
+
+def latent_workspace(specs, max_kv_len, batch, device):
+    """(partial latents, partial statistics) of one decode step, shared by all layers."""
+    n = max(batch * s.heads * latent_parts(s, max_kv_len, batch) * s.rp for s in specs)
+    m = max(batch * s.heads * latent_parts(s, max_kv_len, batch) for s in specs)
+    f32 = dict(dtype=F32, device=device)
+    return torch.empty(n, **f32), torch.empty(2 * m, **f32)
+
+
+def _pages(pages, spec, dtype):
+    _req(pages.dim() == 3 and pages.shape[1:] == (64, spec.rp) and pages.is_contiguous() and pages.dtype == dtype,
+         "latent pages [blocks, 64, rp]")
+
+
+def latent_store(row, spec, norm, eps, slots, pages, keep=True):
+    """Normed latents of every token into the pages at `slots`; returns them as rows [T + KEY_PAD, rp] if `keep`."""
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    _req(spec.own and row.shape[1] >= spec.off_c + spec.rp and row.stride(0) % 8 == 0, "projection rows")
+    _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == T, "slots int32[T]")
+    _vec(norm, spec.rp, F32, "latent norm")
+    _pages(pages, spec, row.dtype)
+    out = torch.empty((T + KEY_PAD, spec.rp), dtype=row.dtype, device=row.device) if keep else None
+    check(_lib.lib().ragk_latent_store(row.data_ptr(), row.stride(0), spec.off_c, spec.rank, spec.rp, norm.data_ptr(),
+                                       float(eps), slots.data_ptr(), pages.data_ptr(), ptr(out), T, KEY_PAD, f32,
+                                       stream_ptr()), "ragk_latent_store")
+    return out
+
+
+def latent_gather(pages, spec, meta, kr):
+    """Packed latent rows [kr.rows + KEY_PAD, rp] of the visible tokens of a step's sequences."""
+    _pages(pages, spec, pages.dtype)
+    _req(meta.block_tables.dtype == I32 and meta.block_tables.shape[0] >= kr.seqs and kr.cu_k.numel() == kr.seqs + 1
+         and kr.key_off.numel() >= kr.seqs, "key rows")
+    out = torch.empty((kr.rows + KEY_PAD, spec.rp), dtype=pages.dtype, device=pages.device)
+    check(_lib.lib().ragk_latent_gather(pages.data_ptr(), spec.rp, meta.block_tables.data_ptr(), meta.block_tables.stride(0),
+                                        kr.cu_k.data_ptr(), kr.key_off.data_ptr(), kr.seqs, kr.rows, KEY_PAD, out.data_ptr(),
+                                        int(pages.dtype == F32), stream_ptr()), "ragk_latent_gather")
+    return out
+
+
+def row_attention(row, spec, kv, kr, meta, out):
+    """Attention of the first kr.seqs sequences' tokens over expanded key / value rows, output gates applied."""
+    f32 = _act(row, "row")
+    T = row.shape[0]
+    S, cu = _meta(meta, T, False)
+    _req(kv.dtype == row.dtype and kv.dim() == 2 and kv.is_contiguous() and kv.shape[1] == spec.kv_row
+         and kv.shape[0] >= kr.rows + KEY_PAD and kr.key_off.numel() == S, "key / value rows")
+    _req(row.shape[1] >= spec.off_c, "projection rows")
+    _req(out.dtype == row.dtype and out.shape == (T, spec.out_row) and out.is_contiguous(), "out rows")
+    if f32:
+        n = T - kr.tail
+        check(_lib.lib().ragk_row_attn_rows(
+            row.data_ptr(), row.stride(0), kv.data_ptr(), kv.stride(0), spec.off_v, kr.key_off.data_ptr(), cu,
+            meta.kv_lens.data_ptr(), out.data_ptr(), out.stride(0), n, S, spec.heads, spec.dkp, spec.dvp, spec.off_g,
+            spec.window, float(spec.scale), 1, stream_ptr()), "ragk_row_attn_rows")
+        return out
+    tiles = kr.tiles
+    _req(tiles.dtype == I32 and tiles.is_cuda and tiles.is_contiguous(), "query tiles")
+    check(_lib.lib().ragk_row_attn_prefill(
+        row.data_ptr(), row.stride(0), kv.data_ptr(), kv.stride(0), spec.off_v, kr.key_off.data_ptr(), cu,
+        meta.kv_lens.data_ptr(), tiles.data_ptr(), tiles.shape[0], out.data_ptr(), out.stride(0), spec.heads, spec.dkp,
+        spec.dvp, spec.off_g, spec.window, meta.block_tables.stride(0), float(spec.scale), stream_ptr()),
+        "ragk_row_attn_prefill")
+    return out
+
+
+def latent_decode(P, spec, wuk, wuv, pages, meta, out, slots=None, norm=None, eps=0.0, ws=None):
+    """One new token per sequence from projection slabs [S, B, N] (fp32) or rows [B, N] (bf16): queries into latent
+    space, cache append (with `slots`), attention over the latent pages, value map, output gate (bf16 caches)."""
+    rows = P.dim() == 2
+    S, (B, N) = 1 if rows else P.shape[0], P.shape[-2:]
+    ld = P.stride(0) if rows else N
+    _req(P.is_cuda and P.dtype == (BF16 if rows else F32) and P.stride(-1) == 1 and (rows or P.is_contiguous())
+         and N >= spec.off_c + (spec.rp if slots is not None else 0), "projection slabs / rows")
+    _meta(meta, B, True)
+    _pages(pages, spec, BF16)
+    _req(wuk.dtype == BF16 and wuk.is_contiguous() and wuk.shape == (spec.heads, spec.rp, spec.dkp), "wuk [H, rp, dkp]")
+    _req(wuv.dtype == BF16 and wuv.is_contiguous() and wuv.shape == (spec.heads, spec.dvp, spec.rp), "wuv [H, dvp, rp]")
+    _req(out.dtype == BF16 and out.shape[0] == B and out.shape[1] == spec.out_row and out.stride(1) == 1, "out rows")
+    if slots is not None:
+        _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == B, "slots int32[B]")
+        _vec(norm, spec.rp, F32, "latent norm")
+    ws_o, ws_ml = ws if ws is not None else (meta.ws_o, meta.ws_ml)
+    parts = latent_parts(spec, meta.max_kv, B)
+    _req(ws_o.numel() >= B * spec.heads * parts * spec.rp and ws_ml.numel() >= B * spec.heads * parts * 2,
+         "decode workspace too small")
+    qa = torch.empty((B, spec.heads, spec.rp), dtype=BF16, device=P.device)
+    L = _lib.lib()
+    check(L.ragk_latent_absorb(P.data_ptr(), int(rows), S, ld, B, spec.heads, spec.dkp, spec.rank, spec.rp,
+                               spec.off_c if slots is not None else 0, wuk.data_ptr(), qa.data_ptr(),
+                               pages.data_ptr() if slots is not None else None, ptr(slots),
+                               ptr(norm) if slots is not None else None, float(eps), stream_ptr()), "ragk_latent_absorb")
+    check(L.ragk_latent_decode(qa.data_ptr(), pages.data_ptr(), meta.block_tables.data_ptr(), meta.block_tables.stride(0),
+                               meta.kv_lens.data_ptr(), ws_o.data_ptr(), ws_ml.data_ptr(), B, spec.heads, spec.rp,
+                               spec.window, LATENT_MIN_PAGES, parts, latent_heads(spec), float(spec.scale), stream_ptr()),
+          "ragk_latent_decode")
+    check(L.ragk_latent_out(P.data_ptr(), int(rows), S, ld, spec.off_g, ws_o.data_ptr(), ws_ml.data_ptr(),
+                            meta.kv_lens.data_ptr(), wuv.data_ptr(), out.data_ptr(), out.stride(0), B, spec.heads, spec.dvp,
+                            spec.rp, spec.window, LATENT_MIN_PAGES, parts, stream_ptr()), "ragk_latent_out")
+    return out
+
+
+def latent_decode_rows(row, spec, wuk, wuv, pages, meta, out):
+    """The same from fp32 rows with plain fp32 arithmetic (exact replay); the tokens' latents are in the pages."""
+    B = row.shape[0]
+    _req(_act(row, "row") == 1 and row.shape[1] >= spec.off_c, "projection rows")
+    _meta(meta, B, True)
+    _pages(pages, spec, F32)
+    _req(wuk.dtype == F32 and wuk.is_contiguous() and wuk.shape == (spec.heads, spec.rp, spec.dkp), "wuk [H, rp, dkp]")
+    _req(wuv.dtype == F32 and wuv.is_contiguous() and wuv.shape == (spec.heads, spec.dvp, spec.rp), "wuv [H, dvp, rp]")
+    _req(out.dtype == F32 and out.shape == (B, spec.out_row) and out.stride(1) == 1, "out rows")
+    H, L = spec.heads, _lib.lib()
+    qa = torch.empty((B, H * spec.rp), dtype=F32, device=row.device)
+    oc = torch.empty_like(qa)
+    check(L.ragk_head_proj_f32(row.data_ptr(), row.stride(0), spec.dkp, wuk.data_ptr(), spec.rp, None, 0, qa.data_ptr(),
+                               qa.stride(0), B, H, stream_ptr()), "ragk_head_proj_f32")
+    check(L.ragk_shaped_attn_rows(qa.data_ptr(), qa.stride(0), pages.data_ptr(), pages.data_ptr(),
+                                  meta.block_tables.data_ptr(), meta.block_tables.stride(0), None, meta.kv_lens.data_ptr(),
+                                  None, oc.data_ptr(), oc.stride(0), B, B, H, 1, spec.rp, spec.rp, -1, spec.window, 0, 0, 0,
+                                  float(spec.scale), 0.0, 1, stream_ptr()), "ragk_shaped_attn_rows")
+    g = row[:, spec.off_g:]
+    check(L.ragk_head_proj_f32(oc.data_ptr(), oc.stride(0), spec.rp, wuv.data_ptr(), spec.dvp, g.data_ptr(), row.stride(0),
+                               out.data_ptr(), out.stride(0), B, H, stream_ptr()), "ragk_head_proj_f32")
+    return out
 
 
 # ------------------------------------------------------------------------------------- state space

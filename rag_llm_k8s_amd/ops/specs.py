@@ -133,6 +133,58 @@ class SsmSpec:
         return ceil_to(self.inner, 128)
 
 
+MAX_RANK = 1024  # widest latent row the latent-attention kernels take
+
+
+@dataclass
+class LatentSpec:
+    """Latent attention: one cached latent row of `rank` columns per token, keys and values of every head linear in
+    it, a sliding window, one sigmoid output gate per value element. `own` layers project and cache the latent;
+    others read an earlier layer's. Projection row: [q: heads x dkp | gate: heads x dvp | latent: rp if own]."""
+    heads: int
+    dim: int
+    vdim: int
+    rank: int
+    scale: float
+    window: int = 0  # 0: unlimited
+    own: bool = True
+    dkp: int = field(init=False)
+    dvp: int = field(init=False)
+    rp: int = field(init=False)
+
+    q_tile = 128  # query rows of a prefill block: one head, 4 waves of 32
+
+    def __post_init__(self):
+        self.dkp, self.dvp, self.rp = pad_head(self.dim), pad_head(self.vdim), ceil_to(self.rank, 128)
+        if self.rp > MAX_RANK:
+            raise ValueError("latent size %d exceeds %d" % (self.rank, MAX_RANK))
+
+    @property
+    def off_g(self):
+        return self.heads * self.dkp
+
+    @property
+    def off_c(self):
+        return self.off_g + self.heads * self.dvp
+
+    @property
+    def row(self):
+        return ceil_to(self.off_c + (self.rp if self.own else 0), 64)
+
+    @property
+    def off_v(self):
+        """First value column of the expanded key / value rows [k: heads x dkp | v: heads x dvp]."""
+        return self.heads * self.dkp
+
+    @property
+    def kv_row(self):
+        return self.heads * (self.dkp + self.dvp)
+
+    @property
+    def out_row(self):
+        return ceil_to(self.heads * self.dvp, 128)
+
+
 def log_bucket(n: int, rows: int, far: int) -> int:
     """Distance bucket: n itself below half = rows // 2, then half + floor(ln(n / half) / ln(far / half) *
     (rows - half)), at most rows - 1. Evaluated in exact integers, so a boundary distance lands in the

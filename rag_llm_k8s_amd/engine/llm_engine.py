@@ -19,6 +19,8 @@ Here:
 """
 from __future__ import annotations
 
+import contextlib
+import gc
 import itertools
 import logging
 import os
@@ -91,6 +93,19 @@ class Sequence:
     def token_at(self, i):
         n = len(self.prompt)
         return self.prompt[i] if i < n else self.out[i - n]
+
+
+@contextlib.contextmanager
+def no_cyclic_gc():
+    """No cyclic garbage collection inside a stream capture: it may destroy another engine's graphs and free their
+    memory, which the runtime refuses while a capture is open (an exception in a destructor ends the process)."""
+    on = gc.isenabled()
+    gc.disable()
+    try:
+        yield
+    finally:
+        if on:
+            gc.enable()
 
 
 class LLMEngine:
@@ -550,7 +565,7 @@ class LLMEngine:
         if e["graph"] is not None:
             e["graph"].replay()
         else:
-            e["run"]()
+            self._run_decode(e)
         return e["logits"][:n].float().cpu()
 
     def _feed_prefill(self, entries, got):
@@ -737,13 +752,6 @@ class LLMEngine:
         inp = StepInput(ids, pos, slots, meta, None, carry=carry, carry_src=self._tok_out)
 
         entry = dict(packed=packed, samp=samp, out=out_tok, graph=None, meta=meta, inp=inp, logits=None)
-
-        def run():
-            logits = entry["logits"] = m.forward(inp)  # kept: a replayed step's logits can be read back
-            self._sample_rows(logits, samp["temps"], samp["ks"], samp["ps"], samp["seeds"], samp["steps"],
-                              out=out_tok)
-
-        entry["run"] = run
         if self.use_graphs:
             kvl.fill_(1)  # scratch-only rows while capturing
             carry.fill_(-1)
@@ -754,17 +762,23 @@ class LLMEngine:
             s.wait_stream(torch.cuda.current_stream(dev))
             with torch.cuda.stream(s):
                 for _ in range(2):
-                    run()
+                    self._run_decode(entry)
             torch.cuda.current_stream(dev).wait_stream(s)
             g = torch.cuda.CUDAGraph()
             # captured on the warm-up stream: stream-keyed native state (the persistent decode MLP's
             # arrival counters, ops/native.py _me_workspace) was allocated by the warm-up runs above
-            with torch.cuda.graph(g, stream=s):
-                run()
+            with no_cyclic_gc(), torch.cuda.graph(g, stream=s):
+                self._run_decode(entry)
             self._tok_out.copy_(saved)
             entry["graph"] = g
         self.graphs[B] = entry
         return entry
+
+    def _run_decode(self, e):
+        """One decode step of a bucket's static buffers, eagerly or under capture."""
+        logits = e["logits"] = self.model.forward(e["inp"])  # kept: a replayed step's logits can be read back
+        p = e["samp"]
+        self._sample_rows(logits, p["temps"], p["ks"], p["ps"], p["seeds"], p["steps"], out=e["out"])
 
     def warmup_graphs(self, sizes=None):
         if not self.is_cuda:  # CPU plumbing: eager decode, nothing to capture
@@ -976,7 +990,7 @@ class LLMEngine:
                 if e["graph"] is not None:
                     e["graph"].replay()
                 else:
-                    e["run"]()
+                    self._run_decode(e)
                 if forced:
                     self._engine_fault_hook(release=True)
                 tok = e["out"][:n].cpu().tolist()

@@ -206,3 +206,24 @@ def test_peer_wait_error_record_decodes():
     assert describe_error(1 | 1 << 1 | 1 << 4 | 1 << 15).startswith("all-reduce (start barrier), block/row 0, call 1")
     assert describe_error(0) == "no error"
     assert rec < 2 ** 31  # ragk_ar_error returns it as a non-negative int
+
+
+def test_no_cyclic_gc_inside_a_capture():
+    """The guard around graph capture: no cyclic collection inside, the previous setting afterwards."""
+    import gc
+
+    from rag_llm_k8s_amd.engine.llm_engine import no_cyclic_gc
+
+    assert gc.isenabled()
+    with pytest.raises(RuntimeError):
+        with no_cyclic_gc():
+            assert not gc.isenabled()
+            raise RuntimeError
+    assert gc.isenabled()
+    gc.disable()
+    try:
+        with no_cyclic_gc():
+            pass
+        assert not gc.isenabled()
+    finally:
+        gc.enable()

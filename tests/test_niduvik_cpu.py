@@ -8,14 +8,15 @@ import sys
 import pytest
 import torch
 
-import niduvik_cases as C
 import niduvik_oracle as O
 import niduvik_util as U
+from decoder_cases import Cases
 from rag_llm_k8s_amd.engine.kv_manager import SequenceCache, StateSlots, make_block_manager
 from rag_llm_k8s_amd.models import registry
 from rag_llm_k8s_amd.models.niduvik import NiduvikConfig, niduvik_tiny, write_niduvik_checkpoint
 from rag_llm_k8s_amd.ops.specs import AttnSpec, SsmSpec, distance_table, log_bucket
 
+C = Cases(U)
 F32 = torch.float32
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 

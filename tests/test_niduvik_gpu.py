@@ -1,15 +1,16 @@
 """Niduvik on the GPU: every kernel against the plain implementation's functions, then the model-level checks
-(tests/niduvik_cases.py) in bf16 -- the serving kernels -- and in fp32."""
+(tests/decoder_cases.py) in bf16 -- the serving kernels -- and in fp32."""
 import pytest
 import torch
 
-import niduvik_cases as C
 import niduvik_oracle as O
 import niduvik_util as U
+from decoder_cases import Cases
 from rag_llm_k8s_amd.ops.backend import AttnMeta, get_backend
 from rag_llm_k8s_amd.ops.specs import AttnSpec, SsmSpec, ceil_to, distance_table
 
 pytestmark = pytest.mark.gpu
+C = Cases(U)
 DEV = "cuda"
 F32, BF16 = torch.float32, torch.bfloat16
 BOTH = [BF16, F32]

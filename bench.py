@@ -69,7 +69,7 @@ def parse():
                          "spanning every GPU (untimed; p50_latency_c1_tp_ms, the xGMI latency path); 0 = skip")
     ap.add_argument("--c1-tp-timeout", type=float, default=float(os.environ.get("RAGK_BENCH_TP_TIMEOUT", "420")),
                     help="seconds the TP=N C=1 phase may take before the headline line is printed without it")
-    ap.add_argument("--layers", default=None, choices=["niduvik"],
+    ap.add_argument("--layers", default=None, choices=["niduvik", "rolesun"],
                     help="instead of the headline: layer throughput of this model family beside Llama layers of equal "
                          "size (one GPU, random weights)")
     ap.add_argument("--json-out", default=None)
@@ -131,7 +131,7 @@ def main():
         from rag_llm_k8s_amd.utils import layer_bench
 
         _build.build_all()
-        return layer_bench.main(a.json_out)
+        return layer_bench.main(a.layers, a.json_out)
     import torch
 
     from rag_llm_k8s_amd import _build

@@ -422,40 +422,73 @@ def row_attention(row, spec, kv, kr, meta, out):
     return out
 
 
-def latent_decode(P, spec, wuk, wuv, pages, meta, out, slots=None, norm=None, eps=0.0, ws=None):
-    """One new token per sequence from projection slabs [S, B, N] (fp32) or rows [B, N] (bf16): queries into latent
-    space, cache append (with `slots`), attention over the latent pages, value map, output gate (bf16 caches)."""
+def _proj(P, spec, own):
+    """(bf16 rows?, slabs, B, leading dimension) of projection slabs [S, B, N] (fp32) or rows [B, N] (bf16)."""
     rows = P.dim() == 2
     S, (B, N) = 1 if rows else P.shape[0], P.shape[-2:]
-    ld = P.stride(0) if rows else N
     _req(P.is_cuda and P.dtype == (BF16 if rows else F32) and P.stride(-1) == 1 and (rows or P.is_contiguous())
-         and N >= spec.off_c + (spec.rp if slots is not None else 0), "projection slabs / rows")
-    _meta(meta, B, True)
-    _pages(pages, spec, BF16)
-    _req(wuk.dtype == BF16 and wuk.is_contiguous() and wuk.shape == (spec.heads, spec.rp, spec.dkp), "wuk [H, rp, dkp]")
-    _req(wuv.dtype == BF16 and wuv.is_contiguous() and wuv.shape == (spec.heads, spec.dvp, spec.rp), "wuv [H, dvp, rp]")
-    _req(out.dtype == BF16 and out.shape[0] == B and out.shape[1] == spec.out_row and out.stride(1) == 1, "out rows")
-    if slots is not None:
-        _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == B, "slots int32[B]")
-        _vec(norm, spec.rp, F32, "latent norm")
+         and N >= spec.off_c + (spec.rp if own else 0), "projection slabs / rows")
+    return int(rows), S, B, P.stride(0) if rows else N
+
+
+def _partials(spec, meta, B, ws):
     ws_o, ws_ml = ws if ws is not None else (meta.ws_o, meta.ws_ml)
     parts = latent_parts(spec, meta.max_kv, B)
-    _req(ws_o.numel() >= B * spec.heads * parts * spec.rp and ws_ml.numel() >= B * spec.heads * parts * 2,
-         "decode workspace too small")
+    _req(ws_o.dtype == F32 and ws_ml.dtype == F32 and ws_o.numel() >= B * spec.heads * parts * spec.rp
+         and ws_ml.numel() >= B * spec.heads * parts * 2, "decode workspace too small")
+    return ws_o, ws_ml, parts
+
+
+def latent_absorb(P, spec, wuk, pages=None, slots=None, norm=None, eps=0.0):
+    """Queries into latent space, qa [B, H, rp]; with `slots`, the tokens' normed latents into the pages too."""
+    own = slots is not None
+    rows, S, B, ld = _proj(P, spec, own)
+    _req(wuk.dtype == BF16 and wuk.is_contiguous() and wuk.shape == (spec.heads, spec.rp, spec.dkp), "wuk [H, rp, dkp]")
+    if own:
+        _pages(pages, spec, BF16)
+        _req(slots.dtype == I32 and slots.is_contiguous() and slots.numel() == B, "slots int32[B]")
+        _vec(norm, spec.rp, F32, "latent norm")
     qa = torch.empty((B, spec.heads, spec.rp), dtype=BF16, device=P.device)
-    L = _lib.lib()
-    check(L.ragk_latent_absorb(P.data_ptr(), int(rows), S, ld, B, spec.heads, spec.dkp, spec.rank, spec.rp,
-                               spec.off_c if slots is not None else 0, wuk.data_ptr(), qa.data_ptr(),
-                               pages.data_ptr() if slots is not None else None, ptr(slots),
-                               ptr(norm) if slots is not None else None, float(eps), stream_ptr()), "ragk_latent_absorb")
-    check(L.ragk_latent_decode(qa.data_ptr(), pages.data_ptr(), meta.block_tables.data_ptr(), meta.block_tables.stride(0),
-                               meta.kv_lens.data_ptr(), ws_o.data_ptr(), ws_ml.data_ptr(), B, spec.heads, spec.rp,
-                               spec.window, LATENT_MIN_PAGES, parts, latent_heads(spec), float(spec.scale), stream_ptr()),
-          "ragk_latent_decode")
-    check(L.ragk_latent_out(P.data_ptr(), int(rows), S, ld, spec.off_g, ws_o.data_ptr(), ws_ml.data_ptr(),
-                            meta.kv_lens.data_ptr(), wuv.data_ptr(), out.data_ptr(), out.stride(0), B, spec.heads, spec.dvp,
-                            spec.rp, spec.window, LATENT_MIN_PAGES, parts, stream_ptr()), "ragk_latent_out")
+    check(_lib.lib().ragk_latent_absorb(P.data_ptr(), rows, S, ld, B, spec.heads, spec.dkp, spec.rank, spec.rp,
+                                        spec.off_c if own else 0, wuk.data_ptr(), qa.data_ptr(), ptr(pages) if own else None,
+                                        ptr(slots), ptr(norm) if own else None, float(eps), stream_ptr()),
+          "ragk_latent_absorb")
+    return qa
+
+
+def latent_attend(qa, spec, pages, meta, ws=None):
+    """Attention of one query per sequence and head over the latent pages, left as partitions in the workspace."""
+    B = qa.shape[0]
+    _req(qa.is_cuda and qa.dtype == BF16 and qa.is_contiguous() and qa.shape == (B, spec.heads, spec.rp), "qa [B, H, rp]")
+    _meta(meta, B, True)
+    _pages(pages, spec, BF16)
+    ws_o, ws_ml, parts = _partials(spec, meta, B, ws)
+    check(_lib.lib().ragk_latent_decode(
+        qa.data_ptr(), pages.data_ptr(), meta.block_tables.data_ptr(), meta.block_tables.stride(0), meta.kv_lens.data_ptr(),
+        ws_o.data_ptr(), ws_ml.data_ptr(), B, spec.heads, spec.rp, spec.window, LATENT_MIN_PAGES, parts, latent_heads(spec),
+        float(spec.scale), stream_ptr()), "ragk_latent_decode")
+
+
+def latent_out(P, spec, wuv, meta, out, ws=None):
+    """Joined partitions through the value map, times the output gates of P, into `out` rows."""
+    rows, S, B, ld = _proj(P, spec, False)
+    _meta(meta, B, True)
+    _req(wuv.dtype == BF16 and wuv.is_contiguous() and wuv.shape == (spec.heads, spec.dvp, spec.rp), "wuv [H, dvp, rp]")
+    _req(out.dtype == BF16 and out.shape == (B, spec.out_row) and out.stride(1) == 1, "out rows")
+    ws_o, ws_ml, parts = _partials(spec, meta, B, ws)
+    check(_lib.lib().ragk_latent_out(P.data_ptr(), rows, S, ld, spec.off_g, ws_o.data_ptr(), ws_ml.data_ptr(),
+                                     meta.kv_lens.data_ptr(), wuv.data_ptr(), out.data_ptr(), out.stride(0), B, spec.heads,
+                                     spec.dvp, spec.rp, spec.window, LATENT_MIN_PAGES, parts, stream_ptr()),
+          "ragk_latent_out")
     return out
+
+
+def latent_decode(P, spec, wuk, wuv, pages, meta, out, slots=None, norm=None, eps=0.0, ws=None):
+    """One new token per sequence from projection slabs or rows: queries into latent space, cache append (with
+    `slots`), attention over the latent pages, value map, output gate (bf16 caches)."""
+    qa = latent_absorb(P, spec, wuk, pages, slots, norm, eps)
+    latent_attend(qa, spec, pages, meta, ws)
+    return latent_out(P, spec, wuv, meta, out, ws)
 
 
 def latent_decode_rows(row, spec, wuk, wuv, pages, meta, out):

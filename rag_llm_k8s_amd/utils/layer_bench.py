@@ -1,6 +1,6 @@
 """Throughput of a model family's layers at realistic sizes, beside Llama layers of equal size (random weights).
 
-    python bench.py --layers niduvik
+    python bench.py --layers niduvik | rolesun
 
 For each size: prefill tokens/s (whole steps through model.forward) and decode tokens/s (replays of the engine's
 captured decode graph), then the single kernels with the share of their roofline they reach -- the larger of
@@ -13,7 +13,7 @@ import time
 
 import torch
 
-from ..engine.llm_engine import RUNNING, LLMEngine, SamplingParams, Sequence
+from ..engine.llm_engine import RUNNING, LLMEngine, SamplingParams, Sequence, no_cyclic_gc
 from ..models import llama as L
 from ..models import niduvik as N
 from ..ops.backend import AttnMeta
@@ -63,7 +63,7 @@ def timed_graph(fn, iters):
         fn()
     torch.cuda.current_stream().wait_stream(st)
     g = torch.cuda.CUDAGraph()
-    with torch.cuda.graph(g, stream=st):
+    with no_cyclic_gc(), torch.cuda.graph(g, stream=st):
         for _ in range(iters):
             fn()
     return timed(g.replay, 4) / iters
@@ -125,7 +125,7 @@ def _meta_prefill(model, n, length, dev):
     bt = torch.arange(n * nb, dtype=torch.int32, device=dev).view(n, nb)
     tiles, qtiles = model.prefill_work(q, dev)
     return AttnMeta("prefill", torch.full((n,), length, dtype=torch.int32, device=dev), bt, cu_q=cu, tiles=tiles,
-                    qtiles=qtiles, host_kv_lens=q, host_q_lens=q, states=torch.arange(1, n + 1, dtype=torch.int32, device=dev))
+                    qtiles=qtiles, max_kv=length, key_rows=model.key_rows(q, q, dev), host_kv_lens=q, host_q_lens=q, states=torch.arange(1, n + 1, dtype=torch.int32, device=dev))
 
 
 def _meta_decode(model, batch, ctx, dev):
@@ -261,41 +261,48 @@ def kernel_rows(size, nid, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
     return rows
 
 
-def run(sizes=None, kernels=True):
+def _niduvik(s, dev):
+    cfg = niduvik_config(s)
+    return N.NiduvikModel(cfg, N.NiduvikWeights.from_state_dict(cfg, N.niduvik_state_dict(cfg, 0, device=dev), dev), dev)
+
+
+def run(family, sizes=None, kernels=True):
+    from . import layer_bench_rolesun as R
+
     dev = "cuda"
+    build, rows_of, layers = {"niduvik": (_niduvik, kernel_rows, "4 (2 attention + 2 mamba2) / 4"),
+                              "rolesun": (R.build, R.kernel_rows, "4 / 4")}[family]
     res = {}
     for size in sizes or SIZES:
         s = SIZES[size]
-        cfg = niduvik_config(s)
-        sd = N.niduvik_state_dict(cfg, 0, device=dev)
-        nid = N.NiduvikModel(cfg, N.NiduvikWeights.from_state_dict(cfg, sd, dev), dev)
-        del sd
+        mod = build(s, dev)
         lcfg = llama_config(s)
         lla = L.LlamaModel(lcfg, L.LlamaWeights.random(lcfg, dev), dev, max_positions=16384)
-        r = {"layers": "4 (2 attention + 2 mamba2) / 4", "prefill_tok_s": {}, "decode_tok_s": {}}
+        r = {"layers": layers, "prefill_tok_s": {}, "decode_tok_s": {}}
+        pair = ((family, mod), ("llama", lla))
         for n, T in ((1, 2048), (1, 8192), (16, 2048)):
             key = "%dx%d" % (n, T)
-            r["prefill_tok_s"][key] = {k: round(prefill_rate(m, n, T)) for k, m in (("niduvik", nid), ("llama", lla))}
+            r["prefill_tok_s"][key] = {k: round(prefill_rate(m, n, T)) for k, m in pair}
             print("layer bench: %s prefill %s %s" % (size, key, r["prefill_tok_s"][key]), flush=True)
         for B, ctx in ((1, 4096), (8, 4096), (32, 4096), (64, 4096)):
             key = "b%d ctx%d" % (B, ctx)
-            r["decode_tok_s"][key] = {k: round(decode_rate(m, B, ctx), 1) for k, m in (("niduvik", nid), ("llama", lla))}
+            r["decode_tok_s"][key] = {k: round(decode_rate(m, B, ctx), 1) for k, m in pair}
             print("layer bench: %s decode %s %s" % (size, key, r["decode_tok_s"][key]), flush=True)
         if kernels:
-            r["kernels"] = kernel_rows(size, nid, lla, dev)
+            r["kernels"] = rows_of(size, mod, lla, dev)
             for k in r["kernels"]:
                 print("layer bench: %s %-34s %-8s %9.1f us  %.3f of roofline" % (size, k["kernel"], k["model"], k["us"],
                                                                                k["roofline"]), flush=True)
         res[size] = r
-        del nid, lla
+        del mod, lla, pair
         torch.cuda.empty_cache()
     return res
 
 
-def main(json_out=None):
+def main(family="niduvik", json_out=None):
     t0 = time.time()
-    line = json.dumps({"layer_bench": "niduvik beside llama layers of equal size", "data": "random weights and tokens",
-                       "dtype": "bf16", "sizes": run(), "seconds": round(time.time() - t0, 1)})
+    line = json.dumps({"layer_bench": "%s beside llama layers of equal size" % family, "data": "random weights and tokens",
+                       "dtype": "bf16", "sizes": run(family), "seconds": round(time.time() - t0, 1)})
     print(line, flush=True)
     if json_out:
         with open(json_out, "w") as f:

@@ -180,20 +180,6 @@ __device__ __forceinline__ Shape make_shape(float scale, float softcap) {
   return Shape{softcap > 0.f ? 2.f * scale * LOG2E / softcap : 0.f, softcap > 0.f ? softcap * LOG2E : 0.f, scale * LOG2E};
 }
 
-// high and low bf16 parts of 8 probabilities as MFMA operands
-__device__ __forceinline__ void split_p(const f32x4& a, const f32x4& b, bf16x8& hi, bf16x8& lo) {
-  u32x4 h, l;
-#pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    h[i] = pk2bf(a[2 * i], a[2 * i + 1]);
-    h[2 + i] = pk2bf(b[2 * i], b[2 * i + 1]);
-    l[i] = pk2bf(a[2 * i] - __uint_as_float(h[i] << 16), a[2 * i + 1] - __uint_as_float(h[i] & 0xffff0000u));
-    l[2 + i] = pk2bf(b[2 * i] - __uint_as_float(h[2 + i] << 16), b[2 * i + 1] - __uint_as_float(h[2 + i] & 0xffff0000u));
-  }
-  hi = __builtin_bit_cast(bf16x8, h);
-  lo = __builtin_bit_cast(bf16x8, l);
-}
-
 struct ShapedPrefill {
   ShapedArgs a;
   const int* tiles; int n_hg, gb;  // work list (seq, first query); head groups; heads per block
@@ -257,6 +243,8 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
   const float far_bias = tb ? tb[a.far] * LOG2E : 0.f;
   const Shape shape = make_shape(a.scale, a.softcap);
   const bool capped = shape.cap2 > 0.f;
+  const bool raw = !capped && !tb && shape.c > 0.f;  // the exponential takes the products as they are, times `mul`
+  const float mul = raw ? shape.c : 1.f;
   const int win = a.window > 0 ? a.window : 0x7fffffff;
   // the polynomial in the raw product x: s = x (q0 + x^2 (q1 + ...)), good while |x| <= x_lim
   const float yx = capped ? a.scale / a.softcap : 0.f, yx2 = yx * yx, x_lim = capped ? TANH_R / yx : 0.f;
@@ -340,7 +328,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
               for (int r = 0; r < 4; ++r)
                 s[t][qt][r] = __builtin_fmaf(-2.f * shape.cap2, shape.sigma(s[t][qt][r]), base + shape.cap2);
           }
-        } else {
+        } else if (!raw) {
 #pragma unroll
           for (int t = 0; t < 4; ++t)
 #pragma unroll
@@ -403,7 +391,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][qt][r]);
-          mx = max_xor32(max_xor16(mx));
+          mx = max_xor32(max_xor16(mx)) * mul;
           alpha[qt] = 1.f;
           if (mx > m_i[qt] + RESCALE_LOG2) {
             alpha[qt] = m_i[qt] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_i[qt] - mx);
@@ -415,7 +403,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-              const float p = __builtin_amdgcn_exp2f(s[t][qt][r] - mref);
+              const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][qt][r], mul, -mref));
               s[t][qt][r] = p;
               ls += p;
             }
@@ -437,10 +425,9 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
         for (int dt = 0; dt < CV::DT; ++dt) {
           const bf16x8 vf = load_vt<DV>(sV, dt, ks, lane);
 #pragma unroll
-          for (int qt = 0; qt < 2; ++qt) {
-            o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[qt], o[dt][qt], 0, 0, 0);
-            o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[qt], o[dt][qt], 0, 0, 0);
-          }
+          for (int qt = 0; qt < 2; ++qt) o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[qt], o[dt][qt], 0, 0, 0);
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) o[dt][qt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[qt], o[dt][qt], 0, 0, 0);
         }
       }
     }

@@ -96,6 +96,20 @@ __device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
                   f2bf_s(b[0]), f2bf_s(b[1]), f2bf_s(b[2]), f2bf_s(b[3])};
 }
 
+// high and low bf16 parts of 8 probabilities as MFMA operands
+__device__ __forceinline__ void split_p(const f32x4& a, const f32x4& b, bf16x8& hi, bf16x8& lo) {
+  u32x4 h, l;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    h[i] = pk2bf(a[2 * i], a[2 * i + 1]);
+    h[2 + i] = pk2bf(b[2 * i], b[2 * i + 1]);
+    l[i] = pk2bf(a[2 * i] - __uint_as_float(h[i] << 16), a[2 * i + 1] - __uint_as_float(h[i] & 0xffff0000u));
+    l[2 + i] = pk2bf(b[2 * i] - __uint_as_float(h[2 + i] << 16), b[2 * i + 1] - __uint_as_float(h[2 + i] & 0xffff0000u));
+  }
+  hi = __builtin_bit_cast(bf16x8, h);
+  lo = __builtin_bit_cast(bf16x8, l);
+}
+
 // LDS-DMA piece as inline asm: the compiler's waitcnt pass cannot tell which LDS bytes a
 // buffer_load ... lds intrinsic writes, so it drained vmcnt(0) before the next ds_read of ANY slot
 // (an HBM round trip per fragment read). A kernel that uses this orders its slots itself (vmcnt + barrier per

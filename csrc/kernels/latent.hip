@@ -172,57 +172,102 @@ struct LatentArgs {
   int B, H, window, min_tiles, max_parts;
   float scale;
 };
-__device__ __forceinline__ int first_page(int pos, int window) { return window > 0 ? max(0, pos - window + 1) / KT : 0; }
-__device__ __forceinline__ int part_pages(int n, int min_tiles, int max_parts) {
-  return max(min_tiles, (n + max_parts - 1) / max_parts);
-}
+// A tile is TT tokens of a page; BUFS of them are in LDS, BUFS - 1 of them in flight while one is computed.
+template <int NR>
+struct LatentTile {
+  static constexpr int TT = NR <= 2 ? 64 : 32;
+  static constexpr int BYTES = TT * 256 * NR;
+  static constexpr int BUFS = NR <= 4 ? 4 : NR == 5 ? 3 : 2;
+  static constexpr int PIECES = BYTES / 1024 / 4;  // 1-KiB pieces per wave
+};
+// A query visits tiles first .. first + n - 1, `per` of them in each partition.
+struct Split {
+  int first, n, per;
+  __device__ __forceinline__ Split(int pos, int window, int tt, int min_tiles, int max_parts) {
+    first = window > 0 ? max(0, pos - window + 1) / tt : 0;
+    n = pos / tt + 1 - first;
+    per = max(min_tiles, (n + max_parts - 1) / max_parts);
+  }
+  __device__ __forceinline__ int parts() const { return (n + per - 1) / per; }
+};
 // the latent tile serves row reads (keys) and transposed reads (values): 32-B granules kept, 8 rows on distinct banks
 __device__ __forceinline__ int cswz(int row) { return 2 * (row & 7); }
 __device__ __forceinline__ void lds_barrier() {
   asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
   __builtin_amdgcn_sched_barrier(0);
 }
+template <int N>
+__device__ __forceinline__ void wait_vmcnt() {
+  static_assert(N < 64, "vmcnt has six bits");
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
 
-constexpr int P_STRIDE = 72;  // bf16 per head row of the weights in LDS (64 keys, padded)
-
-// grid: (max_parts, groups of 16 NHT heads, batch); 4 waves share each 64-token page: a wave scores 16 of its tokens for
-// all the block's heads and accumulates a quarter of the latent columns.
+// grid: (max_parts, groups of 16 NHT heads, batch). The 4 waves share every tile: each scores a part of its tokens and
+// heads, the scores meet in LDS, and each accumulates a quarter of the latent columns for all heads, with the whole
+// softmax in its own registers. Queries and latents come by LDS-DMA alone and the page list is read once, so no load
+// of the loop makes the compiler drain the DMA queue.
 template <int NR, int NHT>
 __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
-  constexpr int Rp = 128 * NR, ROWB = 2 * Rp, NC = Rp / 8, TILE = KT * ROWB, PIECES = TILE / 1024 / 4, BUFS = NR <= 4 ? 2 : 1;
+  using C = LatentTile<NR>;
+  constexpr int Rp = 128 * NR, ROWB = 2 * Rp, NC = Rp / 8, TT = C::TT, BUFS = C::BUFS, PIECES = C::PIECES;
   constexpr int KS = Rp / 32, DT = Rp / 64, NH = 16 * NHT;  // k-steps of a score; 16-column tiles per wave; heads
+  constexpr int QT = TT == 64 ? NHT : 1;                    // head tiles that one wave scores
+  constexpr int SS = TT + 4;                                // floats per head of the scores in LDS
+  static_assert(NH <= TT, "the queries pass through one tile buffer");
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  bf16_t* s_p = reinterpret_cast<bf16_t*>(smem + BUFS * TILE);   // [hi | lo][NH][P_STRIDE]
-  float* s_m = reinterpret_cast<float*>(s_p + 2 * NH * P_STRIDE);  // [4][NH]
+  float* s_s = reinterpret_cast<float*>(smem + BUFS * C::BYTES);  // [NH][SS]
+  int* s_bt = reinterpret_cast<int*>(s_s + NH * SS);              // this partition's page list
   const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int fr = lane & 15, fh = lane >> 4;
   const int part = blockIdx.x, h0 = blockIdx.y * NH, b = blockIdx.z;
-  const int pos = a.kv_lens[b] - 1, p0 = first_page(pos, a.window), np = pos / KT + 1 - p0;
-  const int pt = part_pages(np, a.min_tiles, a.max_parts), it0 = part * pt;
-  if (it0 >= np) return;  // block-uniform, before any barrier
-  const int it1 = min(it0 + pt, np);
-  const int* bt = a.block_tables + (size_t)b * a.bt_stride + p0;
+  const int pos = a.kv_lens[b] - 1;
+  const Split sp(pos, a.window, TT, a.min_tiles, a.max_parts);
+  if (part * sp.per >= sp.n) return;  // block-uniform, before any barrier
+  const int it0 = sp.first + part * sp.per, it1 = sp.first + min((part + 1) * sp.per, sp.n);
+  const int pg0 = it0 * TT / KT, npg = ((it1 - 1) * TT) / KT + 1 - pg0;
+  const int* bt = a.block_tables + (size_t)b * a.bt_stride + pg0;
+  for (int i = threadIdx.x; i < npg; i += 256) s_bt[i] = bt[i];
 
+  const unsigned lds0 = lds_addr(smem);
   int off[PIECES];
 #pragma unroll
   for (int i = 0; i < PIECES; ++i) {
     const int idx = (wid + 4 * i) * 64 + lane, row = idx / NC, ph = idx % NC;
     off[i] = row * ROWB + 16 * (ph ^ cswz(row));
   }
-  const unsigned lds0 = lds_addr(smem);
-  auto stage = [&](int it, int buf) {
-    const i32x4 srd = make_srd(a.pages + (size_t)__builtin_amdgcn_readfirstlane(bt[it]) * KT * Rp, TILE);
+  auto stage = [&](int it) {
+    const int pg = __builtin_amdgcn_readfirstlane(s_bt[it * TT / KT - pg0]), buf = (it - it0) % BUFS;
+    const i32x4 srd = make_srd(a.pages + ((size_t)pg * KT + it * TT % KT) * Rp, C::BYTES);
 #pragma unroll
-    for (int i = 0; i < PIECES; ++i) blds16_asm(srd, off[i], 0, lds0 + buf * TILE + (wid + 4 * i) * 1024);
+    for (int i = 0; i < PIECES; ++i) blds16_asm(srd, off[i], 0, lds0 + buf * C::BYTES + (wid + 4 * i) * 1024);
   };
-  stage(it0, 0);
-
-  bf16x8 qf[NHT][KS];
+  __syncthreads();  // page list
+  {                 // queries into the buffer that the first tiles leave free (heads past the last repeat it)
+    const int last = min(NH, a.H - h0) - 1;
+    const i32x4 srd = make_srd(a.qa + ((size_t)b * a.H + h0) * Rp, (last + 1) * ROWB);
 #pragma unroll
-  for (int t = 0; t < NHT; ++t) {
-    const bf16_t* q = a.qa + ((size_t)b * a.H + min(h0 + 16 * t + fr, a.H - 1)) * Rp + 8 * fh;
+    for (int i = 0; i < NH * NR / 16; ++i) {
+      const int idx = (wid + 4 * i) * 64 + lane, row = idx / NC, ph = idx % NC;
+      blds16_asm(srd, min(row, last) * ROWB + 16 * (ph ^ cswz(row)), 0, lds0 + (BUFS - 1) * C::BYTES + (wid + 4 * i) * 1024);
+    }
+  }
 #pragma unroll
-    for (int s = 0; s < KS; ++s) qf[t][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
+  for (int k = 0; k < BUFS - 1; ++k)
+    if (it0 + k < it1) stage(it0 + k);
+  if (it1 - it0 >= BUFS - 1) wait_vmcnt<(BUFS - 1) * PIECES>();
+  else wait_vmcnt0();
+  lds_barrier();
+  const int tg = TT == 64 ? wid : wid & 1, ht = TT == 64 ? 0 : wid >> 1;  // the tokens and heads this wave scores
+  const bool scores = ht < NHT;
+  bf16x8 qf[QT][KS];
+  if (scores) {
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      const int row = 16 * (ht + t) + fr;
+#pragma unroll
+      for (int s = 0; s < KS; ++s)
+        qf[t][s] = *reinterpret_cast<const bf16x8*>(smem + (BUFS - 1) * C::BYTES + row * ROWB + 16 * ((4 * s + fh) ^ cswz(row)));
+    }
   }
   f32x4 o[DT][NHT];
 #pragma unroll
@@ -237,73 +282,76 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
   }
   const float c = a.scale * LOG2E;
   const int win = a.window > 0 ? a.window : 0x7fffffff;
-  wait_vmcnt0();
-  lds_barrier();
 
   for (int it = it0; it < it1; ++it) {
-    const int buf = BUFS == 2 ? (it - it0) & 1 : 0, k0 = (p0 + it) * KT;
-    const char* tile = smem + buf * TILE;
-    if (BUFS == 2 && it + 1 < it1) stage(it + 1, buf ^ 1);
-    f32x4 s4[NHT];
+    const int k0 = it * TT;
+    const char* tile = smem + ((it - it0) % BUFS) * C::BYTES;
+    if (it1 - it > BUFS - 2) wait_vmcnt<(BUFS - 2) * PIECES>();
+    else wait_vmcnt0();
+    lds_barrier();  // the tile has landed for all waves; the buffer of the one before it and the scores are free
+    if (it + BUFS - 1 < it1) stage(it + BUFS - 1);
+    if (scores) {
+      f32x4 s4[QT][2];
 #pragma unroll
-    for (int t = 0; t < NHT; ++t) s4[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const int row = 16 * wid + fr;
+      for (int t = 0; t < QT; ++t) s4[t][0] = s4[t][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      const int row = 16 * tg + fr;
 #pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      const bf16x8 kf = *reinterpret_cast<const bf16x8*>(tile + row * ROWB + 16 * ((4 * s + fh) ^ cswz(row)));
+      for (int s = 0; s < KS; ++s) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(tile + row * ROWB + 16 * ((4 * s + fh) ^ cswz(row)));
 #pragma unroll
-      for (int t = 0; t < NHT; ++t) s4[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[t][s], s4[t], 0, 0, 0);
+        for (int t = 0; t < QT; ++t) s4[t][s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[t][s], s4[t][s & 1], 0, 0, 0);
+      }
+      const int d0 = pos - k0 - 16 * tg - 4 * fh;  // distance of this lane's first token
+      const bool edge = pos < k0 + TT - 1 || pos - k0 >= win;
+#pragma unroll
+      for (int t = 0; t < QT; ++t) {
+        f32x4 x = (s4[t][0] + s4[t][1]) * c;
+        if (edge) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) x[r] = d0 - r >= 0 && d0 - r < win ? x[r] : -INFINITY;
+        }
+        *reinterpret_cast<f32x4*>(s_s + (16 * (ht + t) + fr) * SS + 16 * tg + 4 * fh) = x;
+      }
     }
-    const int d0 = pos - k0 - 16 * wid - 4 * fh;  // distance of this lane's first token
-    const bool edge = pos < k0 + KT - 1 || pos - k0 >= win;
+    lds_barrier();
+    bf16x8 hi[TT / 32][NHT], lo[TT / 32][NHT];  // tokens 32 ks + 4 fh + 0..3 and 16 further, as the value fragments order them
+    float alpha[NHT];
 #pragma unroll
     for (int t = 0; t < NHT; ++t) {
-      float mx = -INFINITY;
+      f32x4 x[TT / 16];
+      float mx = m[t];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = d0 - r;
-        s4[t][r] = !edge || (d >= 0 && d < win) ? s4[t][r] * c : -INFINITY;
-        mx = fmaxf(mx, s4[t][r]);
+      for (int g = 0; g < TT / 16; ++g) {
+        x[g] = *reinterpret_cast<const f32x4*>(s_s + (16 * t + fr) * SS + 16 * g + 4 * fh);
+        mx = fmaxf(fmaxf(mx, fmaxf(x[g][0], x[g][1])), fmaxf(x[g][2], x[g][3]));
       }
       mx = max_xor32(max_xor16(mx));
-      if (fh == 0) s_m[wid * NH + 16 * t + fr] = mx;
-    }
-    lds_barrier();
+      const float mu = mx == -INFINITY ? 0.f : mx;
+      alpha[t] = __builtin_amdgcn_exp2f(m[t] - mu);
+      m[t] = mx;
+      float sum = 0.f;
 #pragma unroll
-    for (int t = 0; t < NHT; ++t) {
-      float mn = m[t];
+      for (int g = 0; g < TT / 16; ++g)
 #pragma unroll
-      for (int w = 0; w < 4; ++w) mn = fmaxf(mn, s_m[w * NH + 16 * t + fr]);
-      const float mu = mn == -INFINITY ? 0.f : mn, alpha = __builtin_amdgcn_exp2f(m[t] - mu);
-      m[t] = mn;
-      float p[4], sum = 0.f;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        p[r] = __builtin_amdgcn_exp2f(s4[t][r] - mu);
-        sum += p[r];
-      }
-      l[t] = l[t] * alpha + sum;
-      const unsigned a0 = pk2bf(p[0], p[1]), a1 = pk2bf(p[2], p[3]);
-      bf16_t* dst = s_p + (16 * t + fr) * P_STRIDE + 16 * wid + 4 * fh;
-      *reinterpret_cast<uint2*>(dst) = make_uint2(a0, a1);
-      *reinterpret_cast<uint2*>(dst + NH * P_STRIDE) =
-          make_uint2(pk2bf(p[0] - __uint_as_float(a0 << 16), p[1] - __uint_as_float(a0 & 0xffff0000u)),
-                     pk2bf(p[2] - __uint_as_float(a1 << 16), p[3] - __uint_as_float(a1 & 0xffff0000u)));
-#pragma unroll
-      for (int d = 0; d < DT; ++d) o[d][t] *= alpha;
-    }
-    lds_barrier();
-#pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      bf16x8 pf[2][NHT];  // tokens 32 ks + 4 fh + 0..3 and 16 further, as load_vt orders them
-#pragma unroll
-      for (int t = 0; t < NHT; ++t)
-#pragma unroll
-        for (int x = 0; x < 2; ++x) {
-          const bf16_t* src = s_p + (x * NH + 16 * t + fr) * P_STRIDE + 32 * ks + 4 * fh;
-          const bf16x4 u = *reinterpret_cast<const bf16x4*>(src), v = *reinterpret_cast<const bf16x4*>(src + 16);
-          pf[x][t] = (bf16x8){u[0], u[1], u[2], u[3], v[0], v[1], v[2], v[3]};
+        for (int r = 0; r < 4; ++r) {
+          x[g][r] = __builtin_amdgcn_exp2f(x[g][r] - mu);
+          sum += x[g][r];
         }
+      l[t] = l[t] * alpha[t] + sum;
+#pragma unroll
+      for (int ks = 0; ks < TT / 32; ++ks) split_p(x[2 * ks], x[2 * ks + 1], hi[ks][t], lo[ks][t]);
+    }
+    bool moved = false;
+#pragma unroll
+    for (int t = 0; t < NHT; ++t) moved |= alpha[t] != 1.f;
+    if (__builtin_amdgcn_ballot_w64(moved)) {
+#pragma unroll
+      for (int d = 0; d < DT; ++d)
+#pragma unroll
+        for (int t = 0; t < NHT; ++t) o[d][t] *= alpha[t];
+    }
+#pragma unroll
+    for (int ks = 0; ks < TT / 32; ++ks) {
       const int r0 = 32 * ks + 4 * fh + (fr >> 2), r1 = r0 + 16;
 #pragma unroll
       for (int d = 0; d < DT; ++d) {
@@ -312,29 +360,17 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
         const bf16x4 v = tr_read(tile + r1 * ROWB + 16 * (chunk ^ cswz(r1)) + 8 * (fr & 1));
         const bf16x8 vf = (bf16x8){u[0], u[1], u[2], u[3], v[0], v[1], v[2], v[3]};
 #pragma unroll
-        for (int t = 0; t < NHT; ++t) {
-          o[d][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[0][t], o[d][t], 0, 0, 0);
-          o[d][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[1][t], o[d][t], 0, 0, 0);
-        }
+        for (int t = 0; t < NHT; ++t) o[d][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[ks][t], o[d][t], 0, 0, 0);
+#pragma unroll
+        for (int t = 0; t < NHT; ++t) o[d][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[ks][t], o[d][t], 0, 0, 0);
       }
     }
-    if (BUFS == 1 && it + 1 < it1) {
-      lds_barrier();  // every wave has read the page
-      stage(it + 1, 0);
-    }
-    wait_vmcnt0();
-    lds_barrier();  // the next page has landed; the weights and maxima of this one are read
   }
 
 #pragma unroll
   for (int t = 0; t < NHT; ++t) {
     l[t] += __shfl_xor(l[t], 16, 64);
     l[t] += __shfl_xor(l[t], 32, 64);
-    if (fh == 0) s_m[wid * NH + 16 * t + fr] = l[t];
-  }
-  lds_barrier();
-#pragma unroll
-  for (int t = 0; t < NHT; ++t) {
     const int h = h0 + 16 * t + fr;
     if (h >= a.H) continue;
     const size_t pi = ((size_t)b * a.H + h) * a.max_parts + part;
@@ -342,11 +378,8 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
 #pragma unroll
     for (int d = 0; d < DT; ++d) *reinterpret_cast<f32x4*>(po + 16 * d) = o[d][t];
     if (wid == 0 && fh == 0) {
-      float L = 0.f;
-#pragma unroll
-      for (int w = 0; w < 4; ++w) L += s_m[w * NH + 16 * t + fr];
       a.part_ml[pi * 2] = m[t];
-      a.part_ml[pi * 2 + 1] = L;
+      a.part_ml[pi * 2 + 1] = l[t];
     }
   }
 }
@@ -362,32 +395,49 @@ struct OutArgs {
   int B, H, DV, window, min_tiles, max_parts;
 };
 
-// grid: (H * ceil(DV / 64), batch / DB): joins the partitions of one head, 64 rows of its value map, gate
-template <typename TP, int NR>
+// grid: (H * ceil(DV / 64), batch / NB): joins the partitions of one head for NB sequences, 64 rows of its value map, gate
+template <typename TP, int NR, int NB>
 __global__ __launch_bounds__(256) void latent_out_kernel(OutArgs<TP> a) {
-  constexpr int Rp = 128 * NR, KS = Rp / 32, ST = Rp + 8;
-  __shared__ __attribute__((aligned(16))) bf16_t s_c[DB * ST];
-  __shared__ float s_w[DB * MAX_PARTS];  // exp2(m_p - M) / L
+  constexpr int Rp = 128 * NR, KS = Rp / 32, ST = Rp + 8, TT = LatentTile<NR>::TT;
+  constexpr int U = NB <= 4 ? 16 : 8;  // partitions requested at a time
+  __shared__ __attribute__((aligned(16))) bf16_t s_c[NB * ST];
+  __shared__ float s_w[NB * MAX_PARTS];  // exp2(m_p - M) / L
+  __shared__ int s_n[NB];                // partitions
   const int nd = (a.DV + 63) / 64, h = blockIdx.x / nd, d0 = (blockIdx.x % nd) * 64;
-  const int b0 = blockIdx.y * DB, nb = min(DB, a.B - b0);
+  const int b0 = blockIdx.y * NB, nb = min(NB, a.B - b0);
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, fr = lane & 15, fh = lane >> 4;
   const int dr = d0 + 16 * wid;  // this wave's 16 value rows
   const bool live = dr < a.DV;   // DV is a multiple of 16
+  const int col = h * a.DV + dr + 4 * fh;
   bf16x8 wf[KS];
-  if (live) {
+  f32x4 z = {0.f, 0.f, 0.f, 0.f};
+  if (live) {  // requested before the join
 #pragma unroll
     for (int s = 0; s < KS; ++s)
       wf[s] = *reinterpret_cast<const bf16x8*>(a.wuv + ((size_t)h * a.DV + dr + fr) * Rp + 32 * s + 8 * fh);
+    if (a.off_g >= 0) {
+      const TP* g = a.P.P + (size_t)(b0 + min(fr, nb - 1)) * a.P.ld + a.off_g + col;
+      if constexpr (sizeof(TP) == 4) {
+        for (int s0 = 0; s0 < a.P.S; s0 += PSU) {
+          f32x4 u[PSU];
+#pragma unroll
+          for (int k = 0; k < PSU; ++k) u[k] = *reinterpret_cast<const f32x4*>(g + (size_t)min(s0 + k, a.P.S - 1) * a.P.slab);
+#pragma unroll
+          for (int k = 0; k < PSU; ++k)
+            if (s0 + k < a.P.S) z += u[k];
+        }
+      } else {
+        const bf16x4 zz = *reinterpret_cast<const bf16x4*>(g);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) z[r] = bf2f_s(zz[r]);
+      }
+    }
   }
   // partition weights: 16 lanes per sequence
-  {
+  if (threadIdx.x < 16 * NB) {
     const int b = threadIdx.x >> 4, q = threadIdx.x & 15;
     int n = 0;
-    if (b < nb) {
-      const int pos = a.kv_lens[b0 + b] - 1, np = pos / KT + 1 - first_page(pos, a.window);
-      const int pt = part_pages(np, a.min_tiles, a.max_parts);
-      n = (np + pt - 1) / pt;
-    }
+    if (b < nb) n = Split(a.kv_lens[b0 + b] - 1, a.window, TT, a.min_tiles, a.max_parts).parts();
     const float* ml = a.part_ml + ((size_t)(b0 + min(b, nb - 1)) * a.H + h) * a.max_parts * 2;
     float M = -INFINITY, L = 0.f;
     for (int p = q; p < n; p += 16) M = fmaxf(M, ml[2 * p]);
@@ -400,23 +450,20 @@ __global__ __launch_bounds__(256) void latent_out_kernel(OutArgs<TP> a) {
     const float inv = L > 0.f ? 1.f / L : 0.f;
     for (int p = q; p < MAX_PARTS; p += 16)
       s_w[b * MAX_PARTS + p] = p < n ? __builtin_amdgcn_exp2f(ml[2 * p] - Mu) * inv : 0.f;
+    if (q == 0) s_n[b] = n;
   }
   __syncthreads();
-  for (int i = threadIdx.x; i < DB * (Rp / 4); i += 256) {
-    const int b = i / (Rp / 4), c = (i % (Rp / 4)) * 4;
+  for (int i = threadIdx.x; i < NB * (Rp / 4); i += 256) {
+    const int b = i / (Rp / 4), c = (i % (Rp / 4)) * 4, n = s_n[b];
     f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (b < nb) {
-      const float* po = a.part_o + ((size_t)(b0 + b) * a.H + h) * a.max_parts * Rp + c;
-      const int pos = a.kv_lens[b0 + b] - 1, np = pos / KT + 1 - first_page(pos, a.window);
-      const int pt = part_pages(np, a.min_tiles, a.max_parts), n = (np + pt - 1) / pt;
-      for (int p = 0; p < n; p += 8) {
-        f32x4 u[8];
+    const float* po = a.part_o + ((size_t)(b0 + min(b, nb - 1)) * a.H + h) * a.max_parts * Rp + c;
+    for (int p = 0; p < n; p += U) {
+      f32x4 u[U];
 #pragma unroll
-        for (int k = 0; k < 8; ++k) u[k] = *reinterpret_cast<const f32x4*>(po + (size_t)min(p + k, n - 1) * Rp);
+      for (int k = 0; k < U; ++k) u[k] = *reinterpret_cast<const f32x4*>(po + (size_t)min(p + k, n - 1) * Rp);
 #pragma unroll
-        for (int k = 0; k < 8; ++k)
-          if (p + k < n) v += u[k] * s_w[b * MAX_PARTS + p + k];
-      }
+      for (int k = 0; k < U; ++k)
+        if (p + k < n) v += u[k] * s_w[b * MAX_PARTS + p + k];
     }
     *reinterpret_cast<uint2*>(s_c + b * ST + c) = make_uint2(pk2bf(v[0], v[1]), pk2bf(v[2], v[3]));
   }
@@ -424,22 +471,12 @@ __global__ __launch_bounds__(256) void latent_out_kernel(OutArgs<TP> a) {
   if (!live) return;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int s = 0; s < KS; ++s) {
-    const bf16x8 cf = *reinterpret_cast<const bf16x8*>(s_c + fr * ST + 32 * s + 8 * fh);
+  for (int s = 0; s < KS; ++s) {  // matrix columns past NB repeat and are dropped
+    const bf16x8 cf = *reinterpret_cast<const bf16x8*>(s_c + fr % NB * ST + 32 * s + 8 * fh);
     acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[s], cf, acc, 0, 0, 0);
   }
   if (fr >= nb) return;
-  const int col = h * a.DV + dr + 4 * fh;
   if (a.off_g >= 0) {
-    const TP* g = a.P.P + (size_t)(b0 + fr) * a.P.ld + a.off_g + col;
-    f32x4 z = {0.f, 0.f, 0.f, 0.f};
-    if constexpr (sizeof(TP) == 4) {
-      for (int s = 0; s < a.P.S; ++s) z += *reinterpret_cast<const f32x4*>(g + (size_t)s * a.P.slab);
-    } else {
-      const bf16x4 zz = *reinterpret_cast<const bf16x4*>(g);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) z[r] = bf2f_s(zz[r]);
-    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) acc[r] *= __builtin_amdgcn_rcpf(1.f + __expf(-z[r]));
   }
@@ -448,8 +485,9 @@ __global__ __launch_bounds__(256) void latent_out_kernel(OutArgs<TP> a) {
 
 template <int NR, int NHT>
 int launch_decode(const LatentArgs& a, hipStream_t st) {
-  constexpr int NH = 16 * NHT;
-  constexpr int lds = (NR <= 4 ? 2 : 1) * KT * 256 * NR + 2 * NH * P_STRIDE * 2 + 4 * NH * 4;
+  using C = LatentTile<NR>;
+  constexpr int NH = 16 * NHT, lds = C::BUFS * C::BYTES + NH * (C::TT + 4) * 4 + MAX_BT * 4;
+  static_assert(lds <= 160 * 1024, "LDS of a CU");
   (void)hipFuncSetAttribute((const void*)latent_decode_kernel<NR, NHT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   hipLaunchKernelGGL((latent_decode_kernel<NR, NHT>), dim3(a.max_parts, (a.H + NH - 1) / NH, a.B), dim3(256), lds, st, a);
   return (int)hipGetLastError();
@@ -473,7 +511,10 @@ int launch_absorb(const AbsorbArgs<TP>& a, int DK, hipStream_t st) {
 }
 template <int NR, typename TP>
 int launch_out(const OutArgs<TP>& a, hipStream_t st) {
-  hipLaunchKernelGGL((latent_out_kernel<TP, NR>), dim3(a.H * ((a.DV + 63) / 64), (a.B + DB - 1) / DB), dim3(256), 0, st, a);
+  const int gx = a.H * ((a.DV + 63) / 64);  // fewer sequences a block where that is what fills the chip
+  if (gx * ((a.B + 15) / 16) >= 256) hipLaunchKernelGGL((latent_out_kernel<TP, NR, 16>), dim3(gx, (a.B + 15) / 16), dim3(256), 0, st, a);
+  else if (gx * ((a.B + 7) / 8) >= 256) hipLaunchKernelGGL((latent_out_kernel<TP, NR, 8>), dim3(gx, (a.B + 7) / 8), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((latent_out_kernel<TP, NR, 4>), dim3(gx, (a.B + 3) / 4), dim3(256), 0, st, a);
   return (int)hipGetLastError();
 }
 
@@ -553,7 +594,7 @@ RAGK_API int ragk_latent_decode(const void* qa, const void* pages, const int* bl
                                 float* part_o, float* part_ml, int B, int H, int Rp, int window, int min_tiles,
                                 int max_parts, int heads, float scale, hipStream_t st) {
   if (B <= 0) return 0;
-  if (!rank_ok(1, Rp) || window < 0 || min_tiles < 1 || max_parts < 1 || max_parts > MAX_PARTS || B > 65535)
+  if (!rank_ok(1, Rp) || window < 0 || min_tiles < 1 || max_parts < 1 || max_parts > MAX_PARTS || B > 65535 || bt_stride > MAX_BT)
     return (int)hipErrorInvalidValue;
   const LatentArgs a{(const bf16_t*)qa, (const bf16_t*)pages, block_tables, bt_stride, kv_lens, part_o, part_ml, B, H,
                      window, min_tiles, max_parts, scale};

@@ -308,8 +308,8 @@ def attn_decode(P, bias, spec, table, slots, kc, vc, meta, out, v_first=None, la
 
 # ------------------------------------------------------------------------------------- latent attention
 KEY_PAD = 64  # zero rows behind packed key rows: attention reads whole 64-row groups
-LATENT_TARGET_BLOCKS = 256  # one block of the widest latents per CU
-LATENT_MIN_PAGES = 2
+LATENT_TARGET_BLOCKS = 256  # a decode block fills a CU's LDS
+LATENT_MIN_TOKENS = 128  # of a partition
 LATENT_MAX_PARTS = 64
 
 
@@ -343,17 +343,29 @@ def key_rows(q_lens, kv_lens, window, device):
                    bool((ctx > 0).any()))
 
 
-def latent_heads(spec):
-    """Query heads that one decode block scores."""
-    return 32 if spec.rp <= 512 and spec.heads > 16 else 16
+def latent_tile(spec):
+    """Tokens of one LDS tile of the decode kernel (its LatentTile)."""
+    return 64 if spec.rp <= 256 else 32
+
+
+def latent_min_tiles(spec):
+    return LATENT_MIN_TOKENS // latent_tile(spec)
+
+
+def latent_split(spec, max_kv_len, batch):
+    """(partitions per sequence, query heads per block) of a decode step."""
+    tt = latent_tile(spec)
+    tiles = -(-max_kv_len // tt)
+    if spec.window > 0:
+        tiles = min(tiles, -(-spec.window // tt) + 1)
+    most = min(-(-tiles // latent_min_tiles(spec)), LATENT_MAX_PARTS)
+    wide = spec.rp <= 512 and spec.heads > 16 and batch * -(-spec.heads // 32) * most >= LATENT_TARGET_BLOCKS
+    heads = 32 if wide else 16
+    return min(-(-LATENT_TARGET_BLOCKS // (batch * -(-spec.heads // heads))), most), heads
 
 
 def latent_parts(spec, max_kv_len, batch):
-    pages = -(-max_kv_len // 64)
-    if spec.window > 0:
-        pages = min(pages, -(-spec.window // 64) + 1)
-    rows = batch * -(-spec.heads // latent_heads(spec))
-    return max(1, min(-(-LATENT_TARGET_BLOCKS // rows), -(-pages // LATENT_MIN_PAGES), LATENT_MAX_PARTS))
+    return latent_split(spec, max_kv_len, batch)[0]
 
 
 def latent_workspace(specs, max_kv_len, batch, device):
@@ -433,10 +445,10 @@ def _proj(P, spec, own):
 
 def _partials(spec, meta, B, ws):
     ws_o, ws_ml = ws if ws is not None else (meta.ws_o, meta.ws_ml)
-    parts = latent_parts(spec, meta.max_kv, B)
+    parts, heads = latent_split(spec, meta.max_kv, B)
     _req(ws_o.dtype == F32 and ws_ml.dtype == F32 and ws_o.numel() >= B * spec.heads * parts * spec.rp
          and ws_ml.numel() >= B * spec.heads * parts * 2, "decode workspace too small")
-    return ws_o, ws_ml, parts
+    return ws_o, ws_ml, parts, heads
 
 
 def latent_absorb(P, spec, wuk, pages=None, slots=None, norm=None, eps=0.0):
@@ -462,10 +474,10 @@ def latent_attend(qa, spec, pages, meta, ws=None):
     _req(qa.is_cuda and qa.dtype == BF16 and qa.is_contiguous() and qa.shape == (B, spec.heads, spec.rp), "qa [B, H, rp]")
     _meta(meta, B, True)
     _pages(pages, spec, BF16)
-    ws_o, ws_ml, parts = _partials(spec, meta, B, ws)
+    ws_o, ws_ml, parts, heads = _partials(spec, meta, B, ws)
     check(_lib.lib().ragk_latent_decode(
         qa.data_ptr(), pages.data_ptr(), meta.block_tables.data_ptr(), meta.block_tables.stride(0), meta.kv_lens.data_ptr(),
-        ws_o.data_ptr(), ws_ml.data_ptr(), B, spec.heads, spec.rp, spec.window, LATENT_MIN_PAGES, parts, latent_heads(spec),
+        ws_o.data_ptr(), ws_ml.data_ptr(), B, spec.heads, spec.rp, spec.window, latent_min_tiles(spec), parts, heads,
         float(spec.scale), stream_ptr()), "ragk_latent_decode")
 
 
@@ -475,10 +487,10 @@ def latent_out(P, spec, wuv, meta, out, ws=None):
     _meta(meta, B, True)
     _req(wuv.dtype == BF16 and wuv.is_contiguous() and wuv.shape == (spec.heads, spec.dvp, spec.rp), "wuv [H, dvp, rp]")
     _req(out.dtype == BF16 and out.shape == (B, spec.out_row) and out.stride(1) == 1, "out rows")
-    ws_o, ws_ml, parts = _partials(spec, meta, B, ws)
+    ws_o, ws_ml, parts, _ = _partials(spec, meta, B, ws)
     check(_lib.lib().ragk_latent_out(P.data_ptr(), rows, S, ld, spec.off_g, ws_o.data_ptr(), ws_ml.data_ptr(),
                                      meta.kv_lens.data_ptr(), wuv.data_ptr(), out.data_ptr(), out.stride(0), B, spec.heads,
-                                     spec.dvp, spec.rp, spec.window, LATENT_MIN_PAGES, parts, stream_ptr()),
+                                     spec.dvp, spec.rp, spec.window, latent_min_tiles(spec), parts, stream_ptr()),
           "ragk_latent_out")
     return out
 

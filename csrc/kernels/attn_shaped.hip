@@ -186,9 +186,11 @@ struct ShapedPrefill {
   int sb_stride;                   // floats per head of the LDS bias table, 0: none
 };
 
+// PLAIN: no soft cap, bias, kept first tokens or zero score, and a positive scale: the maxima run over the raw products.
 // BOUNDED: every score is known to stay within a range whose exponentials fp32 holds (soft cap + largest bias), so
 // the sums need no running maximum: the weights are 2^s, and the extra zero score adds exactly 1.
-template <int DK, int DV, bool BOUNDED>
+enum PrefillMode { GENERAL, BOUNDED, PLAIN };
+template <int DK, int DV, PrefillMode MODE>
 __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_shaped_prefill_kernel(ShapedPrefill pa) {
   using CK = Cfg<DK>;
   using CV = Cfg<DV>;
@@ -207,7 +209,8 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
   const int q_off = a.cu_q[seq], q_len = a.cu_q[seq + 1] - q_off, kv_len = a.kv_lens[seq];
   const int ctx0 = kv_len - q_len;
   const int qt_rows = 32 * (4 / gb);
-  const Pages pg = visited(ctx0 + q_start, ctx0 + min(q_start + qt_rows, q_len) - 1, a.window, a.keep);
+  const int keep = MODE == PLAIN ? 0 : a.keep, sink = MODE == PLAIN ? 0 : a.sink;
+  const Pages pg = visited(ctx0 + q_start, ctx0 + min(q_start + qt_rows, q_len) - 1, a.window, keep);
   const int wave_pmin = ctx0 + pbase, wave_pmax = ctx0 + min(pbase + 31, q_len - 1);
   const int fr = lane & 15, fh = lane >> 4;
 
@@ -228,23 +231,21 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
   float m_i[2], l_i[2];
 #pragma unroll
   for (int qt = 0; qt < 2; ++qt) {
-    m_i[qt] = a.sink ? 0.f : -INFINITY;
-    l_i[qt] = a.sink && fh == 0 ? 1.f : 0.f;
+    m_i[qt] = sink ? 0.f : -INFINITY;
+    l_i[qt] = sink && fh == 0 ? 1.f : 0.f;
   }
   const int* bt = a.block_tables + (size_t)seq * a.bt_stride;
   for (int i = threadIdx.x; i < pg.n; i += 256) s_bt[i] = a.entry(bt, seq, pg.page(i));
-  if (a.table && pa.sb_stride)
+  if (MODE != PLAIN && a.table && pa.sb_stride)
     for (int h = 0; h < gb; ++h)
       for (int i = threadIdx.x; i <= a.far; i += 256)
         s_bias[h * pa.sb_stride + i] = a.table[(size_t)(h0 + h) * (a.far + 1) + i] * LOG2E;
   __syncthreads();
-  const float* tb = a.table ? a.table + (size_t)hq * (a.far + 1) : nullptr;
+  const float* tb = MODE != PLAIN && a.table ? a.table + (size_t)hq * (a.far + 1) : nullptr;
   const float* s_tb = s_bias + hb * pa.sb_stride;  // the same row in LDS, in log2 units
   const float far_bias = tb ? tb[a.far] * LOG2E : 0.f;
   const Shape shape = make_shape(a.scale, a.softcap);
-  const bool capped = shape.cap2 > 0.f;
-  const bool raw = !capped && !tb && shape.c > 0.f;  // the exponential takes the products as they are, times `mul`
-  const float mul = raw ? shape.c : 1.f;
+  const bool capped = MODE != PLAIN && shape.cap2 > 0.f;
   const int win = a.window > 0 ? a.window : 0x7fffffff;
   // the polynomial in the raw product x: s = x (q0 + x^2 (q1 + ...)), good while |x| <= x_lim
   const float yx = capped ? a.scale / a.softcap : 0.f, yx2 = yx * yx, x_lim = capped ? TANH_R / yx : 0.f;
@@ -265,8 +266,8 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     voff[i] = row * a.v_row * 2 + 16 * (ph ^ vswz<DV>(row));
   }
   const unsigned lds0 = lds_addr(smem);
-  auto stage = [&](int it, int buf) {
-    const int e0 = __builtin_amdgcn_readfirstlane(s_bt[it]);
+  auto stage = [&](int entry, int buf) {
+    const int e0 = __builtin_amdgcn_readfirstlane(entry);
     const i32x4 srd_k = make_srd((const bf16_t*)a.kc + e0 * a.k_unit + kvh * a.k_head, (63 * a.k_row + DK) * 2);
     const i32x4 srd_v = make_srd((const bf16_t*)a.vc + e0 * a.v_unit + kvh * a.v_head, (63 * a.v_row + DV) * 2);
     const unsigned l = lds0 + buf * (CK::TILEB + CV::TILEB);
@@ -275,7 +276,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
 #pragma unroll
     for (int i = 0; i < VP; ++i) blds16_asm(srd_v, voff[i], 0, l + CK::TILEB + (wid_u + 4 * i) * 1024);
   };
-  stage(0, 0);  // pg.n >= 1: a query always sees its own page
+  stage(s_bt[0], 0);  // pg.n >= 1: a query always sees its own page
   wait_vmcnt0();
   __syncthreads();
 
@@ -283,7 +284,8 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
     const int cur = it & 1, k0 = pg.page(it) * KT;
     const char* sK = smem + cur * (CK::TILEB + CV::TILEB);
     const char* sV = sK + CK::TILEB;
-    const bool active = k0 <= wave_pmax && (wave_pmin - (k0 + KT - 1) < win || k0 < a.keep);
+    const bool active = k0 <= wave_pmax && (wave_pmin - (k0 + KT - 1) < win || k0 < keep);
+    const int next = s_bt[min(it + 1, pg.n - 1)];
     f32x4 s[4][2];
     if (active) {
 #pragma unroll
@@ -298,9 +300,9 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
         }
       }
     }
-    if (it + 1 < pg.n) stage(it + 1, cur ^ 1);  // DMA of the next page behind the QK^T products
+    if (it + 1 < pg.n) stage(next, cur ^ 1);  // DMA of the next page behind the QK^T products
     if (active) {
-      const bool all_visible = k0 + KT - 1 <= wave_pmin && (wave_pmax - k0 < win || k0 + KT <= a.keep);
+      const bool all_visible = k0 + KT - 1 <= wave_pmin && (wave_pmax - k0 < win || k0 + KT <= keep);
       const bool far_only = !tb || wave_pmin - (k0 + KT - 1) >= a.far;  // one bias for the whole page
       // scores in log2 units, with the page-wide bias; wave-uniform branches around whole pages of elements
       const float base = far_only ? far_bias : 0.f;
@@ -328,7 +330,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
               for (int r = 0; r < 4; ++r)
                 s[t][qt][r] = __builtin_fmaf(-2.f * shape.cap2, shape.sigma(s[t][qt][r]), base + shape.cap2);
           }
-        } else if (!raw) {
+        } else if constexpr (MODE != PLAIN) {
 #pragma unroll
           for (int t = 0; t < 4; ++t)
 #pragma unroll
@@ -366,12 +368,12 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int d = d0 - 16 * t - r;
-              const bool ok = (d >= 0) & ((d < win) | (qpos - d < a.keep));
+              const bool ok = (d >= 0) & ((d < win) | (qpos - d < keep));
               s[t][qt][r] = ok ? s[t][qt][r] : -INFINITY;
             }
         }
       }
-      if constexpr (BOUNDED) {
+      if constexpr (MODE == BOUNDED) {
 #pragma unroll
         for (int qt = 0; qt < 2; ++qt)
 #pragma unroll
@@ -391,7 +393,8 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][qt][r]);
-          mx = max_xor32(max_xor16(mx)) * mul;
+          mx = max_xor32(max_xor16(mx));
+          if constexpr (MODE == PLAIN) mx *= shape.c;
           alpha[qt] = 1.f;
           if (mx > m_i[qt] + RESCALE_LOG2) {
             alpha[qt] = m_i[qt] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_i[qt] - mx);
@@ -403,7 +406,7 @@ __global__ __launch_bounds__(256, (DK <= 128 && DV <= 128) ? 2 : 1) void attn_sh
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-              const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][qt][r], mul, -mref));
+              const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][qt][r], MODE == PLAIN ? shape.c : 1.f, -mref));
               s[t][qt][r] = p;
               ls += p;
             }
@@ -742,24 +745,26 @@ __global__ void attn_shaped_merge_kernel(ShapedDecode a, int DV) {
   a.out[(size_t)b * a.ldo + h * DV + d] = f2bf(L > 0.f ? O / L * slab_gate(a, b, h) : 0.f);
 }
 
+template <int DK, int DV, PrefillMode MODE>
+int launch_prefill_mode(const ShapedPrefill& pa, int n_tiles, int lds, hipStream_t st) {
+  (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV, MODE>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                            lds);
+  hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV, MODE>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
+  return (int)hipGetLastError();
+}
 template <int DK, int DV>
 int launch_prefill(ShapedPrefill pa, int n_tiles, int bounded, hipStream_t st) {
   constexpr int base = 2 * (Cfg<DK>::TILEB + Cfg<DV>::TILEB) + MAX_BT * 4;
   constexpr int room = ((DK <= 128 && DV <= 128) ? 80 * 1024 : 160 * 1024) - base;
-  int extra = pa.a.table ? pa.gb * (pa.a.far + 1) * 4 : 0;
+  const ShapedArgs& a = pa.a;
+  int extra = a.table ? pa.gb * (a.far + 1) * 4 : 0;
   if (extra > room) extra = 0;  // a very long table is read through the caches
-  pa.sb_stride = extra ? pa.a.far + 1 : 0;
+  pa.sb_stride = extra ? a.far + 1 : 0;
   const int lds = base + (extra + 15) / 16 * 16;
-  if (bounded) {
-    (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV, true>,
-                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV, true>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
-  } else {
-    (void)hipFuncSetAttribute((const void*)attn_shaped_prefill_kernel<DK, DV, false>,
-                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    hipLaunchKernelGGL((attn_shaped_prefill_kernel<DK, DV, false>), dim3(n_tiles * pa.n_hg), dim3(256), lds, st, pa);
-  }
-  return (int)hipGetLastError();
+  if (bounded) return launch_prefill_mode<DK, DV, BOUNDED>(pa, n_tiles, lds, st);
+  if (!a.table && !a.keep && !a.sink && !(a.softcap > 0.f) && a.scale > 0.f)
+    return launch_prefill_mode<DK, DV, PLAIN>(pa, n_tiles, lds, st);
+  return launch_prefill_mode<DK, DV, GENERAL>(pa, n_tiles, lds, st);
 }
 
 template <int DK, int DV>

@@ -168,7 +168,7 @@ struct LatentArgs {
   const int* block_tables; int bt_stride;
   const int* kv_lens;
   float* part_o;       // [B][H][max_parts][Rp], not normalised
-  float* part_ml;      // [B][H][max_parts][2]: maximum (log2 units) and sum
+  float* part_ml;      // [B][H][max_parts][2]: reference of the exponentials (log2 units) and sum
   int B, H, window, min_tiles, max_parts;
   float scale;
 };
@@ -319,16 +319,19 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentArgs a) {
 #pragma unroll
     for (int t = 0; t < NHT; ++t) {
       f32x4 x[TT / 16];
-      float mx = m[t];
+      float mx = -INFINITY;
 #pragma unroll
       for (int g = 0; g < TT / 16; ++g) {
         x[g] = *reinterpret_cast<const f32x4*>(s_s + (16 * t + fr) * SS + 16 * g + 4 * fh);
         mx = fmaxf(fmaxf(mx, fmaxf(x[g][0], x[g][1])), fmaxf(x[g][2], x[g][3]));
       }
       mx = max_xor32(max_xor16(mx));
-      const float mu = mx == -INFINITY ? 0.f : mx;
-      alpha[t] = __builtin_amdgcn_exp2f(m[t] - mu);
-      m[t] = mx;
+      alpha[t] = 1.f;
+      if (mx > m[t] + RESCALE_LOG2) {
+        alpha[t] = m[t] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[t] - mx);
+        m[t] = mx;
+      }
+      const float mu = m[t] == -INFINITY ? 0.f : m[t];
       float sum = 0.f;
 #pragma unroll
       for (int g = 0; g < TT / 16; ++g)

@@ -75,16 +75,16 @@ struct GatedArgs {
   const int* slots; const int* kv_lens;
 };
 
-template <int MAXV, typename TY, typename TO>
-__global__ __launch_bounds__(256) void gated_residual_kernel(GatedArgs a) {
-  __shared__ float red[4];
+template <int NT, int MAXV, typename TY, typename TO>
+__global__ __launch_bounds__(NT) void gated_residual_kernel(GatedArgs a) {
+  __shared__ float red[NT / 64];
   const int row = blockIdx.x, nvec = a.W >> 3;
   const size_t base = (size_t)row * a.W;
   constexpr bool PRE = MAXV <= 2;  // the stream's row and the weights are requested before the reduction
   constexpr int PV = PRE ? MAXV : 1;
   float v[MAXV][8], hv[PV][8], wv[PV][8];
   auto fetch = [&](int i, int k) {
-    const int vi = min((int)threadIdx.x + i * 256, nvec - 1);
+    const int vi = min((int)threadIdx.x + i * NT, nvec - 1);
     ld8(a.h + base + vi * 8, hv[k]);
     ld8(a.w + vi * 8, wv[k]);
   };
@@ -95,17 +95,28 @@ __global__ __launch_bounds__(256) void gated_residual_kernel(GatedArgs a) {
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
-    const int vi = threadIdx.x + i * 256;
+    const int vi = threadIdx.x + i * NT;
     if (vi < nvec) {
       const TY* yp = (const TY*)a.y + base + vi * 8;
-      if constexpr (sizeof(TY) == 4) sum_slabs8(yp, a.S, a.slab, v[i]);
-      else ld8(yp, v[i]);
+      const TY* zp = (const TY*)a.z + base + vi * 8;
+      float z[8], b[8];
+      if constexpr (sizeof(TY) == 4) {  // both sets of slabs in flight together
+        f32x4 py[PSU][2], pz[PSU][2];
+        load_slabs8(yp, a.S, a.slab, py);
+        if (a.zb != nullptr) {
+          load_slabs8(zp, a.SZ, a.slab, pz);
+          ld8(a.zb + vi * 8, b);
+        }
+        add_slabs8(py, yp, a.S, a.slab, v[i]);
+        if (a.zb != nullptr) add_slabs8(pz, zp, a.SZ, a.slab, z);
+      } else {
+        ld8(yp, v[i]);
+        if (a.zb != nullptr) {
+          ld8(zp, z);
+          ld8(a.zb + vi * 8, b);
+        }
+      }
       if (a.zb != nullptr) {
-        float z[8], b[8];
-        const TY* zp = (const TY*)a.z + base + vi * 8;
-        if constexpr (sizeof(TY) == 4) sum_slabs8(zp, a.SZ, a.slab, z);
-        else ld8(zp, z);
-        ld8(a.zb + vi * 8, b);
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[i][e] /= 1.f + expf(-(z[e] + b[e]));
       }
@@ -122,7 +133,7 @@ __global__ __launch_bounds__(256) void gated_residual_kernel(GatedArgs a) {
   }
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
-    const int vi = threadIdx.x + i * 256;
+    const int vi = threadIdx.x + i * NT;
     if (vi < nvec) {
       const int k = PRE ? i : 0;
       if constexpr (!PRE) fetch(i, 0);
@@ -141,15 +152,21 @@ __global__ __launch_bounds__(256) void gated_residual_kernel(GatedArgs a) {
   }
 }
 
-template <typename TY, typename TO>
-int launch_gated(const GatedArgs& a, int M, hipStream_t st) {
-  const int per = (a.W / 8 + 255) / 256;
-  if (per <= 1) hipLaunchKernelGGL((gated_residual_kernel<1, TY, TO>), dim3(M), dim3(256), 0, st, a);
-  else if (per <= 2) hipLaunchKernelGGL((gated_residual_kernel<2, TY, TO>), dim3(M), dim3(256), 0, st, a);
-  else if (per <= 4) hipLaunchKernelGGL((gated_residual_kernel<4, TY, TO>), dim3(M), dim3(256), 0, st, a);
-  else if (per <= 8) hipLaunchKernelGGL((gated_residual_kernel<8, TY, TO>), dim3(M), dim3(256), 0, st, a);
+template <int NT, typename TY, typename TO>
+int launch_gated_nt(const GatedArgs& a, int M, hipStream_t st) {
+  const int per = (a.W / 8 + NT - 1) / NT;
+  if (per <= 1) hipLaunchKernelGGL((gated_residual_kernel<NT, 1, TY, TO>), dim3(M), dim3(NT), 0, st, a);
+  else if (per <= 2) hipLaunchKernelGGL((gated_residual_kernel<NT, 2, TY, TO>), dim3(M), dim3(NT), 0, st, a);
+  else if (per <= 4) hipLaunchKernelGGL((gated_residual_kernel<NT, 4, TY, TO>), dim3(M), dim3(NT), 0, st, a);
+  else if (per <= 8) hipLaunchKernelGGL((gated_residual_kernel<NT, 8, TY, TO>), dim3(M), dim3(NT), 0, st, a);
   else return (int)hipErrorInvalidValue;
   return (int)hipGetLastError();
+}
+template <typename TY, typename TO>
+int launch_gated(const GatedArgs& a, int M, hipStream_t st) {
+  // few rows of slabs: one vector a thread, so that a row is one round of loads
+  if (sizeof(TY) == 4 && a.W > 2048 && M <= 256) return launch_gated_nt<512, TY, TO>(a, M, st);
+  return launch_gated_nt<256, TY, TO>(a, M, st);
 }
 
 // cu null: one token per sequence. The block of a sequence's first new token reads the state and then replaces it by

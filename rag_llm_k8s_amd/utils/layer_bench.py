@@ -55,6 +55,12 @@ def timed(fn, iters, warmup=2):
     return a.elapsed_time(b) / iters * 1e-3
 
 
+def timed_turns(fns, iters, rounds=5):
+    """Median seconds per call of each function, measured in turn so that clocks and power are alike."""
+    ts = [[timed(f, iters) for f in fns] for _ in range(rounds)]
+    return [sorted(t)[rounds // 2] for t in zip(*ts)]
+
+
 def timed_graph(fn, iters):
     """Seconds per call of a decode kernel without host launch gaps: `iters` calls in one captured graph."""
     st = torch.cuda.Stream()

@@ -4,7 +4,7 @@ from __future__ import annotations
 import torch
 
 from ..models import rolesun as R
-from .layer_bench import SIZES, VOCAB, _meta_decode, _meta_prefill, _roof, rotate, timed, timed_graph
+from .layer_bench import SIZES, VOCAB, _meta_decode, _meta_prefill, _roof, rotate, timed, timed_graph, timed_turns
 
 RANK = {"2k": 256, "4k": 512}
 
@@ -46,11 +46,13 @@ def kernel_rows(size, mod, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
     out = torch.empty(M, sp.out_row, **bf)
     kv = torch.randn(M + be.q.KEY_PAD, sp.kv_row, **bf)
     fl = 4.0 * n * T * T / 2 * H * D
-    add("attention prefill", "rolesun", timed(lambda: be.q.row_attention(row, sp, kv, kr, mR, out), 8),
-        2.0 * M * 5 * H * D, fl)
     kc, vc = lla.kv_cache[0]
-    add("attention prefill", "llama", timed(lambda: be.attn_prefill(row, kc, vc, mL, out, H, G, D), 8),
-        2.0 * M * (2 * H * D + 2 * G * D), fl)
+    kc.normal_()
+    vc.normal_()
+    ta, tl = timed_turns([lambda: be.q.row_attention(row, sp, kv, kr, mR, out),
+                          lambda: be.attn_prefill(row, kc, vc, mL, out, H, G, D)], 8)
+    add("attention prefill", "rolesun", ta, 2.0 * M * 5 * H * D, fl)
+    add("attention prefill", "llama", tl, 2.0 * M * (2 * H * D + 2 * G * D), fl)
     del kv
     x = torch.randn(M, W, **bf)
 
@@ -93,7 +95,7 @@ def kernel_rows(size, mod, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
         xb, ob = torch.randn(B, W, **bf), torch.empty(B, sp.out_row, **bf)
         P = be.proj_rows(xb, mx.win)[0]
         cb, ub = 2.0 * B * ctx * rp, 2.0 * lw["uk"].numel()
-        pages = rotate(lambda: torch.zeros(nb, 64, rp, **bf), cb)
+        pages = rotate(lambda: torch.randn(nb, 64, rp, **bf), cb)
         uk, uv = rotate(lambda: lw["uk"].clone(), ub), rotate(lambda: lw["uv"].clone(), ub)
         qa = be.q.latent_absorb(P, sp, lw["uk"])
         parts = be.q.latent_parts(sp, ctx, B)
@@ -109,7 +111,7 @@ def kernel_rows(size, mod, lla, dev, prefill=(4, 4096), decode=((1, 4096), (32, 
             cb + 2 * ub, af)
         del pages, uk, uv
         kvb = 2.0 * B * ctx * G * D * 2
-        caches = rotate(lambda: (torch.zeros(nb, G, 64, D, **bf), torch.zeros(nb, G, 64, D, **bf)), kvb)
+        caches = rotate(lambda: (torch.randn(nb, G, 64, D, **bf), torch.randn(nb, G, 64, D, **bf)), kvb)
         PL = be.gemm_part(xb, LW["wqkv"])
         ol = torch.empty(B, H * D, **bf)
 
